@@ -4,7 +4,7 @@
 #include "../../include/mongoose_hip.h"
 #include "kernels.h"
 #include "prefill.h"
-#include "fused_infer.h"
+#include "context.h"
 
 #include <atomic>
 #include <cstdio>

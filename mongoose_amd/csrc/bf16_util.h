@@ -1,0 +1,29 @@
+// bf16_util.h -- bfloat16 conversions and the matrix-core vector types shared by the kernel files.
+#pragma once
+#include <hip/hip_runtime.h>
+
+namespace mg {
+
+__device__ __forceinline__ unsigned short f32_to_bf16_rne(float f) {
+    unsigned u = __builtin_bit_cast(unsigned, f);
+    u += 0x7fffu + ((u >> 16) & 1u);          // round to nearest even (inputs are finite)
+    return (unsigned short)(u >> 16);
+}
+__device__ __forceinline__ float bf16_to_f32(unsigned short h) {
+    return __builtin_bit_cast(float, (unsigned)h << 16);
+}
+// The two bf16 values of a dword.
+__device__ __forceinline__ float bf16_lo(unsigned u) { return __builtin_bit_cast(float, u << 16); }
+__device__ __forceinline__ float bf16_hi(unsigned u) { return __builtin_bit_cast(float, u & 0xffff0000u); }
+__device__ __forceinline__ unsigned bf16_pack(float lo, float hi) {
+    return f32_to_bf16_rne(lo) | ((unsigned)f32_to_bf16_rne(hi) << 16);
+}
+
+// Activations between the multi-row kernels: bf16 (stored as its 16 bits) or fp32.
+typedef unsigned short bf16_t;
+__device__ __forceinline__ void store_act(bf16_t* p, float v) { *p = f32_to_bf16_rne(v); }
+__device__ __forceinline__ void store_act(float* p, float v) { *p = v; }
+__device__ __forceinline__ float load_act(const bf16_t* p) { return bf16_to_f32(*p); }
+__device__ __forceinline__ float load_act(const float* p) { return *p; }
+
+}  // namespace mg

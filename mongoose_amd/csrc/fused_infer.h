@@ -4,7 +4,7 @@
 // runs the batch-1 decode step.  Method names follow the Go methods they
 // stand in for; the mg_* C functions are thin wrappers over them.
 #pragma once
-#include "kernels.h"
+#include "context.h"
 #include "flow.h"
 
 #include <cstdint>
@@ -21,17 +21,6 @@ struct DevMat {
     size_t bytes = 0;       // bytes a token reads from this matrix (weights + scales)
 };
 
-inline size_t alignUp256(size_t v) { return (v + 255) & ~(size_t)255; }
-
-// One device allocation handed out in 256-byte aligned pieces.
-struct Slab {
-    char* base = nullptr;
-    size_t size = 0, used = 0;
-    int init(size_t bytes);
-    void* take(size_t bytes);
-    void release();
-};
-
 struct LayerWeights {
     float* norm1 = nullptr;
     float* norm2 = nullptr;
@@ -41,15 +30,12 @@ struct LayerWeights {
     DevMat wq, wk, wv, wo, gate, up, down;
 };
 
-void set_error(const std::string& s);
-const std::string& get_error();
-
-class HIPFusedInference {
+class HIPFusedInference : public DecodeContext {
 public:
     // NewCUDAFusedInference, cuda_fused_infer.go:144-229
     static HIPFusedInference* New(int dim, int kvDim, int headDim, int nHeads, int nKVHeads, int ffnDim,
                                   int vocabSize, int nLayers, int maxSeq, double ropeTheta, float eps);
-    ~HIPFusedInference();
+    ~HIPFusedInference() override;
 
     int NumWeights() const { return nLayers * 12 + 2; }                           // :231
     int SetWeight(int idx, const float* data, size_t n);                          // :241
@@ -58,26 +44,18 @@ public:
     int SetEmbeddingF16(const uint16_t* table);
     int SetEmbeddingF32(const float* table);
     int SetLayerRange(int layerStart, int layerEnd);                              // :542
-    int ResetKV();                                                                // :530
+    int ResetKV() override;                                                        // :530
     int PartialStep(const float* hiddenIn, int pos, int layerStart, int layerEnd,
                     float* hiddenOut, float* logitsOut);                          // :392, :456, q4:92, q4:272
     int StepLayerResident(int layer, int pos, const float* hiddenIn, float* preOut,
                           float* postOut, float* logitsOut);                      // cuda_fused_infer_q4.go:451
-    int ExportHidden(float* out);                                                 // :235
-    int DecodeToken(int token, int pos, int* nextToken, float* logitsOut);
-    int Generate(const int* prompt, int nPrompt, int nDecode, int* outTokens, bool useGraph);
-    int GraphCapture();                                                           // cuda_graph.go:315
-    int GraphLaunch(int token, int pos, int* nextToken);                          // cuda_graph.go:663
-    int GraphValidate(int token, int pos, float* maxAbsDiff);                     // cuda_graph.go:554
-    int TimedDecode(int token, int pos, int steps, bool useGraph, float* elapsedMs);
-    int ProfileDecode(int token, int pos, int steps, unsigned classMask, float* classMs, int* classLaunches);
     // Batched prefill of nTokens positions starting at pos0 (Q8 weights): fills the KV caches,
     // leaves the last position's hidden state, logits and greedy token, and the device step
     // state ready for the decode that follows.
-    int Prefill(const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs);
-    int GeneratePrefill(const int* prompt, int nPrompt, int nDecode, int* outTokens);
-    uint64_t WeightBytesPerToken() const;
-    uint64_t KVBytesAt(int pos) const { return (uint64_t)2 * nLayers * (uint64_t)(pos + 1) * kvDim * (kvHalf ? 2 : 4); }
+    int Prefill(const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs) override;
+    int PrefillLogits(const int* tokens, int nTokens, int pos0, const int* want, int nWant, float* logitsOut) override;
+    uint64_t WeightBytesPerToken() const override;
+    uint64_t KVBytesAt(int pos) const override { return (uint64_t)2 * nLayers * (uint64_t)(pos + 1) * kvDim * (kvHalf ? 2 : 4); }
     // L3 bridge (cuda_fused_infer.go:118-131, :556-737): a pinned host buffer, [0:4] mailbox counter,
     // [64:] hidden state, for handing a pipeline stage's output to the host without a device sync.
     int QueueHiddenToL3();                    // :688  copy stream waits for compute, then D2H into the bridge
@@ -107,34 +85,37 @@ public:
     void releaseFlow();
 
     // shape
-    int dim, kvDim, headDim, nHeads, nKVHeads, ffnDim, vocabSize, nLayers, maxSeq;
+    int kvDim, headDim, nHeads, nKVHeads, ffnDim;
     double ropeTheta;
-    float eps;
 
     // used by the streaming front end
     // Objects that keep a pointer to this context (stream front ends) register where they keep it; the
     // destructor clears those pointers, so that destroying the context first leaves them inert.
     std::vector<HIPFusedInference**> backrefs;
-    hipStream_t stream = nullptr;
     std::vector<LayerWeights> layers;
     std::vector<float*> kCache, vCache;
-    float* hidden[2] = {nullptr, nullptr};
-    int hiddenIdx = 0;
     int enqueueLayer(const LayerWeights& L, int layer, const StepState* st, int posImm);
     int enqueueFinal(bool withArgmax);
-    float* logits = nullptr;
     float* finalNorm = nullptr;
     DevMat lmHead;
 
 private:
     HIPFusedInference() = default;
-    bool built = false;
-    int invalidateGraphs();
+    int checkReady() override;
+    void graphsInvalidated() override { flowTableDirty = true; }     // whatever invalidates the graphs may have moved a weight or a cache
+    int prepareRun() override;
+    bool hostPositions() const override { return execMode == 0; }
+    int enqueueTokenAt(int pos) override;
+    int setHostPositions(int mode) override;
+    bool captureCurrent() const override;
+    int beforeCapture() override;
+    int finishRun() override { return checkFlowError(); }
+    int prefillRows(const int* tokens, int nTokens, int pos0);
     int uploadMat(int idx, DevMat& m, int rows, int cols, const int8_t* q, const float* scales);
     int uploadMatQ4(int idx, DevMat& m, int rows, int cols, const uint8_t* raw, size_t nbytes);
     int setVec(int idx, float*& dst, const float* data, size_t n, size_t expect);
     int slotAddr(int idx, char** out);
-    Slab scratch, headSlab, prefillSlab, prefillKVSlab;
+    Slab headSlab, prefillSlab, prefillKVSlab;
     int prefillCap = 0;             // rows the prefill buffers hold
     int prefillKVCap = 0;           // cache rows the attention's split planes hold
     void* pfKVSplit = nullptr;
@@ -154,10 +135,8 @@ private:
     MvParams downParams(const LayerWeights& L) const;
     void planPrefetch(const LayerWeights& L, const LayerWeights* next, int layer, PfJob& job) const;
     EmbedRef embedRef() const;
-    int primeGraph();
-    bool fuseEmbed = false;      // set while the graphs are captured
     int enqueueLayerPerOp(const LayerWeights& L, int layer, int pos);
-    int enqueueEmbed();
+    int enqueueEmbed() override;
     // persistent layer launch (flow.hip)
 public:
     FlowGeometry flowGeo{};
@@ -179,8 +158,6 @@ public:
     bool FlowInUse() const { return flowEligible(0, nLayers); }
     long long flowLimitTicks = 5000000;       // per wait of the persistent launch: 50 ms of the 100 MHz wall clock
     void SetFlowWaitLimit(long long ticks) { invalidateGraphs(); flowLimitTicks = ticks; }
-    int statePosHost = -1;                    // the device state's position where the host knows it (set with the state, advanced
-                                              // with whole tokens run in the persistent launch), else -1
     // Whole tokens inside the persistent launch (embedding, layers, final norm, lm_head, argmax): on where the model
     // allows it; tokensPerLaunch of them in one launch where a caller asks for a run of tokens (Generate, TimedDecode,
     // GeneratePrefill), 1 = a launch (or a graph replay) per token.
@@ -204,16 +181,16 @@ private:
     bool flowTailEligible() const;
     FlowTail* dFlowTail = nullptr;
     int enqueueTokensFlow(int nTokens);
-    int decodeRun(int nTokens, bool useGraph);      // nTokens decode steps from the device state
-    bool runsInLaunch(bool useGraph) const;         // ... as runs of tokens inside the persistent launch
-    int setState(int pos, int token, int count, int nPrompt);
+    int decodeRun(int nTokens, bool useGraph) override;   // nTokens decode steps from the device state
+    bool runsInLaunch(bool useGraph) const override;      // ... as runs of tokens inside the persistent launch
+    int setState(int pos, int token, int count, int nPrompt) override;
     int flowComputeWgs(int cus) const;
     bool q4ActQuant = false;      // exec mode 0: Q4_0 matrices through the int8-activation matvecs
     void* q8Scratch = nullptr;    // (max(dim, ffnDim)/32)*40 bytes of activation blocks (cuda_fused_infer.go:175-179)
     int ensureFlow();
     int enqueueLayersFlow(int l0, int l1, const StepState* st, int posImm, bool resetFirst, int nTokens = 0);
     int checkFlowError();
-    int enqueueToken(bool withHead);      // embed -> layers -> final(+argmax) / advance, all from device state
+    int enqueueToken(bool withHead) override;      // embed -> layers -> final(+argmax) / advance, all from device state
 
     // scratch (cuda_fused_infer.go:56-69, :626)
     float *normed = nullptr, *Q = nullptr, *K = nullptr, *V = nullptr, *attnOut = nullptr, *proj = nullptr;
@@ -224,44 +201,13 @@ private:
     int smax = 1, splitLen = 256, attnHeadsPerWG = 0;
     int* attnCounters = nullptr;
     float* ropeCur = nullptr;        // cos then sin row of the device-resident position
-    RopeCur ropeRef() const;
-    // embedding table (optional)
-    int embedKind = -1;       // -1: tied lm_head
-    void* embedTable = nullptr;
-    // token-level state
-    StepState* dState = nullptr;
-    StepState* hState = nullptr;    // pinned mirror
-    int* hGate = nullptr;           // pinned flag the timing gate kernel polls
-    float* amaxVal = nullptr;
-    int* amaxIdx = nullptr;
-    int amaxParts = 0;
-    int* dHistory = nullptr;
-    int* dPrompt = nullptr;
-    int* hTokens = nullptr;         // pinned
+    RopeCur ropeRef() const override;
     bool graphsUseFlow = false;       // the whole-token graphs were captured with the persistent layer launch
-    unsigned graphGeneration = 0;     // bumped by whatever makes captured graphs stale (weights, caches, modes)
-    hipGraph_t graphFull = nullptr, graphPrompt = nullptr;
-    hipGraphExec_t execFull = nullptr, execPrompt = nullptr;
-    hipEvent_t ev0 = nullptr, ev1 = nullptr;
     // L3 bridge
     char* l3 = nullptr;               // pinned: [0:4] mailbox counter, [64:64+dim*4] hidden
     hipStream_t copyStream = nullptr;
     hipEvent_t computeDone = nullptr;
     unsigned mailboxSignaled = 0, mailboxExpected = 1;
-    // instrumented run: an event between every two launches of a token
-    std::vector<hipEvent_t> profEvents;
-    std::vector<int> profClass;       // class of the launch that follows event i
-    bool profiling = false;
-    unsigned profMask = 0xffu;
-    int profLast = -1;
-    int mark(int cls);
 };
 
 }  // namespace mg
-
-// the opaque handle of the C ABI
-struct mg_layer_graph;
-struct mg_ctx {
-    mg::HIPFusedInference* f;
-    std::vector<mg_layer_graph*> layerGraphs;      // live graph objects: they outlive the context as dead handles
-};

@@ -1,4 +1,5 @@
-// fused_infer.hip -- HIPFusedInference and the mg_* C entry points over it.
+// fused_infer.hip -- HIPFusedInference and the mg_* C entry points of its own (those of every model class are in
+// context.hip).
 // Host code only (no kernels here); compiled with hipcc for the runtime API.
 #include "fused_infer.h"
 #include <mutex>
@@ -13,25 +14,6 @@
 #include <cstring>
 
 namespace mg {
-
-static thread_local std::string g_err;
-void set_error(const std::string& s) { g_err = s; }
-const std::string& get_error() { return g_err; }
-
-#define HIPCHK(expr)                                                                      \
-    do {                                                                                  \
-        hipError_t e_ = (expr);                                                           \
-        if (e_ != hipSuccess) {                                                           \
-            set_error(std::string(#expr) + ": " + hipGetErrorString(e_));                 \
-            (void)hipGetLastError();                                                      \
-            return MG_E_HIP;                                                              \
-        }                                                                                 \
-    } while (0)
-
-#define ARGCHK(cond, msg)                                                                 \
-    do {                                                                                  \
-        if (!(cond)) { set_error(msg); return MG_E_ARG; }                                 \
-    } while (0)
 
 HIPFusedInference* HIPFusedInference::New(int dim, int kvDim, int headDim, int nHeads, int nKVHeads, int ffnDim,
                                           int vocabSize, int nLayers, int maxSeq, double ropeTheta, float eps) {
@@ -84,8 +66,6 @@ HIPFusedInference* HIPFusedInference::New(int dim, int kvDim, int headDim, int n
         delete f;
         return nullptr;
     };
-    if (hipStreamCreateWithFlags(&f->stream, hipStreamNonBlocking) != hipSuccess) return fail("stream create failed");
-    if (hipEventCreate(&f->ev0) != hipSuccess || hipEventCreate(&f->ev1) != hipSuccess) return fail("event create failed");
     // L3 bridge: 64-byte mailbox line + the hidden state, pinned (cuda_fused_infer.go:204-217)
     if (hipHostMalloc(reinterpret_cast<void**>(&f->l3), 64 + (size_t)dim * 4, hipHostMallocDefault) != hipSuccess)
         return fail("L3 bridge allocation failed");
@@ -107,28 +87,21 @@ HIPFusedInference* HIPFusedInference::New(int dim, int kvDim, int headDim, int n
     // positions of the 0.5B and 1.1B shapes, no difference at Llama-3-8B's), the whole group beyond,
     // where every extra pass over the rows is HBM traffic
     f->attnHeadsPerWG = maxSeq <= 1024 ? 1 : (maxSeq <= 8192 ? 2 : 0);
-    f->amaxParts = 4096;
     {
-        size_t floats = (size_t)7 * dim + 2 * (size_t)kvDim + 3 * (size_t)ffnDim + vocabSize +
-                        2 * (size_t)maxSeq * half0 + (size_t)nHeads * f->smax * (headDim + 2) + headDim + f->amaxParts;
-        size_t ints = (size_t)f->amaxParts + 2 * ((size_t)maxSeq + 1) + 64 + attention_columns(nHeads, nKVHeads, 1);
-        size_t bytes = (floats + ints) * 4 + 64 * 256;
-        if (f->scratch.init(bytes) != 0) return fail("scratch alloc failed");
-        if (hipMemsetAsync(f->scratch.base, 0, bytes, f->stream) != hipSuccess || hipStreamSynchronize(f->stream) != hipSuccess)
-            return fail("scratch clear failed");
+        size_t floats = (size_t)5 * dim + 2 * (size_t)kvDim + 3 * (size_t)ffnDim +
+                        2 * (size_t)maxSeq * half0 + (size_t)nHeads * f->smax * (headDim + 2) + headDim;
+        size_t bytes = (floats + attention_columns(nHeads, nKVHeads, 1)) * 4 + 64 * 256;
+        if (f->initTokenState(bytes) != 0) return fail("scratch alloc failed");
     }
     auto takeF = [&](float*& p, size_t n) { p = static_cast<float*>(f->scratch.take(n * 4)); return p != nullptr; };
     auto takeI = [&](int*& p, size_t n) { p = static_cast<int*>(f->scratch.take(n * 4)); return p != nullptr; };
-    bool ok = takeF(f->hidden[0], dim) && takeF(f->hidden[1], dim) && takeF(f->logits, vocabSize) && takeF(f->normed, dim) &&
+    bool ok = takeF(f->normed, dim) &&
               takeF(f->Q, dim) && takeF(f->K, kvDim) && takeF(f->V, kvDim) && takeF(f->attnOut, dim) && takeF(f->proj, dim) &&
               takeF(f->normed2, dim) && takeF(f->gatePre, ffnDim) && takeF(f->upOut, ffnDim) && takeF(f->ffnMid, ffnDim) &&
               takeF(f->cosTab, (size_t)maxSeq * half0) && takeF(f->sinTab, (size_t)maxSeq * half0) &&
               takeF(f->pm, (size_t)nHeads * f->smax) && takeF(f->pl, (size_t)nHeads * f->smax) &&
               takeF(f->pacc, (size_t)nHeads * f->smax * headDim) && takeF(f->ropeCur, headDim) &&
-              takeF(f->amaxVal, f->amaxParts) && takeI(f->amaxIdx, f->amaxParts) &&
-              takeI(f->attnCounters, attention_columns(nHeads, nKVHeads, 1)) &&
-              takeI(f->dHistory, (size_t)maxSeq + 1) && takeI(f->dPrompt, (size_t)maxSeq + 1);
-    if (ok) { f->dState = static_cast<StepState*>(f->scratch.take(sizeof(StepState))); ok = f->dState != nullptr; }
+              takeI(f->attnCounters, attention_columns(nHeads, nKVHeads, 1));
     if (!ok) return fail("scratch slab too small");
 
     // RoPE tables, cuda_fused_infer.go:181-192: angle in double, stored as float.
@@ -146,35 +119,8 @@ HIPFusedInference* HIPFusedInference::New(int dim, int kvDim, int headDim, int n
     if (hipMemcpy(f->cosTab, cosD.data(), cosD.size() * 4, hipMemcpyHostToDevice) != hipSuccess ||
         hipMemcpy(f->sinTab, sinD.data(), sinD.size() * 4, hipMemcpyHostToDevice) != hipSuccess) return fail("rope upload");
 
-    void* hp = nullptr;
-    if (hipHostMalloc(&hp, sizeof(StepState), hipHostMallocDefault) != hipSuccess) return fail("pinned alloc");
-    f->hState = static_cast<StepState*>(hp);
-    if (hipHostMalloc(&hp, 64, hipHostMallocCoherent | hipHostMallocMapped) != hipSuccess) return fail("pinned alloc");
-    f->hGate = static_cast<int*>(hp);
-    *f->hGate = 1;
-    if (hipHostMalloc(&hp, sizeof(int) * ((size_t)maxSeq + 1), hipHostMallocDefault) != hipSuccess) return fail("pinned alloc");
-    f->hTokens = static_cast<int*>(hp);
-
     f->built = true;
     return f;
-}
-
-int Slab::init(size_t bytes) {
-    release();
-    void* v = nullptr;
-    HIPCHK(hipMalloc(&v, bytes ? bytes : 256));
-    base = static_cast<char*>(v); size = bytes; used = 0;
-    return MG_OK;
-}
-void* Slab::take(size_t bytes) {
-    size_t off = alignUp256(used);
-    if (!base || off + bytes > size) return nullptr;
-    used = off + bytes;
-    return base + off;
-}
-void Slab::release() {
-    if (base) (void)hipFree(base);
-    base = nullptr; size = used = 0;
 }
 
 // Device address of a weight slot (allocating the layer's / head's slab on first use).
@@ -197,40 +143,20 @@ HIPFusedInference::~HIPFusedInference() {
     releaseFlow();
     for (HIPFusedInference** ref : backrefs) *ref = nullptr;
     if (stream) (void)hipStreamSynchronize(stream);
-    invalidateGraphs();
-    scratch.release();
     headSlab.release();
     prefillSlab.release();
     prefillKVSlab.release();
     for (auto& sl : layerSlabs) sl.release();
     for (auto& sl : kvSlabs) sl.release();
-    if (embedTable) (void)hipFree(embedTable);
     if (q8Scratch) (void)hipFree(q8Scratch);
     if (dFlowLayers) (void)hipFree(dFlowLayers);
     if (flowXchg) (void)hipFree(flowXchg);
     if (dFlowTail) (void)hipFree(dFlowTail);
     if (dFlowErr) (void)hipFree(dFlowErr);
     if (hFlowErr) (void)hipHostFree(hFlowErr);
-    if (hState) (void)hipHostFree(hState);
-    if (hGate) (void)hipHostFree(hGate);
-    if (hTokens) (void)hipHostFree(hTokens);
-    for (hipEvent_t e : profEvents) (void)hipEventDestroy(e);
     if (copyStream) { (void)hipStreamSynchronize(copyStream); (void)hipStreamDestroy(copyStream); }
     if (computeDone) (void)hipEventDestroy(computeDone);
     if (l3) (void)hipHostFree(l3);
-    if (ev0) (void)hipEventDestroy(ev0);
-    if (ev1) (void)hipEventDestroy(ev1);
-    if (stream) (void)hipStreamDestroy(stream);
-}
-
-int HIPFusedInference::invalidateGraphs() {
-    graphGeneration++;
-    flowTableDirty = true;          // whatever invalidates the graphs may have moved a weight or a cache
-    if (execFull) { (void)hipGraphExecDestroy(execFull); execFull = nullptr; }
-    if (execPrompt) { (void)hipGraphExecDestroy(execPrompt); execPrompt = nullptr; }
-    if (graphFull) { (void)hipGraphDestroy(graphFull); graphFull = nullptr; }
-    if (graphPrompt) { (void)hipGraphDestroy(graphPrompt); graphPrompt = nullptr; }
-    return MG_OK;
 }
 
 // Slot map, cuda_fused_infer.go:241-272.
@@ -425,24 +351,6 @@ uint64_t HIPFusedInference::WeightBytesPerToken() const {
     b += lmHead.bytes;
     if (finalNorm) b += (uint64_t)dim * 4;
     return b;
-}
-
-// While the instrumented graph is being captured: an event before the launch
-// of class `cls` (the previous launch's end).  No-op otherwise.
-int HIPFusedInference::mark(int cls) {
-    if (!profiling) return MG_OK;
-    // an event opens the interval of a wanted class and closes the interval of the one before it
-    const bool opens = cls >= 0 && cls < 8 && ((profMask >> cls) & 1);
-    const bool closes = profLast >= 0 && profLast < 8 && ((profMask >> profLast) & 1);
-    profLast = cls;
-    if (!opens && !closes) return MG_OK;
-    if (!opens) cls = 8;                      // interval that follows is not measured
-    hipEvent_t e = nullptr;
-    HIPCHK(hipEventCreate(&e));
-    profEvents.push_back(e);
-    profClass.push_back(cls);
-    HIPCHK(hipEventRecord(e, stream));
-    return MG_OK;
 }
 
 RopeCur HIPFusedInference::ropeRef() const {
@@ -923,8 +831,8 @@ int HIPFusedInference::SetTokensPerLaunch(int n) {
 // Sets the device-resident step state; where the persistent launch runs whole tokens, also leaves its exchange area
 // reset (a token expects the half of its position's parity so, and resets the other for its successor).
 int HIPFusedInference::setState(int pos, int token, int count, int nPrompt) {
-    HIPCHK(launch_set_state(dState, pos, token, count, nPrompt, ropeRef(), stream));
-    statePosHost = pos;
+    int rc = DecodeContext::setState(pos, token, count, nPrompt);
+    if (rc) return rc;
     if (flowXchg && (execMode == 3 || execMode == 4)) HIPCHK(launch_flow_reset_all(flowXchg, flowGeo, nLayers, flowGrid, stream));
     return MG_OK;
 }
@@ -943,12 +851,30 @@ int HIPFusedInference::decodeRun(int nTokens, bool useGraph) {
         }
         return rc;
     }
-    for (int i = 0; i < nTokens; i++) {
-        statePosHost = -1;                          // (advanced on the device by launches that do not tell the host)
-        if (useGraph) HIPCHK(hipGraphLaunch(execFull, stream));
-        else { int rc = enqueueToken(true); if (rc) return rc; }
-    }
-    return MG_OK;
+    return DecodeContext::decodeRun(nTokens, useGraph);
+}
+
+int HIPFusedInference::prepareRun() { return runsInLaunch(true) ? ensureFlow() : MG_OK; }
+
+int HIPFusedInference::enqueueTokenAt(int pos) {
+    int rc = enqueueEmbed();
+    for (int l = 0; l < nLayers && rc == MG_OK; l++) rc = enqueueLayerPerOp(layers[l], l, pos);
+    return rc ? rc : enqueueFinal(true);
+}
+
+int HIPFusedInference::setHostPositions(int mode) {
+    const int saved = execMode;
+    if (mode >= 0) execMode = mode;
+    else if (execMode == 0) execMode = 1;
+    return saved;
+}
+
+// (the persistent launch may have changed hands since the capture)
+bool HIPFusedInference::captureCurrent() const { return graphsUseFlow == flowEligible(0, nLayers); }
+
+int HIPFusedInference::beforeCapture() {
+    graphsUseFlow = flowEligible(0, nLayers);
+    return graphsUseFlow ? ensureFlow() : MG_OK;
 }
 
 // After a synchronisation: did a wait of the persistent launch give up?  (Its workgroups were then not all
@@ -1149,14 +1075,6 @@ int HIPFusedInference::StepLayerResident(int layer, int pos, const float* hidden
     return MG_OK;
 }
 
-int HIPFusedInference::ExportHidden(float* out) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(out, "ExportHidden: NULL out");
-    HIPCHK(hipStreamSynchronize(stream));
-    HIPCHK(hipMemcpy(out, hidden[hiddenIdx], (size_t)dim * 4, hipMemcpyDeviceToHost));
-    return checkFlowError();
-}
-
 int HIPFusedInference::enqueueEmbed() {
     float* h = hidden[hiddenIdx];
     if (mark(0)) return MG_E_HIP;
@@ -1184,11 +1102,6 @@ EmbedRef HIPFusedInference::embedRef() const {
     e.out = hidden[hiddenIdx]; e.dim = dim; e.vocab = vocabSize;
     return e;
 }
-int HIPFusedInference::primeGraph() {
-    // (a captured token leaves the exchange area reset for its successor; the first one finds it so from setState)
-    return enqueueEmbed();
-}
-
 int HIPFusedInference::enqueueToken(bool withHead) {
     if (withHead && flowTailEligible()) {          // the whole token is one launch
         int rc = ensureFlow();
@@ -1216,64 +1129,12 @@ int HIPFusedInference::enqueueToken(bool withHead) {
     return MG_OK;
 }
 
-static int checkReady(HIPFusedInference* f) {
-    for (int l = 0; l < f->nLayers; l++) {
-        if (!layerComplete(f->layers[l])) { set_error("decode: layer weights incomplete"); return MG_E_STATE; }
-        if (!f->kCache[l]) { set_error("decode: KV cache missing, call SetLayerRange(0, nLayers)"); return MG_E_STATE; }
+int HIPFusedInference::checkReady() {
+    for (int l = 0; l < nLayers; l++) {
+        if (!layerComplete(layers[l])) { set_error("decode: layer weights incomplete"); return MG_E_STATE; }
+        if (!kCache[l]) { set_error("decode: KV cache missing, call SetLayerRange(0, nLayers)"); return MG_E_STATE; }
     }
-    if (!f->finalNorm || !f->lmHead.w) { set_error("decode: final norm / lm_head not set"); return MG_E_STATE; }
-    return MG_OK;
-}
-
-int HIPFusedInference::DecodeToken(int token, int pos, int* nextToken, float* logitsOut) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(pos >= 0 && pos < maxSeq && token >= 0 && token < vocabSize, "DecodeToken: token or pos out of range");
-    int rc = checkReady(this);
-    if (rc) return rc;
-    { int rcs = setState(pos, token, 0, 0); if (rcs) return rcs; }
-    if (execMode == 0) {
-        rc = enqueueEmbed();
-        if (rc) return rc;
-        for (int l = 0; l < nLayers; l++) {
-            rc = enqueueLayerPerOp(layers[l], l, pos);
-            if (rc) return rc;
-        }
-        rc = enqueueFinal(true);
-    } else {
-        rc = enqueueToken(true);
-    }
-    if (rc) return rc;
-    HIPCHK(hipMemcpyAsync(hTokens, dHistory, sizeof(int), hipMemcpyDeviceToHost, stream));
-    HIPCHK(hipStreamSynchronize(stream));
-    if (nextToken) *nextToken = hTokens[0];
-    if (logitsOut) HIPCHK(hipMemcpy(logitsOut, logits, (size_t)vocabSize * 4, hipMemcpyDeviceToHost));
-    return checkFlowError();
-}
-
-int HIPFusedInference::GraphCapture() {
-    if (!built) return MG_E_NOT_BUILT;
-    int rc = checkReady(this);
-    if (rc) return rc;
-    const bool flow = flowEligible(0, nLayers);
-    if (execFull && execPrompt && graphsUseFlow == flow) return MG_OK;     // (the launch may have changed hands since the capture)
-    invalidateGraphs();
-    graphsUseFlow = flow;
-    if (flow) { rc = ensureFlow(); if (rc) return rc; }     // allocations and uploads come before the capture
-    HIPCHK(hipStreamSynchronize(stream));
-    statePosHost = -1;                              // a captured launch is replayed at any position: the variant that covers all
-    for (int which = 0; which < 2; which++) {
-        HIPCHK(hipStreamBeginCapture(stream, hipStreamCaptureModeRelaxed));
-        fuseEmbed = true;
-        rc = enqueueToken(which == 0);
-        fuseEmbed = false;
-        hipGraph_t g = nullptr;
-        hipError_t e = hipStreamEndCapture(stream, &g);
-        if (rc) { if (g) (void)hipGraphDestroy(g); return rc; }
-        HIPCHK(e);
-        hipGraphExec_t ex = nullptr;
-        HIPCHK(hipGraphInstantiate(&ex, g, nullptr, nullptr, 0));
-        if (which == 0) { graphFull = g; execFull = ex; } else { graphPrompt = g; execPrompt = ex; }
-    }
+    if (!finalNorm || !lmHead.w) { set_error("decode: final norm / lm_head not set"); return MG_E_STATE; }
     return MG_OK;
 }
 
@@ -1364,151 +1225,6 @@ int HIPFusedInference::ValidateGraphCapture(const float* hiddenIn, int layerStar
     return MG_OK;
 }
 
-int HIPFusedInference::GraphLaunch(int token, int pos, int* nextToken) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(pos >= 0 && pos < maxSeq && token >= 0 && token < vocabSize, "GraphLaunch: token or pos out of range");
-    int rc = GraphCapture();
-    if (rc) return rc;
-    { int rcs = setState(pos, token, 0, 0); if (rcs) return rcs; }
-    rc = primeGraph();
-    if (rc) return rc;
-    statePosHost = -1;
-    HIPCHK(hipGraphLaunch(execFull, stream));
-    HIPCHK(hipMemcpyAsync(hTokens, dHistory, sizeof(int), hipMemcpyDeviceToHost, stream));
-    HIPCHK(hipStreamSynchronize(stream));
-    if (nextToken) *nextToken = hTokens[0];
-    return checkFlowError();
-}
-
-int HIPFusedInference::GraphValidate(int token, int pos, float* maxAbsDiff) {
-    if (!built) return MG_E_NOT_BUILT;
-    std::vector<float> a(vocabSize), b(vocabSize);
-    int t0 = -1, t1 = -1;
-    int saved = execMode;
-    if (execMode == 0) execMode = 1;         // the per-op launches are not captured: compare the graph with the fused launches
-    int rc = DecodeToken(token, pos, &t0, a.data());
-    execMode = saved;
-    if (rc) return rc;
-    rc = GraphLaunch(token, pos, &t1);
-    if (rc) return rc;
-    HIPCHK(hipMemcpy(b.data(), logits, (size_t)vocabSize * 4, hipMemcpyDeviceToHost));
-    float md = 0.f;
-    for (int i = 0; i < vocabSize; i++) md = std::fmax(md, std::fabs(a[i] - b[i]));
-    if (t0 != t1) md = std::fmax(md, 1.0f);
-    if (maxAbsDiff) *maxAbsDiff = md;
-    return MG_OK;
-}
-
-int HIPFusedInference::Generate(const int* prompt, int nPrompt, int nDecode, int* outTokens, bool useGraph) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(prompt && nPrompt >= 1 && nDecode >= 0 && outTokens, "Generate: bad arguments");
-    ARGCHK(nPrompt + nDecode <= maxSeq + 1 && nPrompt <= maxSeq, "Generate: prompt + decode exceeds maxSeq");
-    for (int i = 0; i < nPrompt; i++) ARGCHK(prompt[i] >= 0 && prompt[i] < vocabSize, "Generate: prompt token out of range");
-    int rc = checkReady(this);
-    if (rc) return rc;
-    if (execMode == 0) {
-        // per-op mode: host-driven loop, one synchronisation per token
-        int tok = prompt[0];
-        for (int pos = 0; pos < nPrompt - 1 + nDecode; pos++) {
-            int next = -1;
-            rc = DecodeToken(tok, pos, &next, nullptr);
-            if (rc) return rc;
-            if (pos + 1 < nPrompt) tok = prompt[pos + 1];
-            else { outTokens[pos + 1 - nPrompt] = next; tok = next; }
-        }
-        return MG_OK;
-    }
-    // (where runs of tokens go into one launch no graph is needed: the prompt steps are launched one by one)
-    const bool graphs = useGraph && !runsInLaunch(useGraph);
-    if (graphs) { rc = GraphCapture(); if (rc) return rc; }
-    HIPCHK(hipStreamSynchronize(stream));
-    HIPCHK(hipMemcpy(dPrompt, prompt, sizeof(int) * (size_t)nPrompt, hipMemcpyHostToDevice));
-    { int rcs = setState(0, prompt[0], 0, nPrompt); if (rcs) return rcs; }
-    if (graphs) { rc = primeGraph(); if (rc) return rc; }
-    for (int i = 0; i < nPrompt - 1; i++) {
-        if (graphs) HIPCHK(hipGraphLaunch(execPrompt, stream));
-        else { rc = enqueueToken(false); if (rc) return rc; }
-    }
-    statePosHost = nPrompt - 1;                     // one position a prompt step since setState(0, ..)
-    rc = decodeRun(nDecode, useGraph);
-    if (rc) return rc;
-    if (nDecode > 0) HIPCHK(hipMemcpyAsync(hTokens, dHistory, sizeof(int) * (size_t)nDecode, hipMemcpyDeviceToHost, stream));
-    HIPCHK(hipStreamSynchronize(stream));
-    for (int i = 0; i < nDecode; i++) outTokens[i] = hTokens[i];
-    return checkFlowError();
-}
-
-int HIPFusedInference::TimedDecode(int token, int pos, int steps, bool useGraph, float* elapsedMs) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(steps >= 1 && pos >= 0 && pos + steps <= maxSeq && token >= 0 && token < vocabSize, "TimedDecode: bad arguments");
-    int rc = checkReady(this);
-    if (rc) return rc;
-    const bool graphs = useGraph && !runsInLaunch(useGraph);
-    if (graphs) { rc = GraphCapture(); if (rc) return rc; }
-    if (runsInLaunch(useGraph)) { rc = ensureFlow(); if (rc) return rc; }      // (allocations before the timed region)
-    { int rcs = setState(pos, token, 0, 0); if (rcs) return rcs; }
-    if (graphs) { rc = primeGraph(); if (rc) return rc; }
-    HIPCHK(hipStreamSynchronize(stream));
-    HIPCHK(hipEventRecord(ev0, stream));
-    rc = decodeRun(steps, useGraph);
-    if (rc) return rc;
-    HIPCHK(hipEventRecord(ev1, stream));
-    HIPCHK(hipEventSynchronize(ev1));
-    float ms = 0.f;
-    HIPCHK(hipEventElapsedTime(&ms, ev0, ev1));
-    if (elapsedMs) *elapsedMs = ms;
-    return checkFlowError();
-}
-
-// Per-launch-class durations inside a token.  Events cannot be read back from
-// graph nodes, so the same launches are issued eagerly with an event between
-// every two of them -- behind a gate kernel that holds the stream until the
-// host has queued the whole batch, so the GPU never waits for the host.
-// classMs[c] = mean milliseconds from the end of the previous launch to the
-// end of a launch of class c (0 embed, 1 norm+QKV, 2 attention, 3 Wo,
-// 4 gate/up, 5 down, 6 lm_head, 7 argmax finish); classLaunches[c] = launches per token.
-int HIPFusedInference::ProfileDecode(int token, int pos, int steps, unsigned classMask, float* classMs, int* classLaunches) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(steps >= 1 && steps <= 64 && pos >= 0 && pos + steps <= maxSeq && token >= 0 && token < vocabSize &&
-           classMs && classLaunches, "ProfileDecode: bad arguments (1 <= steps <= 64)");
-    int rc = checkReady(this);
-    if (rc) return rc;
-    HIPCHK(hipStreamSynchronize(stream));
-    for (hipEvent_t e : profEvents) (void)hipEventDestroy(e);
-    profEvents.clear(); profClass.clear();
-    int* gate = hGate;
-    *reinterpret_cast<volatile int*>(gate) = 0;
-    { int rcs = setState(pos, token, 0, 0); if (rcs) return rcs; }
-    HIPCHK(launch_gate(gate, 100LL * 1000 * 500, stream));   // at most 0.5 s
-    profiling = true;
-    profMask = classMask ? classMask : 0xffu;
-    profLast = -1;
-    for (int i = 0; i < steps && rc == 0; i++) {
-        rc = enqueueToken(true);
-        if (rc == 0) rc = mark(8);
-    }
-    profiling = false;
-    *reinterpret_cast<volatile int*>(gate) = 1;
-    HIPCHK(hipStreamSynchronize(stream));
-    if (rc) return rc;
-    double acc[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-    int cnt[8] = {0, 0, 0, 0, 0, 0, 0, 0};
-    for (size_t k = 0; k + 1 < profEvents.size(); k++) {
-        int c = profClass[k];
-        if (c < 0 || c >= 8) continue;
-        float ms = 0.f;
-        HIPCHK(hipEventElapsedTime(&ms, profEvents[k], profEvents[k + 1]));
-        acc[c] += ms; cnt[c]++;
-    }
-    for (int c = 0; c < 8; c++) {
-        classMs[c] = cnt[c] ? (float)(acc[c] / cnt[c]) : 0.f;
-        classLaunches[c] = cnt[c] / steps;
-    }
-    for (hipEvent_t e : profEvents) (void)hipEventDestroy(e);
-    profEvents.clear(); profClass.clear();
-    return MG_OK;
-}
-
 // ---------------------------------------------------------------------------
 // Batched prefill (Q8): the layer of the decode step applied to T rows at
 // once, the seven projections as MFMA GEMMs.
@@ -1557,11 +1273,12 @@ int HIPFusedInference::ensurePrefill(int rows, int kvRows) {
     return MG_OK;
 }
 
-int HIPFusedInference::Prefill(const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs) {
+// The layers over all rows: pfX holds the rows' hidden states afterwards.
+int HIPFusedInference::prefillRows(const int* tokens, int nTokens, int pos0) {
     if (!built) return MG_E_NOT_BUILT;
     ARGCHK(tokens && nTokens >= 1 && pos0 >= 0 && pos0 + nTokens <= maxSeq, "Prefill: bad token count or position");
     for (int i = 0; i < nTokens; i++) ARGCHK(tokens[i] >= 0 && tokens[i] < vocabSize, "Prefill: token out of range");
-    int rc = checkReady(this);
+    int rc = checkReady();
     if (rc) return rc;
     for (const auto& L : layers) {
         // q/k/v and gate/up share a launch: one weight format each
@@ -1628,6 +1345,13 @@ int HIPFusedInference::Prefill(const int* tokens, int nTokens, int pos0, int* ne
         normSplitDone = g.wroteNext != 0;
         g.Ahi = static_cast<const unsigned short*>(pfHi); g.Alo = static_cast<const unsigned short*>(pfLo);
     }
+    return MG_OK;
+}
+
+int HIPFusedInference::Prefill(const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs) {
+    int rc = prefillRows(tokens, nTokens, pos0);
+    if (rc) return rc;
+    const int T = nTokens;
     // the last position continues on the decode path: final norm, lm_head, greedy token, state -> pos0 + T
     HIPCHK(hipMemcpyAsync(hidden[hiddenIdx], pfX + (size_t)(T - 1) * dim, (size_t)dim * 4, hipMemcpyDeviceToDevice, stream));
     { int rcs = setState(pos0 + T - 1, tokens[T - 1], 0, 0); if (rcs) return rcs; }
@@ -1643,23 +1367,20 @@ int HIPFusedInference::Prefill(const int* tokens, int nTokens, int pos0, int* ne
     return MG_OK;
 }
 
-// Prompt through the GEMM path, then nDecode - 1 graph replays from the device state it left.
-int HIPFusedInference::GeneratePrefill(const int* prompt, int nPrompt, int nDecode, int* outTokens) {
-    if (!built) return MG_E_NOT_BUILT;
-    ARGCHK(prompt && nPrompt >= 1 && nDecode >= 1 && outTokens, "GeneratePrefill: bad arguments");
-    ARGCHK(nPrompt + nDecode <= maxSeq + 1, "GeneratePrefill: prompt + decode exceeds maxSeq");
-    const bool graphs = !runsInLaunch(true);
-    int rc = graphs ? GraphCapture() : MG_OK;
+int HIPFusedInference::PrefillLogits(const int* tokens, int nTokens, int pos0, const int* want, int nWant, float* logitsOut) {
+    ARGCHK(nWant >= 0 && (nWant == 0 || (want && logitsOut)), "PrefillLogits: bad arguments");
+    for (int i = 0; i < nWant; i++) ARGCHK(want[i] >= 0 && want[i] < nTokens, "PrefillLogits: wanted row out of range");
+    int rc = prefillRows(tokens, nTokens, pos0);
     if (rc) return rc;
-    rc = Prefill(prompt, nPrompt, 0, nullptr, nullptr, nullptr);
-    if (rc) return rc;
-    if (nDecode > 1 && graphs) { rc = primeGraph(); if (rc) return rc; }
-    rc = decodeRun(nDecode - 1, true);
-    if (rc) return rc;
-    HIPCHK(hipMemcpyAsync(hTokens, dHistory, sizeof(int) * (size_t)nDecode, hipMemcpyDeviceToHost, stream));
+    for (int i = 0; i < nWant; i++) {
+        HIPCHK(hipMemcpyAsync(hidden[hiddenIdx], pfX + (size_t)want[i] * dim, (size_t)dim * 4, hipMemcpyDeviceToDevice, stream));
+        rc = enqueueFinal(false);
+        if (rc) return rc;
+        HIPCHK(hipMemcpyAsync(logitsOut + (size_t)i * vocabSize, logits, (size_t)vocabSize * 4, hipMemcpyDeviceToHost, stream));
+        HIPCHK(hipStreamSynchronize(stream));
+    }
     HIPCHK(hipStreamSynchronize(stream));
-    for (int i = 0; i < nDecode; i++) outTokens[i] = hTokens[i];
-    return checkFlowError();
+    return MG_OK;
 }
 
 }  // namespace mg
@@ -1671,27 +1392,27 @@ using mg::HIPFusedInference;
 
 extern "C" {
 
-const char* mg_last_error(void) { return mg::get_error().c_str(); }
-
 mg_ctx* mg_create(int dim, int kvDim, int headDim, int nHeads, int nKVHeads, int ffnDim, int vocabSize, int nLayers,
                   int maxSeq, double ropeTheta, float eps) {
     mg::set_error("");
     HIPFusedInference* f = HIPFusedInference::New(dim, kvDim, headDim, nHeads, nKVHeads, ffnDim, vocabSize, nLayers,
                                                   maxSeq, ropeTheta, eps);
     if (!f) return nullptr;
-    return new mg_ctx{f};
+    mg_ctx* c = new mg_ctx;
+    c->f = f; c->fused = f;
+    return c;
 }
 struct mg_layer_graph { mg_ctx* c; mg::HIPFusedInference::LayerGraph lg; };
-void mg_destroy(mg_ctx* c) {
-    if (!c) return;
-    for (mg_layer_graph* g : c->layerGraphs) { if (c->f) c->f->LayerGraphDestroy(g->lg); g->c = nullptr; }
-    delete c->f;
-    delete c;
+static void drop_layer_graphs(mg_ctx* c) {
+    for (mg_layer_graph* g : c->layerGraphs) { if (c->fused) c->fused->LayerGraphDestroy(g->lg); g->c = nullptr; }
 }
 
-#define CTX(c) if (!(c) || !(c)->f) { mg::set_error("NULL context"); return MG_E_NOT_BUILT; } HIPFusedInference* f = (c)->f
+#define CTX(c)                                                                                                    \
+    if (!(c) || !(c)->f) { mg::set_error("NULL context"); return MG_E_NOT_BUILT; }                                  \
+    if (!(c)->fused) { mg::set_error("not available for this model class"); return MG_E_UNSUPPORTED; }              \
+    HIPFusedInference* f = (c)->fused
 
-int mg_num_weights(const mg_ctx* c) { return c && c->f ? c->f->NumWeights() : 0; }
+int mg_num_weights(const mg_ctx* c) { return c && c->fused ? c->fused->NumWeights() : 0; }
 int mg_set_weight(mg_ctx* c, int idx, const float* data, size_t n) { CTX(c); return f->SetWeight(idx, data, n); }
 int mg_set_weight_q8(mg_ctx* c, int idx, const int8_t* q, const float* scales) { CTX(c); return f->SetWeightQ8(idx, q, scales); }
 int mg_set_weight_q4_0(mg_ctx* c, int idx, const uint8_t* d, size_t n) { CTX(c); return f->SetWeightQ4_0(idx, d, n); }
@@ -1704,7 +1425,6 @@ int mg_set_quant_rounding(mg_ctx* c, int mode) {
 int mg_set_embedding_f16(mg_ctx* c, const uint16_t* t) { CTX(c); return f->SetEmbeddingF16(t); }
 int mg_set_embedding_f32(mg_ctx* c, const float* t) { CTX(c); return f->SetEmbeddingF32(t); }
 int mg_set_layer_range(mg_ctx* c, int a, int b) { CTX(c); return f->SetLayerRange(a, b); }
-int mg_reset_kv(mg_ctx* c) { CTX(c); return f->ResetKV(); }
 int mg_set_kv_format(mg_ctx* c, int fmt) { CTX(c); return f->SetKVFormat(fmt); }
 int mg_partial_step(mg_ctx* c, const float* hiddenIn, int pos, int l0, int l1, float* hiddenOut, float* logitsOut) {
     CTX(c); return f->PartialStep(hiddenIn, pos, l0, l1, hiddenOut, logitsOut);
@@ -1712,14 +1432,12 @@ int mg_partial_step(mg_ctx* c, const float* hiddenIn, int pos, int l0, int l1, f
 int mg_step_layer_resident(mg_ctx* c, int layer, int pos, const float* hiddenIn, float* preOut, float* postOut, float* logitsOut) {
     CTX(c); return f->StepLayerResident(layer, pos, hiddenIn, preOut, postOut, logitsOut);
 }
-int mg_export_hidden(mg_ctx* c, float* out) { CTX(c); return f->ExportHidden(out); }
 int mg_queue_hidden_to_l3(mg_ctx* c) { CTX(c); return f->QueueHiddenToL3(); }
 int mg_wait_l3(mg_ctx* c) { CTX(c); return f->WaitL3(); }
-const float* mg_get_l3_hidden(mg_ctx* c) { return c && c->f ? c->f->GetL3Hidden() : nullptr; }
+const float* mg_get_l3_hidden(mg_ctx* c) { return c && c->fused ? c->fused->GetL3Hidden() : nullptr; }
 int mg_signal_mailbox(mg_ctx* c) { CTX(c); return f->SignalMailbox(); }
 int mg_wait_mailbox(mg_ctx* c, int timeoutMs) { CTX(c); return f->WaitMailbox(timeoutMs); }
 int mg_swap_hidden_buffer(mg_ctx* c) { CTX(c); return f->SwapHiddenBuffer(); }
-int mg_hidden_idx(mg_ctx* c) { CTX(c); return f->hiddenIdx; }
 int mg_set_exec_mode(mg_ctx* c, int mode) {
     CTX(c);
     if (mode < 0 || mode > 4) { mg::set_error("exec mode must be 0, 1, 2, 3 or 4"); return MG_E_ARG; }
@@ -1727,26 +1445,20 @@ int mg_set_exec_mode(mg_ctx* c, int mode) {
     return MG_OK;
 }
 int mg_set_q4_act_quant(mg_ctx* c, int on) { CTX(c); return f->SetQ4ActQuant(on); }
-int mg_decode_token(mg_ctx* c, int token, int pos, int* next, float* logitsOut) { CTX(c); return f->DecodeToken(token, pos, next, logitsOut); }
-int mg_generate(mg_ctx* c, const int* prompt, int nPrompt, int nDecode, int* out, int useGraph) {
-    CTX(c); return f->Generate(prompt, nPrompt, nDecode, out, useGraph != 0);
-}
-int mg_graph_capture(mg_ctx* c) { CTX(c); return f->GraphCapture(); }
-int mg_graph_launch(mg_ctx* c, int token, int pos, int* next) { CTX(c); return f->GraphLaunch(token, pos, next); }
-int mg_graph_validate(mg_ctx* c, int token, int pos, float* md) { CTX(c); return f->GraphValidate(token, pos, md); }
 mg_layer_graph* mg_layer_graph_capture(mg_ctx* c, int layerStart, int layerEnd, int streamCount, int pipelineBreak, int pos) {
-    if (!c || !c->f) { mg::set_error("NULL context"); return nullptr; }
+    if (!c || !c->fused) { mg::set_error("NULL context"); return nullptr; }
     if (streamCount == 0) streamCount = 1;                                   // cuda_graph.go:316
     if (streamCount != 1 && streamCount != 2) { mg::set_error("CaptureGraph: unsupported StreamCount (use 1 or 2)"); return nullptr; }
     if (streamCount == 2 && (pipelineBreak <= layerStart || pipelineBreak >= layerEnd)) {   // :396-400
         mg::set_error("CaptureGraph: PipelineBreak must lie between LayerStart and LayerEnd");
         return nullptr;
     }
-    if (pos < 0 || pos >= c->f->maxSeq) { mg::set_error("CaptureGraph: pos out of range"); return nullptr; }
+    if (pos < 0 || pos >= c->fused->maxSeq) { mg::set_error("CaptureGraph: pos out of range"); return nullptr; }
     mg_layer_graph* g = new mg_layer_graph{c, {}};
     g->lg.l0 = layerStart; g->lg.l1 = layerEnd;
-    if (c->f->LayerGraphCapture(g->lg) != MG_OK) { delete g; return nullptr; }
+    if (c->fused->LayerGraphCapture(g->lg) != MG_OK) { delete g; return nullptr; }
     c->layerGraphs.push_back(g);
+    c->dropGraphs = drop_layer_graphs;
     return g;
 }
 static bool live(mg_layer_graph* g) {
@@ -1756,23 +1468,22 @@ static bool live(mg_layer_graph* g) {
 }
 int mg_layer_graph_launch(mg_layer_graph* g, int pos) {
     if (!live(g)) return MG_E_STATE;
-    return g->c->f->LayerGraphLaunch(g->lg, pos);
+    return g->c->fused->LayerGraphLaunch(g->lg, pos);
 }
 int mg_layer_graph_update_and_launch(mg_layer_graph* g, int pos) {
     if (!live(g)) return 0;
-    return g->c->f->LayerGraphLaunch(g->lg, pos) == MG_OK ? 1 : 0;
+    return g->c->fused->LayerGraphLaunch(g->lg, pos) == MG_OK ? 1 : 0;
 }
 void mg_layer_graph_destroy(mg_layer_graph* g) {
     if (!g) return;
     if (g->c) {
-        g->c->f->LayerGraphDestroy(g->lg);
+        g->c->fused->LayerGraphDestroy(g->lg);
         auto& v = g->c->layerGraphs;
         for (size_t i = 0; i < v.size(); i++) if (v[i] == g) { v.erase(v.begin() + (long)i); break; }
     }
     delete g;
 }
 int mg_upload_hidden(mg_ctx* c, const float* data) { CTX(c); return f->UploadHidden(data); }
-int mg_read_hidden(mg_ctx* c, float* out) { CTX(c); return f->ExportHidden(out); }
 int mg_validate_graph_capture(mg_ctx* c, const float* hiddenIn, int layerStart, int layerEnd, float* maxDiff) {
     CTX(c);
     float md = 0.f;
@@ -1780,19 +1491,6 @@ int mg_validate_graph_capture(mg_ctx* c, const float* hiddenIn, int layerStart, 
     if (maxDiff) *maxDiff = md;
     if (rc) return rc;
     return md < 0.001f ? 1 : 0;
-}
-int mg_has_graph_kernel(void) { return 1; }
-int mg_timed_decode(mg_ctx* c, int token, int pos, int steps, int useGraph, float* ms) {
-    CTX(c); return f->TimedDecode(token, pos, steps, useGraph != 0, ms);
-}
-int mg_profile_decode(mg_ctx* c, int token, int pos, int steps, unsigned classMask, float* classMs, int* classLaunches) {
-    CTX(c); return f->ProfileDecode(token, pos, steps, classMask, classMs, classLaunches);
-}
-int mg_prefill(mg_ctx* c, const int* tokens, int nTokens, int pos0, int* next, float* logitsOut, float* ms) {
-    CTX(c); return f->Prefill(tokens, nTokens, pos0, next, logitsOut, ms);
-}
-int mg_generate_prefill(mg_ctx* c, const int* prompt, int nPrompt, int nDecode, int* out) {
-    CTX(c); return f->GeneratePrefill(prompt, nPrompt, nDecode, out);
 }
 // Inspection of the persistent layer launch's exchange area after a step (for tests): copies layer `layer`'s
 // block into out (cap floats) and writes its geometry {stride, offQ, offKc, offVc, offPacc, offPm, offPl,
@@ -1813,17 +1511,17 @@ int mg_flow_exchange(mg_ctx* c, int layer, float* out, size_t cap, int* geo) {
     return MG_OK;
 }
 int mg_flow_in_use(mg_ctx* c) {
-    if (!c || !c->f) return 0;
-    return c->f->FlowInUse() ? 1 : 0;
+    if (!c || !c->fused) return 0;
+    return c->fused->FlowInUse() ? 1 : 0;
 }
 int mg_flow_tail_in_use(mg_ctx* c) {
-    if (!c || !c->f) return 0;
-    return c->f->FlowTailInUse() ? 1 : 0;
+    if (!c || !c->fused) return 0;
+    return c->fused->FlowTailInUse() ? 1 : 0;
 }
 int mg_set_flow_tail(mg_ctx* c, int on) { CTX(c); f->SetFlowTail(on); return MG_OK; }
 int mg_set_flow_generic(mg_ctx* c, int on) { CTX(c); f->SetFlowGeneric(on); return MG_OK; }
 int mg_set_tokens_per_launch(mg_ctx* c, int n) { CTX(c); return f->SetTokensPerLaunch(n); }
-int mg_tokens_per_launch(mg_ctx* c) { return c && c->f ? c->f->tokensPerLaunch : 0; }
+int mg_tokens_per_launch(mg_ctx* c) { return c && c->fused ? c->fused->tokensPerLaunch : 0; }
 int mg_flow_tail_trace(mg_ctx* c, long long* out, size_t cap, int* dims) { CTX(c); return f->FlowTailTrace(out, cap, dims); }
 int mg_flow_set_wait_limit(mg_ctx* c, long long ticks) {
     CTX(c);
@@ -1834,7 +1532,5 @@ int mg_flow_trace(mg_ctx* c, int enable, long long* out, size_t cap, int* dims) 
     CTX(c);
     return f->FlowTrace(enable, out, cap, dims);
 }
-uint64_t mg_weight_bytes_per_token(const mg_ctx* c) { return c && c->f ? c->f->WeightBytesPerToken() : 0; }
-uint64_t mg_kv_bytes_at(const mg_ctx* c, int pos) { return c && c->f ? c->f->KVBytesAt(pos) : 0; }
 
 }  // extern "C"

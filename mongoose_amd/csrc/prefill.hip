@@ -9,6 +9,7 @@
 // by ~4e-3).  Accumulation is fp32; the row scale is applied once at the end.
 // Reference semantics: the same layer as the decode step, applied to T rows
 // (causal attention as kernels/mongoose.cu:251-353 does for training).
+#include "bf16_util.h"
 #include "kernels.h"
 #include "prefill.h"
 
@@ -19,14 +20,6 @@ typedef float float16_t __attribute__((ext_vector_type(16)));
 
 constexpr int PWG = 256;
 
-__device__ __forceinline__ unsigned short f32_to_bf16_rne(float f) {
-    unsigned u = __builtin_bit_cast(unsigned, f);
-    u += 0x7fffu + ((u >> 16) & 1u);          // round to nearest even (inputs are finite)
-    return (unsigned short)(u >> 16);
-}
-__device__ __forceinline__ float bf16_to_f32(unsigned short h) {
-    return __builtin_bit_cast(float, (unsigned)h << 16);
-}
 __device__ __forceinline__ float block_sum256(float v, float* red) {
 #pragma unroll
     for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
@@ -131,8 +124,8 @@ hipError_t launch_rope_store_rows(float* q, const float* k, const float* v, void
     return hipGetLastError();
 }
 
-// Embedding rows of T tokens from the tied Q8 table (kind 0), an fp16 (1) / fp32 (2) table, or the
-// tied Q4_0 table in the split layout (3).
+// Embedding rows of T tokens from the tied Q8 table (kind 0), an fp16 (1) / fp32 (2) table, the
+// tied Q4_0 table in the split layout (3), or a bf16 table (4).
 __global__ void embed_rows_kernel(int kind, const void* table, const float* scales, const int* tokens, float* x, int dim, int vocab) {
     int tok = tokens[blockIdx.x];
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
@@ -141,6 +134,7 @@ __global__ void embed_rows_kernel(int kind, const void* table, const float* scal
         if (kind == 0) o[i] = (float)static_cast<const signed char*>(table)[(size_t)tok * dim + i] * scales[tok];
         else if (kind == 1) o[i] = (float)__builtin_bit_cast(_Float16, static_cast<const unsigned short*>(table)[(size_t)tok * dim + i]);
         else if (kind == 2) o[i] = static_cast<const float*>(table)[(size_t)tok * dim + i];
+        else if (kind == 4) o[i] = bf16_to_f32(static_cast<const unsigned short*>(table)[(size_t)tok * dim + i]);
         else {
             const unsigned char* base = static_cast<const unsigned char*>(table);
             const int nb = dim >> 5, b = i >> 5, e = i & 31;

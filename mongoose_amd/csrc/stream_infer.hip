@@ -206,11 +206,11 @@ struct mg_stream { mg::HIPStreamInfer* s; };
 extern "C" {
 
 mg_stream* mg_stream_build(mg_ctx* ctx) {
-    if (!ctx || !ctx->f) { mg::set_error("mg_stream_build: NULL context"); return nullptr; }
-    if (ctx->f->dim % 32 || ctx->f->ffnDim % 32) { mg::set_error("mg_stream_build: Q4_0 needs dims % 32 == 0"); return nullptr; }
+    if (!ctx || !ctx->fused) { mg::set_error("mg_stream_build: NULL context, or a model class without streamed layers"); return nullptr; }
+    if (ctx->fused->dim % 32 || ctx->fused->ffnDim % 32) { mg::set_error("mg_stream_build: Q4_0 needs dims % 32 == 0"); return nullptr; }
     auto* s = new mg::HIPStreamInfer();
-    s->f = ctx->f;
-    ctx->f->backrefs.push_back(&s->f);
+    s->f = ctx->fused;
+    ctx->fused->backrefs.push_back(&s->f);
     if (s->build() != MG_OK) { delete s; return nullptr; }
     return new mg_stream{s};
 }
