@@ -370,6 +370,10 @@ int mg_profile_decode(mg_ctx* ctx, int token, int pos, int steps, unsigned class
  * with that token, so mg_generate-style graph replays can follow.  elapsedMs
  * (optional) is the device time of the whole call measured with events. */
 int mg_prefill(mg_ctx* ctx, const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs);
+/* mg_prefill with the logits of chosen positions instead of the last one's: want[nWant] are indices into
+ * `tokens`, logitsOut is [nWant, vocab].  nWant may be 0 (then only the caches and states advance).  The
+ * device step state is not set: a decode that follows goes through mg_decode_token / mg_prefill. */
+int mg_prefill_logits(mg_ctx* ctx, const int* tokens, int nTokens, int pos0, const int* want, int nWant, float* logitsOut);
 /* mg_generate with the prompt run through mg_prefill (nDecode >= 1). */
 int mg_generate_prefill(mg_ctx* ctx, const int* prompt, int nPrompt, int nDecode, int* outTokens);
 
@@ -436,6 +440,58 @@ int mg_flow_set_wait_limit(mg_ctx* ctx, long long ticks);
  * bandwidth roofline is computed from), and the KV bytes read at position pos. */
 uint64_t mg_weight_bytes_per_token(const mg_ctx* ctx);
 uint64_t mg_kv_bytes_at(const mg_ctx* ctx, int pos);
+
+/* ------------------------------------------------------------------ */
+/* Models described by a list of layers (Vadonex)                       */
+/* ------------------------------------------------------------------ */
+/* A second model class behind the same handle: every layer names its mixer and its feed-forward with their
+ * sizes; the token loop, graphs, prefill, generation and timing calls above (mg_decode_token, mg_generate,
+ * mg_generate_prefill, mg_prefill, mg_prefill_logits, mg_graph_*, mg_timed_decode, mg_profile_decode, mg_reset_kv,
+ * mg_export_hidden, mg_weight_bytes_per_token, mg_kv_bytes_at) work on it; the calls that are about the
+ * quantized model class return MG_E_UNSUPPORTED.  No counterpart in the reference.
+ *
+ * With layers i = 0 .. n-1, X_0 the embedding and x the running input of a layer:
+ *   x <- rms(alpha x + mixer(x)) * norm1;  x <- rms(alpha x + ff(x)) * norm2 (where there is a feed-forward);
+ *   X_(i+1) = x;  x <- sum_j dwa_i[j] X_j, j = 0 .. i+1;      logits = head (rms(x) * final norm).
+ * A latent attention layer caches its latents and rotated key parts, a delta rule layer carries a state: such a
+ * model only continues at the position where its last call stopped, or starts over at 0 (MG_E_STATE otherwise).
+ * Weights are bf16 matrices and fp32 vectors; f32 = 0: bf16 activations in the multi-row products and bf16 cache
+ * rows, fp32 elsewhere; f32 = 1: fp32 throughout. */
+#define MG_MIX_LATENT_ATTENTION 0
+#define MG_MIX_GENERAL_DELTA    1
+#define MG_MLP_NONE  0
+#define MG_MLP_DENSE 1     /* W_down xIELU(W_up x) */
+#define MG_MLP_MOE   2     /* sum over the chosen experts of softmax score * W_down gelu(W_up x), + shared expert */
+typedef struct {
+    int mixer;
+    int heads, dim;                  /* key channels a head (latent: the unrotated ones) */
+    int rot_dim, vdim, kv_rank, q_rank;   /* latent attention */
+    int window;                      /* keys a position sees, itself included; 0: all */
+    int kv_from;                     /* layer whose latents this one reads, -1: its own */
+    int rope_dims;                   /* rotated entries of the rotated part */
+    double rope_base;
+    float scale;
+    int decay_rank;                  /* delta rule: rows of w1 */
+    int mlp;
+    int ff, experts, top;            /* ff of the dense layer or of one expert */
+    int ff_shared;                   /* 0: no shared expert */
+} mg_layer_desc;
+typedef struct {
+    int width, vocab, n_layers;
+    float eps, alpha;
+    int f32;
+} mg_model_desc;
+mg_ctx* mg_create_layered(const mg_model_desc* model, const mg_layer_desc* layers, int maxSeq);
+/* Tensors by name ("embed", "l0.mix.dq", ...): mg_num_tensors of them; mg_tensor_shape returns the dimension count
+ * (1 or 2) and the sizes, or MG_E_ARG for a name the model does not have. */
+int mg_num_tensors(const mg_ctx* ctx);
+const char* mg_tensor_name(const mg_ctx* ctx, int i);
+int mg_tensor_shape(const mg_ctx* ctx, const char* name, int64_t* shape /* [2] */);
+/* bf16 values, row-major [rows, cols] or [n]. */
+int mg_set_tensor_bf16(mg_ctx* ctx, const char* name, const uint16_t* data, size_t n);
+/* mg_prefill_logits up to and including layer layerEnd - 1: the rows' x after it, [nTokens, width].  Advances the
+ * caches and states of those layers only, so the sequence has to be started over afterwards.  For tests. */
+int mg_prefill_hidden(mg_ctx* ctx, const int* tokens, int nTokens, int pos0, int layerEnd, float* out);
 
 /* ------------------------------------------------------------------ */
 /* Streaming inference (weights larger than device memory)              */

@@ -4,6 +4,7 @@
 
 The library is written next to this file so that it travels with the tree.
 """
+import fcntl
 import os
 import shutil
 import subprocess
@@ -12,8 +13,13 @@ import sys
 HERE = os.path.dirname(os.path.abspath(__file__))
 CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libmongoose_hip.so")
+# The model class of layered.hip without the quantized one (whose persistent launch takes minutes to compile): what a
+# fresh checkout needs to run such a model.  The full library has everything.
+LAYERED_LIB = os.path.join(HERE, "libmongoose_layered.so")
 
-SOURCES = ["kernels.hip", "flow.hip", "prefill.hip", "q4_dp4a.hip", "abi.hip", "fused_infer.hip", "stream_infer.hip", "host_quant.cpp"]
+LAYERED_SOURCES = ["kernels.hip", "prefill.hip", "q4_dp4a.hip", "abi.hip", "context.hip", "host_quant.cpp",
+                   "linear.hip", "latent_attn.hip", "delta_rule.hip", "row_ops.hip", "layered.hip"]
+SOURCES = ["flow.hip", "fused_infer.hip", "stream_infer.hip"] + LAYERED_SOURCES
 
 # -packed-fp32-ops off: hipcc must not form v_pk_*_f32 from float code on this target.
 DEVICE_FLAGS = ["--offload-arch=gfx950", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
@@ -28,19 +34,28 @@ def hipcc():
     return exe
 
 
-def build(verbose=True):
+def build(verbose=True, sources=None, lib=LIB):
+    """Compile `sources` (all of them by default) and link them into `lib`.  One build at a time in a checkout; the
+    library appears under its name only when it is complete."""
     objdir = os.path.join(HERE, "build")
     os.makedirs(objdir, exist_ok=True)
+    with open(os.path.join(objdir, ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        return _build(objdir, verbose, sources or SOURCES, lib)
+
+
+def build_layered(verbose=True):
+    return build(verbose, LAYERED_SOURCES, LAYERED_LIB)
+
+
+def _build(objdir, verbose, sources, lib):
     objs = []
     procs = []
-    for src in SOURCES:
+    for src in sources:
         path = os.path.join(CSRC, src)
-        if not os.path.exists(path):
-            continue
         obj = os.path.join(objdir, src.rsplit(".", 1)[0] + ".o")
-        cmd = [hipcc()] + COMMON_FLAGS + DEVICE_FLAGS + ["-c", path, "-o", obj]
-        if src.endswith(".cpp"):
-            cmd = [hipcc()] + COMMON_FLAGS + ["-x", "hip"] + DEVICE_FLAGS + ["-c", path, "-o", obj]
+        lang = ["-x", "hip"] if src.endswith(".cpp") else []
+        cmd = [hipcc()] + COMMON_FLAGS + lang + DEVICE_FLAGS + ["-c", path, "-o", obj]
         if verbose:
             print(" ".join(cmd), flush=True)
         procs.append((src, subprocess.Popen(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)))
@@ -49,18 +64,20 @@ def build(verbose=True):
     for src, p in procs:
         out, _ = p.communicate()
         lines = [l for l in out.splitlines() if "packed-fp32-ops" not in l or "error" in l]
-        if lines and verbose:
-            print("\n".join(lines), flush=True)
+        if lines and (verbose or p.returncode != 0):
+            print("\n".join(lines), file=sys.stdout if verbose else sys.stderr, flush=True)
         if p.returncode != 0:
             failed = True
             print(f"FAILED: {src}", file=sys.stderr)
     if failed:
         raise RuntimeError("hipcc compile failed")
-    link = [hipcc(), "-shared", "-fPIC", "--offload-arch=gfx950", "-o", LIB] + objs + ["-lpthread"]
+    part = lib + ".part"
+    link = [hipcc(), "-shared", "-fPIC", "--offload-arch=gfx950", "-Wl,-z,defs", "-o", part] + objs + ["-lpthread"]
     if verbose:
         print(" ".join(link), flush=True)
     subprocess.check_call(link)
-    return LIB
+    os.replace(part, lib)
+    return lib
 
 
 if __name__ == "__main__":

@@ -1,4 +1,5 @@
-"""Model shapes of the decode workloads (the five benchmark configurations)."""
+"""Model shapes of the decode workloads (the five benchmark configurations), and the readers of model folders'
+config.json: ARCHITECTURES maps its "architecture" to the function that turns it into a model description."""
 from collections import namedtuple
 
 Shape = namedtuple("Shape", "name nLayers dim nHeads nKVHeads headDim ffnDim vocab eps theta bias tied fmt")
@@ -35,3 +36,61 @@ def weight_bytes_per_token(s):
 
 def kv_bytes_at(s, pos):
     return 2 * s.nLayers * (pos + 1) * kv_dim(s) * 4
+
+
+# ---------------------------------------------------------------------------
+# models described by a list of layers
+# ---------------------------------------------------------------------------
+# layers: one dict of mg_layer_desc fields (include/mongoose_hip.h) a layer
+LayeredModel = namedtuple("LayeredModel", "name width vocab eps alpha layers")
+
+MIX_LATENT_ATTENTION, MIX_GENERAL_DELTA = 0, 1
+MLP_NONE, MLP_DENSE, MLP_MOE = 0, 1, 2
+
+
+def latent_attention(heads, dim, rot_dim, vdim, kv_rank, q_rank, scale, rope_base, rope_dims=None, window=0, kv_from=None):
+    return dict(mixer=MIX_LATENT_ATTENTION, heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank,
+                scale=scale, rope_base=rope_base, rope_dims=rot_dim if rope_dims is None else rope_dims, window=window,
+                kv_from=-1 if kv_from is None else kv_from)
+
+
+def general_delta(heads, dim, decay_rank):
+    return dict(mixer=MIX_GENERAL_DELTA, heads=heads, dim=dim, decay_rank=decay_rank, kv_from=-1)
+
+
+def dense_ff(ff):
+    return dict(mlp=MLP_DENSE, ff=ff)
+
+
+def moe_ff(ff, experts, top, ff_shared=0):
+    return dict(mlp=MLP_MOE, ff=ff, experts=experts, top=top, ff_shared=ff_shared)
+
+
+def read_vadonex(cfg, shape):
+    """Vadonex: latent attention (latents optionally shared between layers) and generalized delta rule layers, dense or
+    mixture feed-forwards, norm after the sum, a learned average over depth.  shape(name) gives a tensor's sizes."""
+    layers = []
+    for i, entry in enumerate(cfg["layers"]):
+        m, mlp, pre = entry["mixer"], entry.get("mlp"), f"l{i}."
+        if entry["type"] == "latent_attention":
+            layer = latent_attention(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], shape(pre + "mix.dq")[0],
+                                     m["scale"], m["rot"]["base"], m["rot"]["dims"], (m.get("mask") or {}).get("size") or 0,
+                                     m.get("kv_from"))
+        elif entry["type"] == "general_delta":
+            layer = general_delta(m["heads"], m["dim"], shape(pre + "mix.w1")[0])
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {entry['type']!r}")
+        if mlp is None:
+            pass
+        elif mlp["kind"] == "dense":
+            layer.update(dense_ff(mlp["ff"]))
+        elif mlp["kind"] == "moe":
+            layer.update(moe_ff(mlp["expert"]["ff"], mlp["router"]["experts"], mlp["router"]["top"],
+                                mlp["shared"]["ff"] if mlp.get("shared") else 0))
+        else:
+            raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+        layers.append(layer)
+    return LayeredModel("vadonex", cfg["width"], cfg["vocab"], cfg["norm"]["eps"], cfg["postln_alpha"], tuple(layers))
+
+
+ARCHITECTURES = {"Vadonex": read_vadonex}

@@ -1,0 +1,25 @@
+// activations.h -- scalar functions of the feed-forwards and gates (device), all in fp32.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <math.h>
+
+namespace mg {
+
+// What is applied to a finished row of a product.
+enum ActKind { ACT_NONE = 0, ACT_GELU = 1, ACT_XIELU = 2, ACT_TANH = 3 };
+// xIELU: z > 0: ap z^2 + z/2;  z <= 0: an (exp(z) - 1 - z) + z/2 with ap = softplus(p), an = 1/2 + softplus(q).
+struct ActParam { int kind; float ap, an; };
+
+__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+__device__ __forceinline__ float xielu_f(float z, float ap, float an) {
+    return z > 0.f ? ap * z * z + 0.5f * z : an * (expm1f(z) - z) + 0.5f * z;
+}
+__device__ __forceinline__ float apply_act(float z, ActParam a) {
+    if (a.kind == ACT_GELU) return gelu_erf_f(z);
+    if (a.kind == ACT_XIELU) return xielu_f(z, a.ap, a.an);
+    if (a.kind == ACT_TANH) return tanhf(z);
+    return z;
+}
+
+}  // namespace mg

@@ -147,7 +147,7 @@ hipError_t launch_q4_0_dp4a(const void* w, bool planar, const void* q8, float* o
 hipError_t launch_argmax_slices(const float* x, int n, int nparts, float* pv, int* pi, hipStream_t s);
 
 // Embedding row of state->token into x[dim]: kind 0 = Q8 row * scale (tied
-// lm_head), 1 = fp16 table, 2 = fp32 table, 3 = Q4_0 split-layout row.
+// lm_head), 1 = fp16 table, 2 = fp32 table, 3 = Q4_0 split-layout row, 4 = bf16 table.
 hipError_t launch_embed_token(int kind, const void* table, const float* scales, const StepState* state,
                               float* x, int dim, int vocab, hipStream_t s);
 // Reduce the lm_head partials to a token, append it to the history and

@@ -1,0 +1,144 @@
+// layered.h -- LayeredInference: a model class whose layers are described one by one (mixer, feed-forward and their
+// sizes), with bf16 weights.  It supplies DecodeContext with the launches of a token and of many rows; the mechanisms
+// themselves are launches of their own (linear.h, latent_attn.h, delta_rule.h, row_ops.h).
+#pragma once
+#include "../../include/mongoose_hip.h"
+#include "context.h"
+#include "delta_rule.h"
+#include "latent_attn.h"
+#include "linear.h"
+#include "row_ops.h"
+
+#include <map>
+#include <string>
+#include <vector>
+
+namespace mg {
+
+// Where index i of a tensor's axis lies in the stored matrix: blocks of `block` entries `blockPad` apart, and inside a
+// block the entries from `split` on start at `splitPad`.
+struct AxisMap {
+    int block = 0x7fffffff, blockPad = 0, split = 0x7fffffff, splitPad = 0;
+    int at(int i) const {
+        const int b = i / block, r = i % block;
+        return b * blockPad + (r < split ? r : splitPad + r - split);
+    }
+};
+
+struct TensorSlot {
+    int rows = 0, cols = 0;              // cols 0: a vector of `rows`
+    unsigned short* mat = nullptr;       // stored bf16 matrix: storedRows x ld
+    int storedRows = 0, ld = 0;
+    AxisMap rowMap, colMap;
+    unsigned short* matT = nullptr;      // per head of headRows rows also [cols, ldT] transposed
+    int headRows = 0, ldT = 0;
+    float* vec = nullptr;                // device vector
+    std::vector<float>* host = nullptr;  // host copy
+    bool set = false;
+};
+
+struct LayerBlock {
+    mg_layer_desc d;
+    // latent attention
+    int dimPad = 0, headW = 0, vPad = 0;
+    bool expanded = false;               // the matrix-core form has a variant for these sizes
+    Bf16Mat proj, uq, uk, uv, out;       // proj: [dq | dkv] or [r | k | v | g | a | w1]
+    unsigned short* ukT = nullptr;       // [heads, kv_rank, ldUkT]
+    int ldUkT = 0;
+    float *qNorm = nullptr, *kvNorm = nullptr;
+    LatentCache cache;                   // of this layer, or of the layer it reads from
+    int splits = 1, splitLen = 0;        // of the decode attention
+    // delta rule
+    DeltaParams delta;
+    float *aBias = nullptr, *w0 = nullptr, *oNorm = nullptr;
+    Bf16Mat w2;
+    float* S = nullptr;
+    // around
+    float *norm1 = nullptr, *norm2 = nullptr, *dwa = nullptr;
+    std::vector<float> dwaHost, actHost;
+    // feed-forward: up / down of the dense layer; gate = [router | shared up], up / down of expert 0
+    Bf16Mat up, down, gate, downShared;
+    size_t upStride = 0, downStride = 0; // elements from expert to expert
+    ActParam act{};
+};
+
+class LayeredInference : public DecodeContext {
+public:
+    static LayeredInference* New(const mg_model_desc& m, const mg_layer_desc* layers, int maxSeq);
+    ~LayeredInference() override;
+
+    int NumTensors() const { return (int)names.size(); }
+    const char* TensorName(int i) const { return i >= 0 && i < (int)names.size() ? names[i].c_str() : nullptr; }
+    int TensorShape(const char* name, int64_t* shape) const;
+    int SetTensor(const char* name, const uint16_t* data, size_t n);
+
+    int Prefill(const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs) override;
+    int PrefillLogits(const int* tokens, int nTokens, int pos0, const int* want, int nWant, float* logitsOut) override;
+    int PrefillHidden(const int* tokens, int nTokens, int pos0, int layerEnd, float* out);
+    int ResetKV() override;
+    int ExportHidden(float* out) override;
+    uint64_t WeightBytesPerToken() const override;
+    uint64_t KVBytesAt(int pos) const override;
+
+private:
+    LayeredInference() = default;
+    int build(const mg_layer_desc* descs);
+    int checkDesc(const mg_layer_desc* descs);
+    int checkReady() override;
+    int enqueueEmbed() override;
+    int enqueueToken(bool withHead) override;
+    int checkPosition(int pos) override;
+    void steppedTo(int pos) override { seqPos = pos; }
+    int saveSequence() override;
+    int restoreSequence() override;
+    EmbedRef embedRef() const;
+
+    int enqueueLatent(LayerBlock& L, const VecInput& in, const float* x, const SideJobs& dwa);
+    int enqueueDelta(LayerBlock& L, const VecInput& in, const float* x, const SideJobs& dwa);
+    int enqueueMlp(LayerBlock& L);
+    int enqueueHead(const VecInput& in, bool advance);
+
+    int ensureRows(int rows, int pos0);
+    int runRows(const int* tokens, int T, int pos0, int layerEnd);
+    int rowsLatent(LayerBlock& L, int T, int pos0);
+    int rowsDelta(LayerBlock& L, int T, int pos0);
+    int rowsMlp(LayerBlock& L, int T, NormRows& after);
+
+    float alpha = 0.f;
+    int f32 = 0;
+    int widthPad = 0;
+    std::vector<LayerBlock> layers;
+    std::map<std::string, TensorSlot> slots;
+    std::vector<std::string> names;
+    std::vector<Slab> slabs;             // weights, caches and states
+    bool recurrent = false;
+    size_t stateBytes = 0;               // of one copy of all states (they lie together)
+    float* states = nullptr;
+    float* statesSaved = nullptr;
+    int seqPos = 0, seqPosSaved = 0;
+    std::map<std::pair<double, int>, std::pair<float*, float*>> ropeTables;
+    Bf16Mat head;
+    float* finalNorm = nullptr;
+
+    // decode vectors
+    float *hist = nullptr;               // X_1 .. X_n
+    float *xcur = nullptr, *x1 = nullptr, *y1 = nullptr, *y2 = nullptr, *part = nullptr;
+    float *z = nullptr, *q = nullptr, *qlat = nullptr, *o = nullptr, *gateOut = nullptr, *hid = nullptr;
+    float *pacc = nullptr, *pm = nullptr, *pl = nullptr;
+
+    // multi-row buffers for rowCap rows
+    Slab rowSlab;
+    int rowCap = 0, keyCap = 0;
+    int* rTokens = nullptr;
+    int* rWant = nullptr;
+    float *rX = nullptr, *rXs = nullptr, *rY = nullptr, *rX1 = nullptr, *rZ = nullptr, *rQf = nullptr, *rQlat = nullptr;
+    float *rGate = nullptr, *rExp = nullptr, *rDec = nullptr, *rAu = nullptr, *rU = nullptr, *rO = nullptr, *rW1 = nullptr;
+    float *rPacc = nullptr, *rPm = nullptr, *rPl = nullptr, *rLogits = nullptr, *rWeights = nullptr;
+    void *aX = nullptr, *aX1 = nullptr, *aCq = nullptr, *aQ = nullptr, *aO = nullptr, *aHid = nullptr, *aShared = nullptr, *aWant = nullptr;
+    unsigned short *rK = nullptr, *rVt = nullptr;
+    int *rIds = nullptr, *rWork = nullptr, *rPerm = nullptr, *rNTiles = nullptr;
+    int4* rTiles = nullptr;
+    int ldz = 0;                         // row stride of rZ
+};
+
+}  // namespace mg

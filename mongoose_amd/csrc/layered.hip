@@ -1,0 +1,943 @@
+// layered.hip -- LayeredInference (layered.h) and its mg_* C entry points.  Host code only (no kernels here).
+#include "layered.h"
+#include "prefill.h"
+
+#include <algorithm>
+#include <cmath>
+#include <cstring>
+
+namespace mg {
+
+static constexpr int ROW_CHUNK = 4096;           // rows of one pass of a prefill
+static constexpr int EXPANDED_MIN_ROWS = 16;     // fewer rows attend in the absorbed form
+
+static Bf16Mat mat(int rows, int cols) {
+    Bf16Mat m;
+    m.rows = rows; m.cols = cols; m.ld = pad_to(cols, 64);
+    return m;
+}
+static double softplus(double v) { return std::log1p(std::exp(-std::fabs(v))) + std::max(v, 0.0); }
+
+int LayeredInference::checkDesc(const mg_layer_desc* d) {
+    ARGCHK(dim >= 1 && dim <= 15360 && vocabSize >= 1 && nLayers >= 1 && maxSeq >= 1, "mg_create_layered: width, vocab, layer count or maxSeq out of range");
+    for (int i = 0; i < nLayers; i++) {
+        const mg_layer_desc& L = d[i];
+        const std::string at = "mg_create_layered: layer " + std::to_string(i) + ": ";
+        ARGCHK(L.heads >= 1 && L.dim >= 1, at + "heads and dim must be positive");
+        if (L.mixer == MG_MIX_LATENT_ATTENTION) {
+            ARGCHK(L.vdim >= 1 && L.q_rank >= 1 && L.window >= 0, at + "vdim, q_rank or window out of range");
+            ARGCHK(latent_decode_supported(L.kv_rank, L.rot_dim), at + "kv_rank must be 1..1024 and rot_dim 0..128");
+            ARGCHK(L.rope_dims >= 0 && L.rope_dims <= L.rot_dim && L.rope_dims % 2 == 0, at + "rope_dims must be even and at most rot_dim");
+            ARGCHK(L.rope_dims == 0 || L.rope_base > 0, at + "rope_base must be positive");
+            ARGCHK(pad_to(L.q_rank, 64) <= 8192 && L.dim <= 4096 && L.vdim <= 4096, at + "sizes out of range");
+            if (L.kv_from >= 0) {
+                ARGCHK(L.kv_from < i && d[L.kv_from].mixer == MG_MIX_LATENT_ATTENTION && d[L.kv_from].kv_from < 0,
+                       at + "kv_from must name an earlier latent attention layer with a cache of its own");
+                const mg_layer_desc& S = d[L.kv_from];
+                ARGCHK(S.kv_rank == L.kv_rank && S.rot_dim == L.rot_dim && S.rope_dims == L.rope_dims && S.rope_base == L.rope_base,
+                       at + "kv_from needs equal kv_rank, rot_dim and rotation");
+            }
+        } else {
+            ARGCHK(L.mixer == MG_MIX_GENERAL_DELTA, at + "unknown mixer");
+            ARGCHK(delta_supported(L.dim) && L.decay_rank >= 1 && L.decay_rank <= 4096, at + "dim must be at most 256, decay_rank 1..4096");
+        }
+        ARGCHK(L.mlp == MG_MLP_NONE || L.mlp == MG_MLP_DENSE || L.mlp == MG_MLP_MOE, at + "unknown feed-forward");
+        if (L.mlp != MG_MLP_NONE) ARGCHK(L.ff >= 1 && L.ff <= 32768, at + "ff out of range");
+        if (L.mlp == MG_MLP_MOE) {
+            ARGCHK(L.experts >= 1 && L.experts <= 512 && L.top >= 1 && L.top <= 32 && L.top <= L.experts, at + "experts must be 1..512, top 1..32");
+            ARGCHK(L.ff_shared >= 0 && (size_t)L.top * pad_to(L.ff, 64) + pad_to(L.ff_shared, 64) <= 36864, at + "top * ff + shared ff too large");
+        }
+    }
+    return MG_OK;
+}
+
+LayeredInference* LayeredInference::New(const mg_model_desc& m, const mg_layer_desc* descs, int maxSeq) {
+    int ndev = 0;
+    if (hipGetDeviceCount(&ndev) != hipSuccess || ndev == 0) {
+        (void)hipGetLastError();
+        set_error("mg_create_layered: no HIP device");
+        return nullptr;
+    }
+    auto* f = new LayeredInference();
+    f->dim = m.width; f->vocabSize = m.vocab; f->nLayers = m.n_layers; f->maxSeq = maxSeq;
+    f->eps = m.eps; f->alpha = m.alpha; f->f32 = m.f32 != 0;
+    if (f->checkDesc(descs) != MG_OK || f->build(descs) != MG_OK) { delete f; return nullptr; }
+    f->built = true;
+    return f;
+}
+
+LayeredInference::~LayeredInference() {
+    if (stream) (void)hipStreamSynchronize(stream);
+    invalidateGraphs();
+    rowSlab.release();
+    for (auto& s : slabs) s.release();
+    if (statesSaved) (void)hipFree(statesSaved);
+}
+
+// Device memory collected first and allocated as one slab.
+struct SlabPlan {
+    struct Item { void** p; size_t bytes; };
+    std::vector<Item> items;
+    size_t total = 0;
+    template <typename T> void want(T*& p, size_t n, size_t elem = sizeof(T)) {
+        items.push_back({(void**)&p, n * elem});
+        total += alignUp256(n * elem);
+    }
+    int place(Slab& s, hipStream_t stream) {
+        int rc = s.init(total + 256);
+        if (rc) return rc;
+        HIPCHK(hipMemsetAsync(s.base, 0, s.size, stream));
+        for (auto& i : items) { *i.p = s.take(i.bytes); if (!*i.p) { set_error("slab plan too small"); return MG_E_STATE; } }
+        return MG_OK;
+    }
+};
+
+int LayeredInference::build(const mg_layer_desc* descs) {
+    widthPad = pad_to(dim, 64);
+    int rc = initTokenState(0);
+    if (rc) return rc;
+    layers.resize(nLayers);
+    auto addMat = [&](const std::string& name, const Bf16Mat& store, int rowOff, int rows, int cols) -> TensorSlot& {
+        TensorSlot t;
+        t.rows = rows; t.cols = cols; t.ld = store.ld; t.storedRows = rows;
+        t.mat = store.w ? const_cast<unsigned short*>(store.w) + (size_t)rowOff * store.ld : nullptr;
+        names.push_back(name);
+        return slots[name] = t;
+    };
+    auto addVec = [&](const std::string& name, float* p, int n, std::vector<float>* host = nullptr) {
+        TensorSlot t;
+        t.rows = n; t.vec = p; t.host = host;
+        names.push_back(name);
+        slots[name] = t;
+    };
+
+    // rotation tables, one for each (base, dims): angle in double, stored as float
+    auto rope = [&](double base, int dims, LatentCache& c) -> int {
+        c.ropeDims = dims;
+        if (!dims) return MG_OK;
+        auto key = std::make_pair(base, dims);
+        auto it = ropeTables.find(key);
+        if (it == ropeTables.end()) {
+            const int half = dims / 2;
+            std::vector<float> cs((size_t)maxSeq * half), sn((size_t)maxSeq * half);
+            for (int i = 0; i < half; i++) {
+                const double fr = std::pow(base, -2.0 * i / dims);
+                for (int p = 0; p < maxSeq; p++) {
+                    cs[(size_t)p * half + i] = (float)std::cos(p * fr);
+                    sn[(size_t)p * half + i] = (float)std::sin(p * fr);
+                }
+            }
+            SlabPlan plan;
+            float *dc = nullptr, *ds = nullptr;
+            plan.want(dc, cs.size());
+            plan.want(ds, sn.size());
+            slabs.emplace_back();
+            int r = plan.place(slabs.back(), stream);
+            if (r) return r;
+            HIPCHK(hipStreamSynchronize(stream));
+            HIPCHK(hipMemcpy(dc, cs.data(), cs.size() * 4, hipMemcpyHostToDevice));
+            HIPCHK(hipMemcpy(ds, sn.data(), sn.size() * 4, hipMemcpyHostToDevice));
+            it = ropeTables.emplace(key, std::make_pair(dc, ds)).first;
+        }
+        c.cosTab = it->second.first;
+        c.sinTab = it->second.second;
+        return MG_OK;
+    };
+
+    // padded sizes first: a cache row has room for the widest head of every layer that reads it
+    for (int i = 0; i < nLayers; i++) {
+        LayerBlock& L = layers[i];
+        L.d = descs[i];
+        const mg_layer_desc& d = L.d;
+        if (d.mixer == MG_MIX_GENERAL_DELTA) { stateBytes += alignUp256((size_t)d.heads * d.dim * d.dim * 4); recurrent = true; continue; }
+        L.dimPad = pad_to(d.dim, 32);
+        const int w = latent_prefill_head_width(L.dimPad, d.rot_dim), v = latent_prefill_value_width(d.vdim);
+        L.expanded = !f32 && latent_prefill_supported(w, v);
+        L.headW = L.expanded ? w : L.dimPad + pad_to(d.rot_dim, 32);
+        L.vPad = L.expanded ? v : pad_to(d.vdim, 32);
+        LatentCache& c = layers[d.kv_from >= 0 ? d.kv_from : i].cache;
+        c.f32 = f32; c.rank = d.kv_rank; c.rankPad = pad_to(d.kv_rank, 64); c.rot = d.rot_dim;
+        c.stride = std::max(c.stride, c.rankPad + std::max(L.headW - L.dimPad, pad_to(d.rot_dim, 8)));
+        c.stride = pad_to(c.stride, 8);
+        const int span = d.window > 0 ? std::min(d.window, maxSeq) : maxSeq;
+        latent_decode_splits(span, d.heads, 1, &L.splits, &L.splitLen);
+    }
+    if (recurrent) {
+        SlabPlan plan;
+        plan.want(states, stateBytes / 4);
+        slabs.emplace_back();
+        rc = plan.place(slabs.back(), stream);
+        if (rc) return rc;
+    }
+
+    size_t zMax = 1, qMax = 1, qlatMax = 1, oMax = 1, gateMax = 1, hidMax = 1, paccMax = 1, pmMax = 1;
+    float* S = states;
+    for (int i = 0; i < nLayers; i++) {
+        LayerBlock& L = layers[i];
+        const mg_layer_desc& d = L.d;
+        const std::string pre = "l" + std::to_string(i) + ".", mx = pre + "mix.", ml = pre + "mlp.";
+        SlabPlan plan;
+        plan.want(L.norm1, dim);
+        if (d.mlp != MG_MLP_NONE) plan.want(L.norm2, dim);
+        plan.want(L.dwa, i + 2);
+        auto wantMat = [&](Bf16Mat& m, size_t copies = 1) { plan.want(m.w, copies * m.rows * m.ld); };
+        const bool ownKv = d.kv_from < 0;
+        const int HD = d.heads * d.dim;
+        if (d.mixer == MG_MIX_LATENT_ATTENTION) {
+            L.proj = mat(d.q_rank + (ownKv ? d.kv_rank + d.rot_dim : 0), dim); wantMat(L.proj);
+            L.uq = mat(d.heads * L.headW, d.q_rank); wantMat(L.uq);
+            if (L.expanded) { L.uk = mat(d.heads * L.dimPad, d.kv_rank); wantMat(L.uk); }
+            L.ldUkT = pad_to(d.dim, 64);
+            plan.want(L.ukT, (size_t)d.heads * d.kv_rank * L.ldUkT);
+            L.uv = mat(d.heads * L.vPad, d.kv_rank); wantMat(L.uv);
+            L.out = mat(dim, d.heads * L.vPad); wantMat(L.out);
+            plan.want(L.qNorm, d.q_rank);
+            if (ownKv) {
+                plan.want(L.kvNorm, d.kv_rank);
+                // (the tiled products read whole tiles of 64 rows)
+                plan.want(L.cache.rows, (size_t)(maxSeq + 64) * L.cache.stride, f32 ? 4 : 2);
+            }
+        } else {
+            L.proj = mat(5 * HD + d.decay_rank, dim); wantMat(L.proj);
+            L.w2 = mat(HD, d.decay_rank); wantMat(L.w2);
+            L.out = mat(dim, HD); wantMat(L.out);
+            plan.want(L.aBias, HD); plan.want(L.w0, HD); plan.want(L.oNorm, HD);
+            L.S = S;
+            S += alignUp256((size_t)d.heads * d.dim * d.dim * 4) / 4;
+        }
+        if (d.mlp == MG_MLP_DENSE) {
+            L.up = mat(d.ff, dim); wantMat(L.up);
+            L.down = mat(dim, d.ff); wantMat(L.down);
+        } else if (d.mlp == MG_MLP_MOE) {
+            L.up = mat(d.ff, dim); wantMat(L.up, d.experts);
+            L.down = mat(dim, d.ff); wantMat(L.down, d.experts);
+            L.upStride = (size_t)L.up.rows * L.up.ld;
+            L.downStride = (size_t)L.down.rows * L.down.ld;
+            L.gate = mat(d.experts + d.ff_shared, dim); wantMat(L.gate);
+            if (d.ff_shared) { L.downShared = mat(dim, d.ff_shared); wantMat(L.downShared); }
+            L.act.kind = ACT_GELU;
+        }
+        slabs.emplace_back();
+        rc = plan.place(slabs.back(), stream);
+        if (rc) return rc;
+
+        addVec(pre + "norm1", L.norm1, dim);
+        if (d.mlp != MG_MLP_NONE) addVec(pre + "norm2", L.norm2, dim);
+        addVec(pre + "dwa", L.dwa, i + 2, &L.dwaHost);
+        if (d.mixer == MG_MIX_LATENT_ATTENTION) {
+            if (ownKv) { rc = rope(d.rope_base, d.rope_dims, L.cache); if (rc) return rc; }
+            else L.cache = layers[d.kv_from].cache;
+            addMat(mx + "dq", L.proj, 0, d.q_rank, dim);
+            addVec(mx + "dq.norm", L.qNorm, d.q_rank);
+            if (ownKv) {
+                addMat(mx + "dkv", L.proj, d.q_rank, d.kv_rank + d.rot_dim, dim);
+                addVec(mx + "dkv.norm", L.kvNorm, d.kv_rank);
+            }
+            TensorSlot& uq = addMat(mx + "uq", L.uq, 0, d.heads * (d.dim + d.rot_dim), d.q_rank);
+            uq.storedRows = L.uq.rows;
+            uq.rowMap = {d.dim + d.rot_dim, L.headW, d.dim, L.dimPad};
+            TensorSlot& uk = addMat(mx + "uk", L.uk, 0, HD, d.kv_rank);
+            uk.storedRows = L.uk.rows;
+            uk.rowMap = {d.dim, L.dimPad, d.dim, 0};
+            uk.matT = L.ukT; uk.headRows = d.dim; uk.ldT = L.ldUkT;
+            TensorSlot& uv = addMat(mx + "uv", L.uv, 0, d.heads * d.vdim, d.kv_rank);
+            uv.storedRows = L.uv.rows;
+            uv.rowMap = {d.vdim, L.vPad, d.vdim, 0};
+            TensorSlot& wo = addMat(mx + "o", L.out, 0, dim, d.heads * d.vdim);
+            wo.colMap = {d.vdim, L.vPad, d.vdim, 0};
+            qMax = std::max(qMax, (size_t)L.uq.rows);
+            qlatMax = std::max(qlatMax, (size_t)d.heads * d.kv_rank);
+            oMax = std::max(oMax, (size_t)d.heads * L.vPad);
+            paccMax = std::max(paccMax, (size_t)d.heads * L.splits * L.cache.rankPad);
+            pmMax = std::max(pmMax, (size_t)d.heads * L.splits);
+        } else {
+            static const char* proj[5] = {"r", "k", "v", "g", "a"};
+            for (int k = 0; k < 5; k++) addMat(mx + proj[k], L.proj, k * HD, HD, dim);
+            addMat(mx + "w1", L.proj, 5 * HD, d.decay_rank, dim);
+            addMat(mx + "w2", L.w2, 0, HD, d.decay_rank);
+            addVec(mx + "a.b", L.aBias, HD);
+            addVec(mx + "w0", L.w0, HD);
+            addVec(mx + "norm", L.oNorm, HD);
+            addMat(mx + "o", L.out, 0, dim, HD);
+            L.delta.heads = d.heads; L.delta.dim = d.dim; L.delta.rank = d.decay_rank;
+            L.delta.aBias = L.aBias; L.delta.w0 = L.w0; L.delta.norm = L.oNorm; L.delta.w2 = L.w2; L.delta.eps = eps;
+            oMax = std::max(oMax, (size_t)HD);
+        }
+        zMax = std::max(zMax, (size_t)L.proj.rows);
+        if (d.mlp == MG_MLP_DENSE) {
+            addMat(ml + "up", L.up, 0, d.ff, dim);
+            addMat(ml + "down", L.down, 0, dim, d.ff);
+            addVec(ml + "act", nullptr, 2, &L.actHost);
+            hidMax = std::max(hidMax, (size_t)d.ff);
+        } else if (d.mlp == MG_MLP_MOE) {
+            for (int e = 0; e < d.experts; e++) {
+                const std::string ep = ml + "e" + std::to_string(e) + ".";
+                addMat(ep + "up", L.up, e * L.up.rows, d.ff, dim);
+                addMat(ep + "down", L.down, e * L.down.rows, dim, d.ff);
+            }
+            addMat(ml + "router", L.gate, 0, d.experts, dim);
+            if (d.ff_shared) {
+                addMat(ml + "shared.up", L.gate, d.experts, d.ff_shared, dim);
+                addMat(ml + "shared.down", L.downShared, 0, dim, d.ff_shared);
+            }
+            gateMax = std::max(gateMax, (size_t)L.gate.rows);
+            hidMax = std::max(hidMax, (size_t)d.top * d.ff);
+        }
+    }
+    {
+        SlabPlan plan;
+        head = mat(vocabSize, dim);
+        plan.want(head.w, (size_t)head.rows * head.ld);
+        plan.want(finalNorm, dim);
+        plan.want(hist, (size_t)nLayers * dim);
+        plan.want(xcur, dim); plan.want(x1, dim); plan.want(y1, dim); plan.want(y2, dim); plan.want(part, dim);
+        plan.want(z, zMax); plan.want(q, qMax); plan.want(qlat, qlatMax); plan.want(o, oMax);
+        plan.want(gateOut, gateMax); plan.want(hid, hidMax);
+        plan.want(pacc, paccMax); plan.want(pm, pmMax); plan.want(pl, pmMax);
+        slabs.emplace_back();
+        rc = plan.place(slabs.back(), stream);
+        if (rc) return rc;
+    }
+    addVec("final.norm", finalNorm, dim);
+    addMat("head", head, 0, vocabSize, dim);
+    {
+        HIPCHK(hipMalloc(&embedTable, (size_t)vocabSize * dim * 2));
+        embedKind = 4;
+        Bf16Mat e;
+        e.w = static_cast<unsigned short*>(embedTable);
+        e.rows = vocabSize; e.cols = dim; e.ld = dim;            // (read one row at a time: not padded)
+        addMat("embed", e, 0, vocabSize, dim);
+    }
+    HIPCHK(hipStreamSynchronize(stream));
+    return MG_OK;
+}
+
+int LayeredInference::TensorShape(const char* name, int64_t* shape) const {
+    auto it = slots.find(name ? name : "");
+    ARGCHK(it != slots.end(), std::string("no tensor of that name: ") + (name ? name : "NULL"));
+    shape[0] = it->second.rows; shape[1] = it->second.cols;
+    return it->second.cols ? 2 : 1;
+}
+
+int LayeredInference::SetTensor(const char* name, const uint16_t* data, size_t n) {
+    if (!built) return MG_E_NOT_BUILT;
+    auto it = slots.find(name ? name : "");
+    ARGCHK(it != slots.end(), std::string("no tensor of that name: ") + (name ? name : "NULL"));
+    TensorSlot& t = it->second;
+    ARGCHK(data && n == (size_t)t.rows * (t.cols ? t.cols : 1), std::string("wrong element count for ") + name);
+    auto widen = [](uint16_t h) { const uint32_t u = (uint32_t)h << 16; float f; std::memcpy(&f, &u, 4); return f; };
+    HIPCHK(hipStreamSynchronize(stream));
+    invalidateGraphs();
+    if (!t.cols) {
+        std::vector<float> v(t.rows);
+        for (int i = 0; i < t.rows; i++) v[i] = widen(data[i]);
+        if (t.vec) HIPCHK(hipMemcpy(t.vec, v.data(), (size_t)t.rows * 4, hipMemcpyHostToDevice));
+        if (t.host) *t.host = v;
+        for (LayerBlock& L : layers)
+            if (t.host == &L.actHost) L.act = ActParam{ACT_XIELU, (float)softplus(v[0]), (float)(0.5 + softplus(v[1]))};
+        t.set = true;
+        return MG_OK;
+    }
+    if (t.mat) {
+        std::vector<uint16_t> m((size_t)t.storedRows * t.ld, 0);
+        const bool plainCols = t.colMap.block == 0x7fffffff;
+        for (int r = 0; r < t.rows; r++) {
+            uint16_t* dst = m.data() + (size_t)t.rowMap.at(r) * t.ld;
+            const uint16_t* src = data + (size_t)r * t.cols;
+            if (plainCols) std::memcpy(dst, src, (size_t)t.cols * 2);
+            else for (int c = 0; c < t.cols; c++) dst[t.colMap.at(c)] = src[c];
+        }
+        HIPCHK(hipMemcpy(t.mat, m.data(), m.size() * 2, hipMemcpyHostToDevice));
+    }
+    if (t.matT) {
+        const int heads = t.rows / t.headRows;
+        std::vector<uint16_t> m((size_t)heads * t.cols * t.ldT, 0);
+        for (int h = 0; h < heads; h++)
+            for (int r = 0; r < t.headRows; r++)
+                for (int c = 0; c < t.cols; c++)
+                    m[((size_t)h * t.cols + c) * t.ldT + r] = data[((size_t)h * t.headRows + r) * t.cols + c];
+        HIPCHK(hipMemcpy(t.matT, m.data(), m.size() * 2, hipMemcpyHostToDevice));
+    }
+    t.set = true;
+    return MG_OK;
+}
+
+int LayeredInference::checkReady() {
+    for (const auto& n : names)
+        if (!slots[n].set) { set_error("tensor not set: " + n); return MG_E_STATE; }
+    return MG_OK;
+}
+
+// Cached rows can be attended to again; a recurrent state only continues where it stopped.
+int LayeredInference::checkPosition(int pos) {
+    if (pos == 0 || pos == seqPos || (!recurrent && pos < seqPos)) return MG_OK;
+    set_error("the sequence holds " + std::to_string(seqPos) + " positions and cannot continue at " + std::to_string(pos));
+    return MG_E_STATE;
+}
+
+int LayeredInference::ResetKV() {
+    if (!built) return MG_E_NOT_BUILT;
+    HIPCHK(hipStreamSynchronize(stream));
+    if (states) HIPCHK(hipMemsetAsync(states, 0, stateBytes, stream));
+    for (const LayerBlock& L : layers)
+        if (L.d.mixer == MG_MIX_LATENT_ATTENTION && L.d.kv_from < 0)
+            HIPCHK(hipMemsetAsync(L.cache.rows, 0, (size_t)(maxSeq + 64) * L.cache.stride * (f32 ? 4 : 2), stream));
+    HIPCHK(hipStreamSynchronize(stream));
+    seqPos = 0;
+    return MG_OK;
+}
+
+int LayeredInference::saveSequence() {
+    seqPosSaved = seqPos;
+    if (!states) return MG_OK;
+    if (!statesSaved) { void* v = nullptr; HIPCHK(hipMalloc(&v, stateBytes)); statesSaved = static_cast<float*>(v); }
+    HIPCHK(hipMemcpyAsync(statesSaved, states, stateBytes, hipMemcpyDeviceToDevice, stream));
+    return MG_OK;
+}
+int LayeredInference::restoreSequence() {
+    seqPos = seqPosSaved;
+    if (states) HIPCHK(hipMemcpyAsync(states, statesSaved, stateBytes, hipMemcpyDeviceToDevice, stream));
+    return MG_OK;
+}
+
+int LayeredInference::ExportHidden(float* out) {
+    if (!built) return MG_E_NOT_BUILT;
+    ARGCHK(out, "ExportHidden: NULL out");
+    HIPCHK(hipStreamSynchronize(stream));
+    HIPCHK(hipMemcpy(out, xcur, (size_t)dim * 4, hipMemcpyDeviceToHost));
+    return MG_OK;
+}
+
+uint64_t LayeredInference::WeightBytesPerToken() const {
+    uint64_t b = head.bytes() + (uint64_t)dim * 4;
+    for (const LayerBlock& L : layers) {
+        b += L.proj.bytes() + L.out.bytes() + (uint64_t)dim * 4 * (L.d.mlp == MG_MLP_NONE ? 1 : 2);
+        if (L.d.mixer == MG_MIX_LATENT_ATTENTION) b += L.uq.bytes() + (uint64_t)L.d.heads * L.d.kv_rank * L.ldUkT * 2 + L.uv.bytes();
+        else b += L.w2.bytes();
+        const uint64_t n = L.d.mlp == MG_MLP_MOE ? L.d.top : L.d.mlp == MG_MLP_DENSE ? 1 : 0;
+        b += n * (L.up.bytes() + L.down.bytes());
+        if (L.d.mlp == MG_MLP_MOE) b += L.gate.bytes() + L.downShared.bytes();
+    }
+    return b;
+}
+uint64_t LayeredInference::KVBytesAt(int pos) const {
+    uint64_t b = 0;
+    for (const LayerBlock& L : layers) {
+        if (L.d.mixer == MG_MIX_GENERAL_DELTA) { b += (uint64_t)2 * L.d.heads * L.d.dim * L.d.dim * 4; continue; }
+        const uint64_t keys = L.d.window > 0 ? std::min(L.d.window, pos + 1) : pos + 1;
+        b += keys * (L.d.kv_rank + L.d.rot_dim) * (f32 ? 4 : 2);
+    }
+    return b;
+}
+
+// ---------------------------------------------------------------------------
+// one token
+// ---------------------------------------------------------------------------
+int LayeredInference::enqueueEmbed() {
+    if (mark(0)) return MG_E_HIP;
+    HIPCHK(launch_embed_token(embedKind, embedTable, nullptr, dState, hidden[hiddenIdx], dim, vocabSize, stream));
+    return MG_OK;
+}
+EmbedRef LayeredInference::embedRef() const {
+    EmbedRef e{};
+    if (!fuseEmbed) return e;
+    e.kind = embedKind; e.table = embedTable; e.out = hidden[hiddenIdx]; e.dim = dim; e.vocab = vocabSize;
+    return e;
+}
+
+int LayeredInference::enqueueLatent(LayerBlock& L, const VecInput& in, const float* x, const SideJobs& dwa) {
+    const mg_layer_desc& d = L.d;
+    if (mark(1)) return MG_E_HIP;
+    MvBf16 m;
+    m.in = in; m.w = L.proj; m.out = z;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    m = MvBf16();
+    m.in.src = z; m.in.n = d.q_rank; m.in.gain = L.qNorm; m.in.eps = eps;
+    m.w = L.uq; m.out = q;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    // the query moves into the latent's space; the same launch writes this position's cache row
+    HeadMv a;
+    a.src = q; a.rowStride = L.uq.rows; a.headStride = L.headW; a.K = d.dim;
+    a.w = L.ukT; a.heads = d.heads; a.rows = d.kv_rank; a.ld = L.ldUkT; a.out = qlat;
+    a.side = dwa;
+    if (d.kv_from < 0) { a.side.cache = L.cache; a.side.z = z + d.q_rank; a.side.gain = L.kvNorm; a.side.eps = eps; }
+    HIPCHK(launch_head_matvec(a, stream));
+    if (mark(2)) return MG_E_HIP;
+    LatentDecode p;
+    p.qlat = qlat; p.q = q; p.headW = L.headW; p.ropeOff = L.dimPad; p.cache = L.cache;
+    p.heads = d.heads; p.window = d.window; p.scale = d.scale; p.state = dState;
+    p.splits = L.splits; p.splitLen = L.splitLen; p.pacc = pacc; p.pm = pm; p.pl = pl;
+    HIPCHK(launch_latent_decode(p, stream));
+    if (mark(3)) return MG_E_HIP;
+    HeadMv v;
+    v.K = d.kv_rank; v.pacc = pacc; v.pm = pm; v.pl = pl; v.splits = L.splits; v.accLd = L.cache.rankPad;
+    v.w = L.uv.w; v.heads = d.heads; v.rows = L.vPad; v.ld = L.uv.ld; v.out = o;
+    HIPCHK(launch_head_matvec(v, stream));
+    m = MvBf16();
+    m.in.src = o; m.in.n = d.heads * L.vPad;
+    m.w = L.out; m.epi = MV_RESID; m.resid = x; m.alpha = alpha; m.out = y1;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    return MG_OK;
+}
+
+int LayeredInference::enqueueDelta(LayerBlock& L, const VecInput& in, const float* x, const SideJobs& dwa) {
+    if (mark(1)) return MG_E_HIP;
+    MvBf16 m;
+    m.in = in; m.w = L.proj; m.out = z;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    if (mark(2)) return MG_E_HIP;
+    DeltaStep p;
+    p.d = L.delta; p.z = z; p.S = L.S; p.state = dState; p.y = o; p.side = dwa;
+    HIPCHK(launch_delta_step(p, stream));
+    if (mark(3)) return MG_E_HIP;
+    m = MvBf16();
+    m.in.src = o; m.in.n = L.d.heads * L.d.dim;
+    m.w = L.out; m.epi = MV_RESID; m.resid = x; m.alpha = alpha; m.out = y1;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    return MG_OK;
+}
+
+// y1 -> norm1 (kept in x1) -> feed-forward -> y2
+int LayeredInference::enqueueMlp(LayerBlock& L) {
+    const mg_layer_desc& d = L.d;
+    VecInput in;
+    in.src = y1; in.n = dim; in.gain = L.norm1; in.eps = eps; in.out = x1;
+    if (mark(4)) return MG_E_HIP;
+    MvBf16 m;
+    if (d.mlp == MG_MLP_DENSE) {
+        m.in = in; m.w = L.up; m.act = L.act; m.out = hid;
+        HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+        if (mark(5)) return MG_E_HIP;
+        m = MvBf16();
+        m.in.src = hid; m.in.n = d.ff;
+        m.w = L.down; m.epi = MV_RESID; m.resid = x1; m.alpha = alpha; m.out = y2;
+        HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+        return MG_OK;
+    }
+    m.in = in; m.w = L.gate; m.act = L.act; m.actFrom = d.experts; m.out = gateOut;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    m = MvBf16();
+    m.in.src = x1; m.in.n = dim;
+    m.w = L.up; m.act = L.act; m.out = hid;
+    m.routerLogits = gateOut; m.experts = d.experts; m.top = d.top; m.expertStride = L.upStride;
+    HIPCHK(launch_matvec_bf16(m, nullptr, stream));
+    if (mark(5)) return MG_E_HIP;
+    MvMoeDown p;
+    p.routerLogits = gateOut; p.experts = d.experts; p.top = d.top; p.hid = hid; p.ff = d.ff;
+    p.down = L.down; p.expertStride = L.downStride;
+    p.hidShared = gateOut + d.experts; p.ffShared = d.ff_shared; p.downShared = L.downShared;
+    p.resid = x1; p.alpha = alpha; p.out = y2;
+    HIPCHK(launch_moe_down(p, stream));
+    return MG_OK;
+}
+
+int LayeredInference::enqueueHead(const VecInput& in, bool advance) {
+    if (mark(6)) return MG_E_HIP;
+    MvBf16 m;
+    m.in = in; m.w = head; m.epi = MV_ARGMAX; m.out = logits; m.amaxVal = amaxVal; m.amaxIdx = amaxIdx;
+    int grid = 0;
+    HIPCHK(launch_matvec_bf16(m, &grid, stream));
+    if (mark(7)) return MG_E_HIP;
+    if (!advance) return MG_OK;
+    if (grid > amaxParts) { set_error("argmax partial buffer too small"); return MG_E_STATE; }
+    statePosHost = -1;
+    HIPCHK(launch_argmax_finish(amaxVal, amaxIdx, grid, dState, nullptr, dHistory, maxSeq + 1, vocabSize, ropeRef(), embedRef(), stream));
+    return MG_OK;
+}
+
+int LayeredInference::enqueueToken(bool withHead) {
+    int rc = fuseEmbed ? MG_OK : enqueueEmbed();
+    if (rc) return rc;
+    // how the running input x comes about: the embedding; then norm and weighted sum at the head of the next launch
+    VecInput in;
+    in.src = hidden[hiddenIdx]; in.n = dim; in.eps = eps;
+    const float* x = hidden[hiddenIdx];
+    for (int i = 0; i < nLayers; i++) {
+        LayerBlock& L = layers[i];
+        SideJobs dwa;                        // sum_j<=i dwa[j] X_j, while this layer's own output is being made
+        dwa.state = dState; dwa.part = part; dwa.coef = L.dwa; dwa.terms = i + 1; dwa.n = dim;
+        dwa.first = hidden[hiddenIdx]; dwa.hist = hist; dwa.histStride = dim;
+        rc = L.d.mixer == MG_MIX_LATENT_ATTENTION ? enqueueLatent(L, in, x, dwa) : enqueueDelta(L, in, x, dwa);
+        if (rc) return rc;
+        const bool mlp = L.d.mlp != MG_MLP_NONE;
+        if (mlp) { rc = enqueueMlp(L); if (rc) return rc; }
+        in = VecInput();
+        in.src = mlp ? y2 : y1; in.n = dim; in.gain = mlp ? L.norm2 : L.norm1; in.eps = eps;
+        in.normOut = hist + (size_t)i * dim;
+        in.part = part; in.coef = L.dwaHost[i + 1]; in.out = xcur;
+        x = xcur;
+    }
+    if (withHead) {
+        in.gain2 = finalNorm;
+        return enqueueHead(in, true);
+    }
+    statePosHost = -1;
+    HIPCHK(launch_advance_prompt(dState, dPrompt, ropeRef(), embedRef(), stream));
+    return MG_OK;
+}
+
+// ---------------------------------------------------------------------------
+// many rows
+// ---------------------------------------------------------------------------
+int LayeredInference::ensureRows(int rows, int pos0) {
+    int keys = 0;
+    for (const LayerBlock& L : layers)
+        if (L.expanded) keys = std::max(keys, std::min(pos0 + rows, L.d.window > 0 ? L.d.window - 1 + rows : pos0 + rows));
+    keys = pad_to(keys, 64);
+    if (rows <= rowCap && keys <= keyCap) return MG_OK;
+    HIPCHK(hipStreamSynchronize(stream));
+    rowSlab.release();
+    const int T = std::max(rowCap, pad_to(rows, 64));
+    const int K = std::max(keyCap, std::min(pad_to(maxSeq, 64), pad_to(keys + T, 1024)));
+    rowCap = keyCap = 0;
+    const size_t ae = f32 ? 4 : 2;
+    size_t zMax = 1, cq = 64, qMax = 64, qlat = 1, oMax = 64, gate = 1, hidA = 64, sh = 64, expOut = 1, HD = 1, w1 = 64, kMax = 1, vMax = 1, tiles = 1, work = 1;
+    size_t top = 1, pacc = 1, pms = 1;
+    for (const LayerBlock& L : layers) {
+        const mg_layer_desc& d = L.d;
+        zMax = std::max(zMax, (size_t)pad_to(L.proj.rows, 4));
+        oMax = std::max(oMax, (size_t)L.out.ld);
+        if (d.mixer == MG_MIX_LATENT_ATTENTION) {
+            cq = std::max(cq, (size_t)L.uq.ld);
+            qMax = std::max(qMax, (size_t)L.uq.rows);
+            const size_t rowsA = L.expanded ? EXPANDED_MIN_ROWS : T, groups = (d.heads + 3) / 4;
+            qlat = std::max(qlat, rowsA * d.heads * d.kv_rank);
+            const size_t parts = 4 * std::max<size_t>(512, groups * rowsA);
+            pacc = std::max(pacc, parts * L.cache.rankPad);
+            pms = std::max(pms, parts);
+            if (L.expanded) { kMax = std::max(kMax, (size_t)L.uk.rows); vMax = std::max(vMax, (size_t)L.uv.rows); }
+        } else {
+            HD = std::max(HD, (size_t)d.heads * d.dim);
+            w1 = std::max(w1, (size_t)L.w2.ld);
+        }
+        if (d.mlp == MG_MLP_DENSE) hidA = std::max(hidA, (size_t)T * L.down.ld);
+        if (d.mlp == MG_MLP_MOE) {
+            hidA = std::max(hidA, (size_t)T * d.top * L.down.ld);
+            gate = std::max(gate, (size_t)pad_to(d.experts, 4));
+            if (d.ff_shared) sh = std::max(sh, (size_t)L.downShared.ld);
+            expOut = std::max(expOut, (size_t)d.top * dim);
+            top = std::max(top, (size_t)d.top);
+            tiles = std::max(tiles, (size_t)moe_max_tiles(T, d.top, d.experts, MOE_TILE_ROWS));
+            work = std::max(work, (size_t)2 * d.experts);
+        }
+    }
+    ldz = (int)zMax;
+    const size_t Ts = T;
+    SlabPlan p;
+    p.want(rTokens, Ts); p.want(rWant, 256);
+    p.want(rX, (size_t)(nLayers + 1) * Ts * dim); p.want(rXs, Ts * dim); p.want(rY, Ts * dim); p.want(rX1, Ts * dim);
+    p.want(rZ, Ts * zMax); p.want(rQf, (size_t)qMax * Ts); p.want(rQlat, qlat);
+    p.want(rGate, Ts * gate); p.want(rExp, Ts * expOut);
+    p.want(rDec, Ts * HD); p.want(rAu, Ts * HD); p.want(rU, Ts * HD); p.want(rO, Ts * HD); p.want(rW1, Ts * w1);
+    p.want(rPacc, pacc); p.want(rPm, pms); p.want(rPl, pms);
+    p.want(rLogits, (size_t)256 * vocabSize); p.want(rWeights, Ts * top);
+    p.want(aX, Ts * widthPad, ae); p.want(aX1, Ts * widthPad, ae); p.want(aCq, Ts * cq, ae); p.want(aQ, Ts * qMax, ae);
+    p.want(aO, Ts * oMax, ae); p.want(aHid, hidA, ae); p.want(aShared, Ts * sh, ae); p.want(aWant, (size_t)256 * widthPad, ae);
+    p.want(rK, (size_t)K * kMax); p.want(rVt, (size_t)K * vMax);
+    p.want(rIds, Ts * top); p.want(rWork, work); p.want(rPerm, Ts * top); p.want(rNTiles, 4); p.want(rTiles, tiles);
+    int rc = p.place(rowSlab, stream);
+    if (rc) return rc;
+    rowCap = T; keyCap = K;
+    return MG_OK;
+}
+
+int LayeredInference::rowsLatent(LayerBlock& L, int T, int pos0) {
+    const mg_layer_desc& d = L.d;
+    Gemm g;
+    g.A = aX; g.f32 = f32; g.lda = widthPad; g.M = T;
+    g.W = L.proj.w; g.ldw = L.proj.ld; g.N = L.proj.rows; g.K = L.proj.ld;
+    g.mode = GEMM_F32; g.out = rZ; g.ldc = ldz;
+    HIPCHK(launch_gemm_bf16w(g, stream));
+    LatentRows r;
+    r.z = rZ; r.ldz = ldz; r.T = T; r.pos0 = pos0; r.qRank = d.q_rank; r.qGain = L.qNorm;
+    r.qAct = aCq; r.actF32 = f32; r.ldq = L.uq.ld; r.eps = eps; r.cache = L.cache;
+    if (d.kv_from < 0) r.kvGain = L.kvNorm;
+    HIPCHK(launch_latent_rows(r, stream));
+    const bool expanded = L.expanded && T >= EXPANDED_MIN_ROWS;
+    g = Gemm();
+    g.A = aCq; g.f32 = f32; g.lda = L.uq.ld; g.M = T;
+    g.W = L.uq.w; g.ldw = L.uq.ld; g.N = L.uq.rows; g.K = L.uq.ld;
+    if (expanded) {
+        g.mode = GEMM_ROPE; g.outAct = aQ; g.ldo = L.uq.rows;
+        g.headW = L.headW; g.ropeOff = L.dimPad; g.ropeDims = d.rope_dims; g.pos0 = pos0;
+        g.cosTab = L.cache.cosTab; g.sinTab = L.cache.sinTab;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        // keys and values of the visible range; values transposed, by multiplying the other way round
+        const int kBase = d.window > 0 ? std::max(0, pos0 - d.window + 1) : 0;
+        const int keys = pad_to(pos0 + T - kBase, 64);
+        const unsigned short* rows = static_cast<const unsigned short*>(L.cache.rows) + (size_t)kBase * L.cache.stride;
+        g = Gemm();
+        g.A = rows; g.lda = L.cache.stride; g.M = keys;
+        g.W = L.uk.w; g.ldw = L.uk.ld; g.N = L.uk.rows; g.K = L.uk.ld;
+        g.mode = GEMM_ACT; g.outAct = rK; g.ldo = L.uk.rows;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        g = Gemm();
+        g.A = L.uv.w; g.lda = L.uv.ld; g.M = L.uv.rows;
+        g.W = rows; g.ldw = L.cache.stride; g.N = keys; g.K = L.uv.ld;
+        g.mode = GEMM_ACT; g.outAct = rVt; g.ldo = keys;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        LatentPrefill p;
+        p.q = static_cast<const unsigned short*>(aQ); p.ldq = L.uq.rows; p.headW = L.headW; p.dimPad = L.dimPad;
+        p.k = rK; p.vt = rVt; p.ldv = keys; p.vPad = L.vPad; p.cache = L.cache; p.kBase = kBase;
+        p.heads = d.heads; p.window = d.window; p.scale = d.scale; p.T = T; p.pos0 = pos0;
+        p.out = static_cast<unsigned short*>(aO); p.ldo = L.out.ld;
+        HIPCHK(launch_latent_prefill(p, stream));
+    } else {
+        g.mode = GEMM_F32; g.out = rQf; g.ldc = L.uq.rows;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        HeadMv a;
+        a.src = rQf; a.rowStride = L.uq.rows; a.headStride = L.headW; a.K = d.dim;
+        a.w = L.ukT; a.heads = d.heads; a.rows = d.kv_rank; a.ld = L.ldUkT; a.out = rQlat; a.T = T;
+        HIPCHK(launch_head_matvec(a, stream));
+        LatentDecode p;
+        p.qlat = rQlat; p.q = rQf; p.headW = L.headW; p.ropeOff = L.dimPad; p.cache = L.cache;
+        p.heads = d.heads; p.window = d.window; p.scale = d.scale; p.pos0 = pos0; p.T = T;
+        const int span = d.window > 0 ? std::min(d.window, pos0 + T) : pos0 + T;
+        latent_decode_splits(span, d.heads, T, &p.splits, &p.splitLen);
+        p.pacc = rPacc; p.pm = rPm; p.pl = rPl;
+        HIPCHK(launch_latent_decode(p, stream));
+        HeadMv v;
+        v.K = d.kv_rank; v.pacc = rPacc; v.pm = rPm; v.pl = rPl; v.splits = p.splits; v.accLd = L.cache.rankPad;
+        v.w = L.uv.w; v.heads = d.heads; v.rows = L.vPad; v.ld = L.uv.ld; v.T = T;
+        v.outAct = aO; v.actF32 = f32; v.ldAct = L.out.ld;
+        HIPCHK(launch_head_matvec(v, stream));
+    }
+    return MG_OK;
+}
+
+int LayeredInference::rowsDelta(LayerBlock& L, int T, int pos0) {
+    Gemm g;
+    g.A = aX; g.f32 = f32; g.lda = widthPad; g.M = T;
+    g.W = L.proj.w; g.ldw = L.proj.ld; g.N = L.proj.rows; g.K = L.proj.ld;
+    g.mode = GEMM_F32; g.out = rZ; g.ldc = ldz;
+    HIPCHK(launch_gemm_bf16w(g, stream));
+    DeltaRows p;
+    p.d = L.delta; p.z = rZ; p.ldz = ldz; p.T = T; p.pos0 = pos0; p.S = L.S;
+    p.w1 = rW1; p.dec = rDec; p.au = rAu; p.u = rU; p.o = rO;
+    p.yAct = aO; p.actF32 = f32; p.ldAct = L.out.ld;
+    HIPCHK(launch_delta_rows(p, stream));
+    return MG_OK;
+}
+
+// aX1 / rX1 (after norm1) -> rY, which `after` norms (with the experts' outputs where there are any)
+int LayeredInference::rowsMlp(LayerBlock& L, int T, NormRows& after) {
+    const mg_layer_desc& d = L.d;
+    Gemm g;
+    if (d.mlp == MG_MLP_DENSE) {
+        g.A = aX1; g.f32 = f32; g.lda = widthPad; g.M = T;
+        g.W = L.up.w; g.ldw = L.up.ld; g.N = d.ff; g.K = L.up.ld;
+        g.mode = GEMM_ACT; g.outAct = aHid; g.ldo = L.down.ld; g.act = L.act;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        g = Gemm();
+        g.A = aHid; g.f32 = f32; g.lda = L.down.ld; g.M = T;
+        g.W = L.down.w; g.ldw = L.down.ld; g.N = dim; g.K = L.down.ld;
+        g.mode = GEMM_RESID; g.out = rY; g.ldc = dim; g.res = rX1; g.ldres = dim; g.alpha = alpha;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        return MG_OK;
+    }
+    const int ldg = pad_to(d.experts, 4);
+    g.A = aX1; g.f32 = f32; g.lda = widthPad; g.M = T;
+    g.W = L.gate.w; g.ldw = L.gate.ld; g.N = L.gate.rows; g.K = L.gate.ld;
+    g.mode = GEMM_SPLIT; g.nSplit = d.experts; g.out = rGate; g.ldc = ldg;
+    g.outAct = aShared; g.ldo = L.downShared.ld; g.act = L.act;
+    HIPCHK(launch_gemm_bf16w(g, stream));
+    MoeRoute r;
+    r.z = rGate; r.ldz = ldg; r.T = T; r.experts = d.experts; r.top = d.top;
+    r.ids = rIds; r.weights = rWeights; r.work = rWork; r.perm = rPerm; r.tiles = rTiles; r.nTiles = rNTiles;
+    HIPCHK(launch_moe_route(r, stream));
+    Gemm e;
+    e.f32 = f32; e.M = T * d.top; e.tiles = rTiles; e.nTiles = rNTiles; e.perm = rPerm;
+    e.maxTiles = moe_max_tiles(T, d.top, d.experts, MOE_TILE_ROWS);
+    g = e;
+    g.A = aX1; g.lda = widthPad; g.permDiv = d.top;
+    g.W = L.up.w; g.ldw = L.up.ld; g.N = d.ff; g.K = L.up.ld; g.expertStride = L.upStride;
+    g.mode = GEMM_ACT; g.outAct = aHid; g.ldo = L.down.ld; g.act = L.act;
+    HIPCHK(launch_gemm_bf16w(g, stream));
+    g = e;
+    g.A = aHid; g.lda = L.down.ld;
+    g.W = L.down.w; g.ldw = L.down.ld; g.N = dim; g.K = L.down.ld; g.expertStride = L.downStride;
+    g.mode = GEMM_SCATTER; g.out = rExp; g.ldc = dim; g.rowScale = rWeights;
+    HIPCHK(launch_gemm_bf16w(g, stream));
+    after.experts = rExp; after.top = d.top; after.ldExperts = dim;
+    if (d.ff_shared) {
+        g = Gemm();
+        g.A = aShared; g.f32 = f32; g.lda = L.downShared.ld; g.M = T;
+        g.W = L.downShared.w; g.ldw = L.downShared.ld; g.N = dim; g.K = L.downShared.ld;
+        g.mode = GEMM_RESID; g.out = rY; g.ldc = dim; g.res = rX1; g.ldres = dim; g.alpha = alpha;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+    } else {
+        after.y = rX1; after.yScale = alpha;
+    }
+    return MG_OK;
+}
+
+// Layers 0 .. layerEnd - 1 over T rows at pos0; rXs (fp32) and aX (activations) hold x afterwards.
+int LayeredInference::runRows(const int* tokens, int T, int pos0, int layerEnd) {
+    HIPCHK(hipStreamSynchronize(stream));
+    HIPCHK(hipMemcpy(rTokens, tokens, sizeof(int) * (size_t)T, hipMemcpyHostToDevice));
+    HIPCHK(launch_embed_rows(embedKind, embedTable, nullptr, rTokens, rX, T, dim, vocabSize, stream));
+    const size_t hs = (size_t)rowCap * dim;
+    NormRows n;
+    n.y = rX; n.T = T; n.n = dim; n.ldy = dim; n.out = rXs; n.ldOut = dim; n.outAct = aX; n.actF32 = f32; n.ldAct = widthPad;
+    HIPCHK(launch_norm_rows(n, stream));
+    for (int i = 0; i < layerEnd; i++) {
+        LayerBlock& L = layers[i];
+        const bool mlp = L.d.mlp != MG_MLP_NONE;
+        int rc = L.d.mixer == MG_MIX_LATENT_ATTENTION ? rowsLatent(L, T, pos0) : rowsDelta(L, T, pos0);
+        if (rc) return rc;
+        Gemm g;
+        g.A = aO; g.f32 = f32; g.lda = L.out.ld; g.M = T;
+        g.W = L.out.w; g.ldw = L.out.ld; g.N = dim; g.K = L.out.ld;
+        g.mode = GEMM_RESID; g.out = rY; g.ldc = dim; g.res = rXs; g.ldres = dim; g.alpha = alpha;
+        HIPCHK(launch_gemm_bf16w(g, stream));
+        // the layer's last norm also makes X_(i+1) and the weighted sum over all X_j
+        NormRows last;
+        last.y = rY; last.T = T; last.n = dim; last.ldy = dim; last.gain = mlp ? L.norm2 : L.norm1; last.eps = eps;
+        last.normOut = rX + (size_t)(i + 1) * hs; last.ldNorm = dim;
+        last.coef = L.dwa; last.terms = i + 1; last.hist = rX; last.histStride = hs; last.ldHist = dim;
+        last.out = rXs; last.ldOut = dim; last.outAct = aX; last.actF32 = f32; last.ldAct = widthPad;
+        if (mlp) {
+            NormRows n1;
+            n1.y = rY; n1.T = T; n1.n = dim; n1.ldy = dim; n1.gain = L.norm1; n1.eps = eps;
+            n1.out = rX1; n1.ldOut = dim; n1.outAct = aX1; n1.actF32 = f32; n1.ldAct = widthPad;
+            HIPCHK(launch_norm_rows(n1, stream));
+            rc = rowsMlp(L, T, last);
+            if (rc) return rc;
+        }
+        HIPCHK(launch_norm_rows(last, stream));
+    }
+    return MG_OK;
+}
+
+int LayeredInference::Prefill(const int* tokens, int nTokens, int pos0, int* nextToken, float* logitsOut, float* elapsedMs) {
+    if (!built) return MG_E_NOT_BUILT;
+    ARGCHK(tokens && nTokens >= 1 && pos0 >= 0 && pos0 + nTokens <= maxSeq, "Prefill: bad token count or position");
+    for (int i = 0; i < nTokens; i++) ARGCHK(tokens[i] >= 0 && tokens[i] < vocabSize, "Prefill: token out of range");
+    int rc = checkReady();
+    if (rc == MG_OK) rc = checkPosition(pos0);
+    if (rc == MG_OK) rc = ensureRows(std::min(nTokens, ROW_CHUNK), pos0 + nTokens - std::min(nTokens, ROW_CHUNK));
+    if (rc) return rc;
+    HIPCHK(hipStreamSynchronize(stream));
+    HIPCHK(hipEventRecord(ev0, stream));
+    steppedTo(-1);
+    int T = 0;
+    for (int at = 0; at < nTokens; at += T) {
+        T = std::min(nTokens - at, ROW_CHUNK);
+        rc = runRows(tokens + at, T, pos0 + at, nLayers);
+        if (rc) return rc;
+    }
+    // the last position continues on the decode path: final norm, lm_head, greedy token, state -> pos0 + nTokens
+    HIPCHK(hipMemcpyAsync(xcur, rXs + (size_t)(T - 1) * dim, (size_t)dim * 4, hipMemcpyDeviceToDevice, stream));
+    rc = setState(pos0 + nTokens - 1, tokens[nTokens - 1], 0, 0);
+    if (rc) return rc;
+    VecInput in;
+    in.src = xcur; in.n = dim; in.gain = finalNorm; in.eps = eps;
+    rc = enqueueHead(in, true);
+    if (rc) return rc;
+    HIPCHK(hipEventRecord(ev1, stream));
+    HIPCHK(hipMemcpyAsync(hTokens, dHistory, sizeof(int), hipMemcpyDeviceToHost, stream));
+    HIPCHK(hipStreamSynchronize(stream));
+    steppedTo(pos0 + nTokens);
+    if (nextToken) *nextToken = hTokens[0];
+    if (logitsOut) HIPCHK(hipMemcpy(logitsOut, logits, (size_t)vocabSize * 4, hipMemcpyDeviceToHost));
+    if (elapsedMs) HIPCHK(hipEventElapsedTime(elapsedMs, ev0, ev1));
+    return MG_OK;
+}
+
+int LayeredInference::PrefillLogits(const int* tokens, int nTokens, int pos0, const int* want, int nWant, float* logitsOut) {
+    if (!built) return MG_E_NOT_BUILT;
+    ARGCHK(tokens && nTokens >= 1 && pos0 >= 0 && pos0 + nTokens <= maxSeq, "PrefillLogits: bad token count or position");
+    ARGCHK(nWant >= 0 && (nWant == 0 || (want && logitsOut)), "PrefillLogits: bad arguments");
+    for (int i = 0; i < nTokens; i++) ARGCHK(tokens[i] >= 0 && tokens[i] < vocabSize, "PrefillLogits: token out of range");
+    for (int i = 0; i < nWant; i++) ARGCHK(want[i] >= 0 && want[i] < nTokens, "PrefillLogits: wanted row out of range");
+    if (nTokens == 1) {                              // one token is a decode step
+        std::vector<float> lg(vocabSize);
+        int rc = DecodeToken(tokens[0], pos0, nullptr, lg.data());
+        for (int i = 0; i < nWant && rc == MG_OK; i++) std::memcpy(logitsOut + (size_t)i * vocabSize, lg.data(), (size_t)vocabSize * 4);
+        return rc;
+    }
+    int rc = checkReady();
+    if (rc == MG_OK) rc = checkPosition(pos0);
+    if (rc == MG_OK) rc = ensureRows(std::min(nTokens, ROW_CHUNK), pos0 + nTokens - std::min(nTokens, ROW_CHUNK));
+    if (rc) return rc;
+    steppedTo(-1);
+    int T = 0;
+    for (int at = 0; at < nTokens; at += T) {
+        T = std::min(nTokens - at, ROW_CHUNK);
+        rc = runRows(tokens + at, T, pos0 + at, nLayers);
+        if (rc) return rc;
+        std::vector<int> rows, outs;
+        for (int i = 0; i < nWant; i++)
+            if (want[i] >= at && want[i] < at + T) { rows.push_back(want[i] - at); outs.push_back(i); }
+        for (size_t b = 0; b < rows.size(); b += 256) {
+            const int n = (int)std::min<size_t>(256, rows.size() - b);
+            HIPCHK(hipStreamSynchronize(stream));
+            HIPCHK(hipMemcpy(rWant, rows.data() + b, sizeof(int) * (size_t)n, hipMemcpyHostToDevice));
+            NormRows r;
+            r.y = rXs; r.T = n; r.n = dim; r.ldy = dim; r.rowIdx = rWant; r.gain = finalNorm; r.eps = eps;
+            r.outAct = aWant; r.actF32 = f32; r.ldAct = widthPad;
+            HIPCHK(launch_norm_rows(r, stream));
+            Gemm g;
+            g.A = aWant; g.f32 = f32; g.lda = widthPad; g.M = n;
+            g.W = head.w; g.ldw = head.ld; g.N = vocabSize; g.K = head.ld;
+            g.mode = GEMM_F32; g.out = rLogits; g.ldc = vocabSize;
+            HIPCHK(launch_gemm_bf16w(g, stream));
+            HIPCHK(hipStreamSynchronize(stream));
+            for (int i = 0; i < n; i++)
+                HIPCHK(hipMemcpy(logitsOut + (size_t)outs[b + i] * vocabSize, rLogits + (size_t)i * vocabSize, (size_t)vocabSize * 4, hipMemcpyDeviceToHost));
+        }
+    }
+    HIPCHK(hipMemcpyAsync(xcur, rXs + (size_t)(T - 1) * dim, (size_t)dim * 4, hipMemcpyDeviceToDevice, stream));
+    HIPCHK(hipStreamSynchronize(stream));
+    statePosHost = -1;
+    steppedTo(pos0 + nTokens);
+    return MG_OK;
+}
+
+int LayeredInference::PrefillHidden(const int* tokens, int nTokens, int pos0, int layerEnd, float* out) {
+    if (!built) return MG_E_NOT_BUILT;
+    ARGCHK(tokens && out && nTokens >= 1 && nTokens <= ROW_CHUNK && pos0 >= 0 && pos0 + nTokens <= maxSeq && layerEnd >= 0 && layerEnd <= nLayers,
+           "PrefillHidden: bad arguments");
+    for (int i = 0; i < nTokens; i++) ARGCHK(tokens[i] >= 0 && tokens[i] < vocabSize, "PrefillHidden: token out of range");
+    int rc = checkReady();
+    if (rc == MG_OK) rc = checkPosition(pos0);
+    if (rc == MG_OK) rc = ensureRows(nTokens, pos0);
+    if (rc) return rc;
+    steppedTo(-1);
+    rc = runRows(tokens, nTokens, pos0, layerEnd);
+    if (rc) return rc;
+    HIPCHK(hipStreamSynchronize(stream));
+    HIPCHK(hipMemcpy(out, rXs, (size_t)nTokens * dim * 4, hipMemcpyDeviceToHost));
+    return MG_OK;
+}
+
+}  // namespace mg
+
+// ---------------------------------------------------------------------------
+// C entry points
+// ---------------------------------------------------------------------------
+#define CTX(c)                                                                                                    \
+    if (!(c) || !(c)->f) { mg::set_error("NULL context"); return MG_E_NOT_BUILT; }                                  \
+    if (!(c)->layered) { mg::set_error("not available for this model class"); return MG_E_UNSUPPORTED; }            \
+    mg::LayeredInference* f = (c)->layered
+
+extern "C" {
+
+mg_ctx* mg_create_layered(const mg_model_desc* model, const mg_layer_desc* layers, int maxSeq) {
+    mg::set_error("");
+    if (!model || !layers) { mg::set_error("mg_create_layered: NULL description"); return nullptr; }
+    mg::LayeredInference* f = mg::LayeredInference::New(*model, layers, maxSeq);
+    if (!f) return nullptr;
+    mg_ctx* c = new mg_ctx;
+    c->f = f; c->layered = f;
+    return c;
+}
+int mg_num_tensors(const mg_ctx* c) { CTX(c); return f->NumTensors(); }
+const char* mg_tensor_name(const mg_ctx* c, int i) { return c && c->layered ? c->layered->TensorName(i) : nullptr; }
+int mg_tensor_shape(const mg_ctx* c, const char* name, int64_t* shape) { CTX(c); return f->TensorShape(name, shape); }
+int mg_set_tensor_bf16(mg_ctx* c, const char* name, const uint16_t* data, size_t n) { CTX(c); return f->SetTensor(name, data, n); }
+int mg_prefill_hidden(mg_ctx* c, const int* tokens, int nTokens, int pos0, int layerEnd, float* out) {
+    CTX(c); return f->PrefillHidden(tokens, nTokens, pos0, layerEnd, out);
+}
+
+}  // extern "C"

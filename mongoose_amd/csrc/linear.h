@@ -1,0 +1,136 @@
+// linear.h -- products with bf16 weights: matrix-vector for the decode step (fp32 vector), MFMA GEMM for many rows
+// (bf16 or fp32 activations), both with their prologues and epilogues (linear.hip).
+//
+// A weight matrix is row-major bf16 with rows of ld elements, ld a multiple of 64; the elements past the real row
+// length are zero, and activation rows have the same padding (finite values there), so no kernel has a K tail.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stddef.h>
+#include "activations.h"
+#include "row_ops.h"
+
+namespace mg {
+
+__host__ __device__ inline int pad_to(int v, int m) { return (v + m - 1) / m * m; }
+
+struct Bf16Mat {
+    const unsigned short* w = nullptr;
+    int rows = 0, cols = 0, ld = 0;
+    size_t bytes() const { return (size_t)rows * ld * 2; }
+};
+
+// How a kernel gets its input vector v[n]: src itself, or, with a gain, v = src / rms(src) * gain; then, with a
+// second operand, v = part + coef * v (the weighted sum over earlier layers' outputs, its last term being this one);
+// then optionally a second norm.  One workgroup also stores the intermediate results where asked.
+struct VecInput {
+    const float* src = nullptr;
+    int n = 0;
+    const float* gain = nullptr;
+    float eps = 0.f;
+    float* normOut = nullptr;        // v after the first norm
+    const float* part = nullptr;
+    float coef = 0.f;
+    float* out = nullptr;            // v after the sum
+    const float* gain2 = nullptr;
+};
+
+enum MvEpilogue { MV_STORE = 0, MV_RESID = 1, MV_ARGMAX = 2 };
+
+struct MvBf16 {
+    VecInput in;
+    Bf16Mat w;
+    int epi = MV_STORE;
+    float* out = nullptr;
+    ActParam act{};                  // applied to rows >= actFrom
+    int actFrom = 0;
+    const float* resid = nullptr;    // MV_RESID: out = alpha * resid + v
+    float alpha = 0.f;
+    float* amaxVal = nullptr;        // MV_ARGMAX: one (max, index) per workgroup
+    int* amaxIdx = nullptr;
+    // mixture of experts, expert s of the chosen ones in grid row s: w is expert 0, expert e lies expertStride
+    // elements further; out is [top, w.rows]
+    const float* routerLogits = nullptr;
+    int experts = 0, top = 0;
+    size_t expertStride = 0;
+};
+hipError_t launch_matvec_bf16(const MvBf16& p, int* gridOut, hipStream_t s);
+
+// Second half of the experts: out = alpha * resid + sum_s weight_s W_e(s) hid_s (+ Wshared hidShared).
+struct MvMoeDown {
+    const float* routerLogits = nullptr;
+    int experts = 0, top = 0;
+    const float* hid = nullptr;      // [top, ff]
+    int ff = 0;
+    Bf16Mat down;                    // expert 0
+    size_t expertStride = 0;
+    const float* hidShared = nullptr;
+    int ffShared = 0;
+    Bf16Mat downShared;              // rows 0: none
+    const float* resid = nullptr;
+    float alpha = 0.f;
+    float* out = nullptr;
+};
+hipError_t launch_moe_down(const MvMoeDown& p, hipStream_t s);
+
+// Block-diagonal product, one block of weights a head: out[t, h, m] = sum_k W[h, m, k] in[t, h, k].  The input is a
+// slice of a row (src + t * rowStride + h * headStride), or, with splits > 0, merged from the partial results of a
+// split attention: partials [t, h, split]: acc [.., accLd], running maximum, sum.
+struct HeadMv {
+    const float* src = nullptr;
+    int rowStride = 0, headStride = 0;
+    int K = 0;                       // real length of a head's slice
+    const float* pacc = nullptr;
+    const float* pm = nullptr;
+    const float* pl = nullptr;
+    int splits = 0, accLd = 0;
+    const unsigned short* w = nullptr;   // [heads, rows, ld]
+    int heads = 0, rows = 0, ld = 0;
+    float* out = nullptr;            // [T, heads, rows]  (fp32), or
+    void* outAct = nullptr;          // the same as activations (bf16 or fp32) with rows of ldAct
+    int actF32 = 0, ldAct = 0;
+    int T = 1;
+    SideJobs side;                   // further workgroups of the launch (T = 1)
+};
+hipError_t launch_head_matvec(const HeadMv& p, hipStream_t s);
+
+enum GemmMode {
+    GEMM_F32 = 0,      // out[m, n] = acc
+    GEMM_ACT = 1,      // outAct[m, n] = act(acc)
+    GEMM_RESID = 2,    // out[m, n] = alpha * res[m, n] + acc
+    GEMM_SPLIT = 3,    // n < nSplit: out[m, n] = acc; else outAct[m, n - nSplit] = act(acc)
+    GEMM_ROPE = 4,     // outAct[m, n] with the pairs (2i, 2i+1) behind column ropeOff of every head turned
+    GEMM_SCATTER = 5,  // out[perm[m], n] = rowScale[perm[m]] * acc
+};
+struct Gemm {
+    const void* A = nullptr;         // activations [M, lda], bf16 (f32 = 0) or fp32
+    int f32 = 0;
+    int lda = 0, M = 0;
+    const void* W = nullptr;         // bf16 [N, ldw]; with wF32 (f32 only) fp32
+    int wF32 = 0;
+    int ldw = 0, N = 0, K = 0;       // K a multiple of 64
+    int mode = GEMM_F32;
+    float* out = nullptr;
+    int ldc = 0;
+    void* outAct = nullptr;
+    int ldo = 0;
+    ActParam act{};
+    const float* res = nullptr;
+    int ldres = 0;
+    float alpha = 0.f;
+    int nSplit = 0;
+    int headW = 0, ropeOff = 0, ropeDims = 0, pos0 = 0;
+    const float* cosTab = nullptr;   // [pos, ropeDims / 2]
+    const float* sinTab = nullptr;
+    // experts: row tiles {expert, first sorted row, rows, -}; sorted row r is entry perm[r] (token * permDiv + choice)
+    const int4* tiles = nullptr;
+    const int* nTiles = nullptr;
+    int maxTiles = 0;
+    const int* perm = nullptr;
+    int permDiv = 0;                 // > 0: A row = perm[r] / permDiv; 0: A row = r
+    const float* rowScale = nullptr;
+    size_t expertStride = 0;
+};
+constexpr int MOE_TILE_ROWS = 64;    // rows of a tile of the experts' products
+hipError_t launch_gemm_bf16w(const Gemm& g, hipStream_t s);
+
+}  // namespace mg

@@ -1,0 +1,531 @@
+// linear.hip -- products with bf16 weights (linear.h).
+//
+// Decode: out[N] = W[N, K] v with v in fp32.  A wave owns NR rows at a time; a lane takes 8 consecutive weights (16
+// bytes) of every 512, the vector lies in LDS.  The first loads of the weights go out before the vector is staged, so
+// that the two round trips overlap; a ring of DEP chunk loads stays in flight.
+//
+// Many rows: Y[M, N] = A[M, K] W[N, K]^T on the matrix cores, v_mfma_f32_32x32x16_bf16 (bf16 activations) or
+// v_mfma_f32_32x32x2_f32 (fp32 activations; the bf16 weights widened).  W is the first operand: a lane then ends up
+// with four consecutive n of one row m, which is what the epilogues (vector stores, RoPE pairs) want.
+#include "linear.h"
+#include "bf16_util.h"
+#include "device_util.h"
+#include "side_jobs.h"
+#include "vec_input.h"
+
+#include <algorithm>
+
+namespace mg {
+
+// ---------------------------------------------------------------------------
+// decode
+// ---------------------------------------------------------------------------
+__device__ __forceinline__ float dot8(uint4 w, const float4* lo, const float4* hi, int c8, float acc) {
+    const float4 a = lo[c8], b = hi[c8];
+    acc = fmaf(bf16_lo(w.x), a.x, acc); acc = fmaf(bf16_hi(w.x), a.y, acc);
+    acc = fmaf(bf16_lo(w.y), a.z, acc); acc = fmaf(bf16_hi(w.y), a.w, acc);
+    acc = fmaf(bf16_lo(w.z), b.x, acc); acc = fmaf(bf16_hi(w.z), b.y, acc);
+    acc = fmaf(bf16_lo(w.w), b.z, acc); acc = fmaf(bf16_hi(w.w), b.w, acc);
+    return acc;
+}
+
+template <int NR, int DEP>
+__global__ __launch_bounds__(WG) void matvec_bf16_kernel(MvBf16 p) {
+    extern __shared__ __attribute__((aligned(16))) float act[];
+    __shared__ float red[4];
+    __shared__ int ids[MAX_TOP];
+    __shared__ float wts[MAX_TOP];
+    __shared__ float bv[4];
+    __shared__ int bi[4];
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int Kp = p.w.ld, N = p.w.rows;
+    const int nch = (Kp + 511) >> 9;
+    const int groups = (N + NR - 1) / NR;
+    const int stride = gridDim.x * 4;
+    const unsigned short* W = p.w.w;
+    if (p.top) {
+        if (wave == 0) choose_experts(p.routerLogits, p.experts, p.top, ids, wts);
+        __syncthreads();
+        W += (size_t)ids[blockIdx.y] * p.expertStride;
+        p.out += (size_t)blockIdx.y * N;
+    }
+    // load cursor (lg, lc) and use cursor (g, c) over (row group, chunk)
+    int g = blockIdx.x * 4 + wave, lg = g, lc = 0;
+    uint4 ring[DEP][NR];
+    auto issue = [&](uint4 (&slot)[NR]) __attribute__((always_inline)) {
+        const int col = lc * 512 + lane * 8;
+#pragma unroll
+        for (int r = 0; r < NR; r++) {
+            const int row = min(lg * NR + r, N - 1);
+            slot[r] = lg < groups && col < Kp ? *reinterpret_cast<const uint4*>(W + (size_t)row * Kp + col) : make_uint4(0, 0, 0, 0);
+        }
+        if (++lc == nch) { lc = 0; lg += stride; }
+    };
+#pragma unroll
+    for (int d = 0; d < DEP; d++) issue(ring[d]);
+    stage_vector(p.in, act, Kp, blockIdx.x == 0 && blockIdx.y == 0, red);
+    const float4* lo = reinterpret_cast<const float4*>(act);
+    const float4* hi = lo + (Kp >> 3);
+    const int last8 = (Kp >> 3) - 1;
+    float best = -INFINITY;
+    int besti = INT_MAX;
+    float acc[NR];
+#pragma unroll
+    for (int r = 0; r < NR; r++) acc[r] = 0.f;
+    int c = 0;
+    while (g < groups) {
+#pragma unroll
+        for (int d = 0; d < DEP; d++) {
+            if (g >= groups) break;
+            const int c8 = min(c * 64 + lane, last8);        // (lanes past the row multiply zero weights)
+#pragma unroll
+            for (int r = 0; r < NR; r++) acc[r] = dot8(ring[d][r], lo, hi, c8, acc[r]);
+            issue(ring[d]);
+            if (++c == nch) {
+                c = 0;
+#pragma unroll
+                for (int r = 0; r < NR; r++) {
+                    const int row = g * NR + r;
+                    float v = wave_sum(acc[r]);
+                    acc[r] = 0.f;
+                    if (row < N) {
+                        if (p.act.kind && row >= p.actFrom) v = apply_act(v, p.act);
+                        if (p.epi == MV_RESID) v = fmaf(p.alpha, p.resid[row], v);
+                        if (lane == 0) p.out[row] = v;
+                        if (v > best) { best = v; besti = row; }
+                    }
+                }
+                g += stride;
+            }
+        }
+    }
+    if (p.epi == MV_ARGMAX) {
+        if (lane == 0) { bv[wave] = best; bi[wave] = besti; }
+        __syncthreads();
+        if (threadIdx.x == 0) {
+            for (int w = 1; w < 4; w++) argmax_pick(best, besti, bv[w], bi[w]);
+            p.amaxVal[blockIdx.x] = best;
+            p.amaxIdx[blockIdx.x] = besti;
+        }
+    }
+}
+
+template <int NR, int DEP>
+static hipError_t run_matvec(const MvBf16& p, int grid, size_t lds, hipStream_t s) {
+    auto k = matvec_bf16_kernel<NR, DEP>;
+    if (lds > (48u << 10)) {
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(k, dim3(grid, p.top ? p.top : 1), dim3(WG), lds, s, p);
+    return hipGetLastError();
+}
+hipError_t launch_matvec_bf16(const MvBf16& p, int* gridOut, hipStream_t s) {
+    if (p.w.rows <= 0 || p.w.ld <= 0 || p.w.ld % 64 || p.in.n > p.w.ld || p.experts > MAX_EXPERTS || p.top > MAX_TOP || p.top > p.experts)
+        return hipErrorInvalidValue;
+    const size_t lds = (size_t)p.w.ld * 4;
+    if (lds > (144u << 10)) return hipErrorInvalidValue;
+    const int rows = p.w.rows * (p.top ? p.top : 1);
+    const int nr = rows >= 16384 ? 4 : rows >= 6144 ? 2 : 1;
+    const int groups = (p.w.rows + nr - 1) / nr;
+    int grid = (groups + 3) / 4;
+    // workgroups that stay for several row groups share one staging of the vector
+    const int cap = p.top ? std::max(1, 2048 / p.top) : 2048;
+    if (grid > cap) grid = cap;
+    if (gridOut) *gridOut = grid;
+    if (nr == 4) return run_matvec<4, 2>(p, grid, lds, s);
+    if (nr == 2) return run_matvec<2, 4>(p, grid, lds, s);
+    return run_matvec<1, 4>(p, grid, lds, s);
+}
+
+// One wave a row of the output: the chosen experts' rows one after the other, then the shared expert's.
+__global__ __launch_bounds__(WG) void moe_down_kernel(MvMoeDown p) {
+    extern __shared__ __attribute__((aligned(16))) float act[];       // [top][ld], [ldShared]
+    __shared__ int ids[MAX_TOP];
+    __shared__ float wts[MAX_TOP];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int Kp = p.down.ld, Ks = p.downShared.rows ? p.downShared.ld : 0;
+    if (wave == 0) choose_experts(p.routerLogits, p.experts, p.top, ids, wts);
+    __syncthreads();
+    for (int s = 0; s < p.top; s++)
+        for (int i = threadIdx.x; i < Kp; i += WG)
+            act[s * Kp + plane_index(i, Kp >> 3)] = i < p.ff ? wts[s] * p.hid[(size_t)s * p.ff + i] : 0.f;
+    for (int i = threadIdx.x; i < Ks; i += WG)
+        act[p.top * Kp + plane_index(i, Ks >> 3)] = i < p.ffShared ? p.hidShared[i] : 0.f;
+    __syncthreads();
+    const int row = blockIdx.x * 4 + wave;
+    if (row >= p.down.rows) return;
+    float acc = 0.f;
+    for (int s = 0; s <= p.top; s++) {
+        const bool sh = s == p.top;
+        const int ld = sh ? Ks : Kp;
+        if (!ld) break;
+        const unsigned short* w = sh ? p.downShared.w + (size_t)row * ld
+                                     : p.down.w + (size_t)__builtin_amdgcn_readfirstlane(ids[s]) * p.expertStride + (size_t)row * ld;
+        const float4* lo = reinterpret_cast<const float4*>(act + s * Kp);
+        const float4* hi = lo + (ld >> 3);
+#pragma unroll 4
+        for (int c8 = lane; c8 < ld >> 3; c8 += 64) acc = dot8(*reinterpret_cast<const uint4*>(w + c8 * 8), lo, hi, c8, acc);
+    }
+    acc = wave_sum(acc);
+    if (lane == 0) p.out[row] = fmaf(p.alpha, p.resid[row], acc);
+}
+hipError_t launch_moe_down(const MvMoeDown& p, hipStream_t s) {
+    if (p.top < 1 || p.top > MAX_TOP || p.experts > MAX_EXPERTS || p.down.ld % 64 || p.ff > p.down.ld) return hipErrorInvalidValue;
+    const size_t lds = ((size_t)p.top * p.down.ld + (p.downShared.rows ? p.downShared.ld : 0)) * 4;
+    if (lds > (144u << 10)) return hipErrorInvalidValue;
+    if (lds > (48u << 10)) {
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(moe_down_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(moe_down_kernel, dim3((p.down.rows + 3) / 4), dim3(WG), lds, s, p);
+    return hipGetLastError();
+}
+
+// Rows of one head: 2^lprLog2 lanes share a row (a row of ld weights is ld / 8 lane loads).
+__global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG, int lprLog2) {
+    extern __shared__ __attribute__((aligned(16))) float act[];
+    __shared__ float red[4];
+    const int h = blockIdx.y, t = blockIdx.z;
+    if (h >= p.heads) {
+        const int wg = (h - p.heads) * gridDim.x + blockIdx.x;
+        if (wg < p.side.wgs()) run_side_job(p.side, wg, red);
+        return;
+    }
+    const int ld = p.ld, nc8 = ld >> 3;
+    if (p.splits) {
+        // out = sum_s e^(m_s - M) acc_s / sum_s e^(m_s - M) l_s; a split that saw no key has m = -inf
+        const size_t b = ((size_t)t * p.heads + h) * p.splits;
+        float M = -INFINITY;
+        for (int s = 0; s < p.splits; s++) M = fmaxf(M, p.pm[b + s]);
+        float L = 0.f;
+        for (int s = 0; s < p.splits; s++) L += p.pm[b + s] == -INFINITY ? 0.f : expf(p.pm[b + s] - M) * p.pl[b + s];
+        const float inv = 1.0f / L;
+        for (int i = threadIdx.x; i < ld; i += WG) {
+            float v = 0.f;
+            if (i < p.K)
+                for (int s = 0; s < p.splits; s++) {
+                    const float m = p.pm[b + s];
+                    if (m != -INFINITY) v = fmaf(expf(m - M), p.pacc[(b + s) * p.accLd + i], v);
+                }
+            act[plane_index(i, nc8)] = v * inv;
+        }
+    } else {
+        const float* src = p.src + (size_t)t * p.rowStride + (size_t)h * p.headStride;
+        for (int i = threadIdx.x; i < ld; i += WG) act[plane_index(i, nc8)] = i < p.K ? src[i] : 0.f;
+    }
+    __syncthreads();
+    const float4* lo = reinterpret_cast<const float4*>(act);
+    const float4* hi = lo + nc8;
+    const int lpr = 1 << lprLog2, sub = threadIdx.x & (lpr - 1), slot = threadIdx.x >> lprLog2, slots = WG >> lprLog2;
+    const int r0 = blockIdx.x * rowsPerWG, r1 = min(r0 + rowsPerWG, p.rows);
+    for (int rb = r0; rb < r1; rb += slots) {
+        const int row = rb + slot;
+        float acc = 0.f;
+        if (row < r1) {
+            const unsigned short* w = p.w + ((size_t)h * p.rows + row) * ld;
+#pragma unroll 2
+            for (int c8 = sub; c8 < nc8; c8 += lpr) acc = dot8(*reinterpret_cast<const uint4*>(w + c8 * 8), lo, hi, c8, acc);
+        }
+        for (int o = lpr >> 1; o > 0; o >>= 1) acc += __shfl_xor(acc, o, 64);
+        if (sub == 0 && row < r1) {
+            if (p.out) p.out[((size_t)t * p.heads + h) * p.rows + row] = acc;
+            if (p.outAct) {
+                const size_t o = (size_t)t * p.ldAct + (size_t)h * p.rows + row;
+                if (p.actF32) static_cast<float*>(p.outAct)[o] = acc;
+                else store_act(static_cast<bf16_t*>(p.outAct) + o, acc);
+            }
+        }
+    }
+}
+hipError_t launch_head_matvec(const HeadMv& p, hipStream_t s) {
+    if (p.T < 1) return hipSuccess;
+    if (p.side.wgs() && p.T != 1) return hipErrorInvalidValue;
+    if (p.ld % 64 || p.K > p.ld || p.rows < 1 || (size_t)p.ld * 4 > (48u << 10)) return hipErrorInvalidValue;
+    int lprLog2 = 3;
+    while (lprLog2 < 6 && (8 << lprLog2) < p.ld) lprLog2++;
+    // enough workgroups for the chip at one row t; a workgroup's staging is worth some rows
+    const int slots = WG >> lprLog2;
+    int rowsPerWG = pad_to((p.rows * p.heads * p.T + 511) / 512, slots);
+    if (rowsPerWG < slots) rowsPerWG = slots;
+    if (rowsPerWG > pad_to(p.rows, slots)) rowsPerWG = pad_to(p.rows, slots);
+    for (int t0 = 0; t0 < p.T; t0 += 32768) {
+        HeadMv q = p;
+        q.T = std::min(p.T - t0, 32768);
+        if (q.src) q.src += (size_t)t0 * p.rowStride;
+        const size_t b = (size_t)t0 * p.heads * p.splits;
+        if (q.splits) { q.pacc += b * p.accLd; q.pm += b; q.pl += b; }
+        if (q.out) q.out += (size_t)t0 * p.heads * p.rows;
+        if (q.outAct) q.outAct = static_cast<char*>(p.outAct) + (size_t)t0 * p.ldAct * (p.actF32 ? 4 : 2);
+        const int gx = (p.rows + rowsPerWG - 1) / rowsPerWG;
+        hipLaunchKernelGGL(head_matvec_kernel, dim3(gx, p.heads + (p.side.wgs() + gx - 1) / gx, q.T), dim3(WG), (size_t)p.ld * 4, s, q, rowsPerWG, lprLog2);
+        hipError_t e = hipGetLastError();
+        if (e != hipSuccess) return e;
+    }
+    return hipSuccess;
+}
+
+// ---------------------------------------------------------------------------
+// many rows
+// ---------------------------------------------------------------------------
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+
+// Four consecutive columns n .. n+3 of row m (sorted row r of an expert tile; m is where it goes).
+template <typename AT>
+__device__ __forceinline__ void gemm_store4(const Gemm& g, int m, int n, float4 v) {
+    const int left = g.N - n;
+    float e[4] = {v.x, v.y, v.z, v.w};
+    if (g.mode == GEMM_SPLIT) {
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            if (i >= left) break;
+            if (n + i < g.nSplit) g.out[(size_t)m * g.ldc + n + i] = e[i];
+            else store_act(static_cast<AT*>(g.outAct) + (size_t)m * g.ldo + (n + i - g.nSplit), apply_act(e[i], g.act));
+        }
+        return;
+    }
+    if (g.mode == GEMM_ROPE) {
+        const int hc = n % g.headW - g.ropeOff;               // headW and ropeOff are multiples of 32
+        if (hc >= 0 && hc < g.ropeDims) {
+            const size_t row = (size_t)(g.pos0 + m) * (g.ropeDims >> 1);
+#pragma unroll
+            for (int i = 0; i < 2; i++) {
+                if (hc + 2 * i >= g.ropeDims) break;
+                const float c = g.cosTab[row + (hc >> 1) + i], s = g.sinTab[row + (hc >> 1) + i];
+                const float a = e[2 * i], b = e[2 * i + 1];
+                e[2 * i] = a * c - b * s;
+                e[2 * i + 1] = b * c + a * s;
+            }
+        }
+    }
+    if (g.mode == GEMM_ACT || g.mode == GEMM_ROPE) {
+        if (g.mode == GEMM_ACT && g.act.kind)
+#pragma unroll
+            for (int i = 0; i < 4; i++) e[i] = apply_act(e[i], g.act);
+        AT* o = static_cast<AT*>(g.outAct) + (size_t)m * g.ldo + n;
+        if (left >= 4) {
+            if (sizeof(AT) == 2) *reinterpret_cast<uint2*>(o) = make_uint2(bf16_pack(e[0], e[1]), bf16_pack(e[2], e[3]));
+            else *reinterpret_cast<float4*>(o) = make_float4(e[0], e[1], e[2], e[3]);
+        } else {
+#pragma unroll
+            for (int i = 0; i < 4; i++)
+                if (i < left) store_act(o + i, e[i]);
+        }
+        return;
+    }
+    float* o = g.out + (size_t)m * g.ldc + n;
+    const float* r = g.mode == GEMM_RESID ? g.res + (size_t)m * g.ldres + n : nullptr;
+    const float sc = g.mode == GEMM_SCATTER ? g.rowScale[m] : 1.0f;
+    if (left >= 4 && ((g.ldc | g.ldres) & 3) == 0) {
+        if (r) {
+            const float4 x = *reinterpret_cast<const float4*>(r);
+            e[0] = fmaf(g.alpha, x.x, e[0]); e[1] = fmaf(g.alpha, x.y, e[1]);
+            e[2] = fmaf(g.alpha, x.z, e[2]); e[3] = fmaf(g.alpha, x.w, e[3]);
+        }
+        *reinterpret_cast<float4*>(o) = make_float4(e[0] * sc, e[1] * sc, e[2] * sc, e[3] * sc);
+    } else {
+#pragma unroll
+        for (int i = 0; i < 4; i++)
+            if (i < left) o[i] = (r ? fmaf(g.alpha, r[i], e[i]) : e[i]) * sc;
+    }
+}
+
+// Which rows and columns a workgroup computes: row tile rows [row0, row0 + rows), column tile at n0.
+struct TileAt { int row0, rows, n0, expert; };
+template <int BM, int BN>
+__device__ __forceinline__ bool find_tile(const Gemm& g, TileAt& t) {
+    const int tilesN = (g.N + BN - 1) / BN;
+    const int total = g.tiles ? *g.nTiles * tilesN : (int)gridDim.x;
+    int id = blockIdx.x;
+    if (id >= total) return false;
+    // workgroup i runs on XCD i & 7: neighbouring tiles, which share operands, go to one XCD
+    const int full = total & ~7;
+    if (id < full) id = (id & 7) * (full >> 3) + (id >> 3);
+    const int tilesM = total / tilesN;
+    // bands of 8 column tiles, row tiles inner: a band's weights stay in the L2 while the rows pass
+    const int band = 8, perBand = band * tilesM;
+    const int b = id / perBand, w = min(band, tilesN - b * band);
+    const int in = id - b * perBand;
+    const int nt = b * band + in % w, mt = in / w;
+    t.n0 = nt * BN;
+    if (g.tiles) {
+        const int4 q = g.tiles[mt];
+        t.expert = q.x; t.row0 = q.y; t.rows = q.z;
+    } else {
+        t.expert = 0; t.row0 = mt * BM; t.rows = min(BM, g.M - t.row0);
+    }
+    return true;
+}
+
+// bf16 activations.  BM rows x BN columns, 4 waves as 2 x 2, K in steps of 64 through two LDS buffers filled by direct
+// global -> LDS loads.  LDS rows are 128 bytes (64 k); the 16-byte piece q of row r lies at q ^ (r & 7).
+template <int BM, int BN>
+__global__ __launch_bounds__(256) void gemm_bf16_kernel(Gemm g) {
+    constexpr int WM = BM / 64, WN = BN / 64;            // 32 x 32 blocks a wave: rows, columns
+    constexpr int ABYTES = BM * 128, BUF = (BM + BN) * 128;
+    constexpr int LOADS = (BM + BN) / 32;                // wave-loads (8 rows of 128 bytes) a wave issues a step
+    extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
+    TileAt tl;
+    if (!find_tile<BM, BN>(g, tl)) return;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const bf16_t* A = static_cast<const bf16_t*>(g.A);
+    const bf16_t* W = static_cast<const bf16_t*>(g.W) + (size_t)tl.expert * g.expertStride;
+    // this wave's loads: load i brings LDS rows 8 * (wave * LOADS + i) .. + 7 (A rows first, then W rows)
+    const bf16_t* src[LOADS];
+#pragma unroll
+    for (int i = 0; i < LOADS; i++) {
+        const int r = 8 * (wave * LOADS + i) + (lane >> 3);
+        const int piece = (lane & 7) ^ (r & 7);
+        if (r < BM) {
+            const int sr = tl.row0 + min(r, tl.rows - 1);
+            const int ar = g.permDiv ? g.perm[sr] / g.permDiv : sr;
+            src[i] = A + (size_t)ar * g.lda + piece * 8;
+        } else {
+            src[i] = W + (size_t)min(tl.n0 + r - BM, g.N - 1) * g.ldw + piece * 8;
+        }
+    }
+    auto issue = [&](int step, int buf) __attribute__((always_inline)) {
+        unsigned char* dst = lds + buf * BUF + wave * LOADS * 1024;
+#pragma unroll
+        for (int i = 0; i < LOADS; i++) {
+            const bf16_t* from = src[i] + step * 64;     // (the builtin's operands must not have a dependent type)
+            __builtin_amdgcn_global_load_lds(from, reinterpret_cast<int4*>(dst + i * 1024), 16, 0, 0);
+        }
+    };
+    f32x16 acc[WN][WM];
+#pragma unroll
+    for (int a = 0; a < WN; a++)
+#pragma unroll
+        for (int b = 0; b < WM; b++)
+#pragma unroll
+            for (int e = 0; e < 16; e++) acc[a][b][e] = 0.f;
+    const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * (BN / 2);
+    const int fr = lane & 31, fh = lane >> 5;
+    const int steps = g.K >> 6;
+    issue(0, 0);
+    for (int st = 0; st < steps; st++) {
+        asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        if (st + 1 < steps) issue(st + 1, (st + 1) & 1);
+        const unsigned char* base = lds + (st & 1) * BUF;
+#pragma unroll
+        for (int ks = 0; ks < 4; ks++) {
+            const int piece = 2 * ks + fh;
+            bf16x8 fa[WM], fw[WN];
+#pragma unroll
+            for (int b = 0; b < WM; b++) {
+                const int r = wm + 32 * b + fr;
+                fa[b] = *reinterpret_cast<const bf16x8*>(base + r * 128 + ((piece ^ (r & 7)) << 4));
+            }
+#pragma unroll
+            for (int a = 0; a < WN; a++) {
+                const int r = wn + 32 * a + fr;
+                fw[a] = *reinterpret_cast<const bf16x8*>(base + ABYTES + r * 128 + ((piece ^ (r & 7)) << 4));
+            }
+#pragma unroll
+            for (int a = 0; a < WN; a++)
+#pragma unroll
+                for (int b = 0; b < WM; b++) acc[a][b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fw[a], fa[b], acc[a][b], 0, 0, 0);
+        }
+    }
+    // lane: row m = wm + 32 b + lane % 32; columns n = 8 q + 4 (lane / 32) + 0..3 of the 32-column block
+#pragma unroll
+    for (int b = 0; b < WM; b++) {
+        const int r = wm + 32 * b + fr;
+        if (r >= tl.rows) continue;
+        const int sr = tl.row0 + r;
+        const int m = g.mode == GEMM_SCATTER ? g.perm[sr] : sr;
+#pragma unroll
+        for (int a = 0; a < WN; a++)
+#pragma unroll
+            for (int q = 0; q < 4; q++) {
+                const int n = tl.n0 + wn + 32 * a + 8 * q + 4 * fh;
+                if (n < g.N) gemm_store4<bf16_t>(g, m, n, make_float4(acc[a][b][4 * q], acc[a][b][4 * q + 1], acc[a][b][4 * q + 2], acc[a][b][4 * q + 3]));
+            }
+    }
+}
+
+// fp32 activations: 64 x 64, 4 waves as 2 x 2 of one 32 x 32 block, K in steps of 32.
+template <typename WT>
+__global__ __launch_bounds__(256) void gemm_f32_kernel(Gemm g) {
+    constexpr int LDT = 36;                              // row stride (floats): 16-byte aligned rows
+    __shared__ __attribute__((aligned(16))) float As[64 * LDT];
+    __shared__ __attribute__((aligned(16))) float Ws[64 * LDT];
+    TileAt tl;
+    if (!find_tile<64, 64>(g, tl)) return;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const float* A = static_cast<const float*>(g.A);
+    const WT* W = static_cast<const WT*>(g.W) + (size_t)tl.expert * g.expertStride;
+    // thread: LDS row tid / 4, k 8 (tid % 4) .. + 7 of both tiles
+    const int lr = threadIdx.x >> 2, lk = (threadIdx.x & 3) * 8;
+    const int sr = tl.row0 + min(lr, tl.rows - 1);
+    const float* ap = A + (size_t)(g.permDiv ? g.perm[sr] / g.permDiv : sr) * g.lda + lk;
+    const WT* wp = W + (size_t)min(tl.n0 + lr, g.N - 1) * g.ldw + lk;
+    f32x16 acc;
+#pragma unroll
+    for (int e = 0; e < 16; e++) acc[e] = 0.f;
+    const int wm = (wave & 1) * 32, wn = (wave >> 1) * 32, fr = lane & 31, fh = lane >> 5;
+    for (int k0 = 0; k0 < g.K; k0 += 32) {
+        const float4 a0 = *reinterpret_cast<const float4*>(ap + k0), a1 = *reinterpret_cast<const float4*>(ap + k0 + 4);
+        float w[8];
+        if (sizeof(WT) == 2) {
+            const uint4 u = *reinterpret_cast<const uint4*>(wp + k0);
+            const unsigned x[4] = {u.x, u.y, u.z, u.w};
+#pragma unroll
+            for (int i = 0; i < 4; i++) { w[2 * i] = bf16_lo(x[i]); w[2 * i + 1] = bf16_hi(x[i]); }
+        } else {
+            const float4 u0 = *reinterpret_cast<const float4*>(wp + k0), u1 = *reinterpret_cast<const float4*>(wp + k0 + 4);
+            w[0] = u0.x; w[1] = u0.y; w[2] = u0.z; w[3] = u0.w; w[4] = u1.x; w[5] = u1.y; w[6] = u1.z; w[7] = u1.w;
+        }
+        __syncthreads();
+        *reinterpret_cast<float4*>(As + lr * LDT + lk) = a0;
+        *reinterpret_cast<float4*>(As + lr * LDT + lk + 4) = a1;
+        *reinterpret_cast<float4*>(Ws + lr * LDT + lk) = make_float4(w[0], w[1], w[2], w[3]);
+        *reinterpret_cast<float4*>(Ws + lr * LDT + lk + 4) = make_float4(w[4], w[5], w[6], w[7]);
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < 32; k += 2)
+            acc = __builtin_amdgcn_mfma_f32_32x32x2f32(Ws[(wn + fr) * LDT + k + fh], As[(wm + fr) * LDT + k + fh], acc, 0, 0, 0);
+    }
+    const int r = wm + fr;
+    if (r >= tl.rows) return;
+    const int s2 = tl.row0 + r;
+    const int m = g.mode == GEMM_SCATTER ? g.perm[s2] : s2;
+#pragma unroll
+    for (int q = 0; q < 4; q++) {
+        const int n = tl.n0 + wn + 8 * q + 4 * fh;
+        if (n < g.N) gemm_store4<float>(g, m, n, make_float4(acc[4 * q], acc[4 * q + 1], acc[4 * q + 2], acc[4 * q + 3]));
+    }
+}
+
+template <int BM, int BN>
+static hipError_t run_gemm_bf16(const Gemm& g, hipStream_t s) {
+    const size_t lds = (size_t)(BM + BN) * 128 * 2;
+    auto k = gemm_bf16_kernel<BM, BN>;
+    if (lds > (48u << 10)) {
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    const int tilesN = (g.N + BN - 1) / BN;
+    const int tilesM = g.tiles ? g.maxTiles : (g.M + BM - 1) / BM;
+    hipLaunchKernelGGL(k, dim3((unsigned)(tilesN * tilesM)), dim3(256), lds, s, g);
+    return hipGetLastError();
+}
+
+hipError_t launch_gemm_bf16w(const Gemm& g, hipStream_t s) {
+    if (g.M <= 0 || g.N <= 0) return hipSuccess;
+    if (g.K <= 0 || g.K % 64 || g.lda < g.K || g.ldw < g.K || g.lda % 8 || g.ldw % 8) return hipErrorInvalidValue;
+    if (g.f32) {
+        const unsigned grid = (unsigned)((g.N + 63) / 64) * (unsigned)(g.tiles ? g.maxTiles : (g.M + 63) / 64);
+        if (g.wF32) hipLaunchKernelGGL(gemm_f32_kernel<float>, dim3(grid), dim3(256), 0, s, g);
+        else hipLaunchKernelGGL(gemm_f32_kernel<bf16_t>, dim3(grid), dim3(256), 0, s, g);
+        return hipGetLastError();
+    }
+    if (g.wF32) return hipErrorInvalidValue;
+    if (g.tiles) return g.N >= 512 ? run_gemm_bf16<MOE_TILE_ROWS, 128>(g, s) : run_gemm_bf16<MOE_TILE_ROWS, 64>(g, s);
+    const long big = (long)((g.M + 127) / 128) * ((g.N + 127) / 128);
+    if (big >= 192) return run_gemm_bf16<128, 128>(g, s);
+    return run_gemm_bf16<64, 64>(g, s);
+}
+
+}  // namespace mg

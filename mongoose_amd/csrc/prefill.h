@@ -23,7 +23,7 @@ size_t prefill_kv_split_bytes(int rows, int kvDim);
 hipError_t launch_prefill_attention(const float* q, const void* Kc, const void* Vc, int kvHalf, void* kvSplit, float* out,
                                     void* splitHi, void* splitLo, int T, int pos0, int rowLimit, int dim, int kvDim, int nHeads,
                                     int nKVHeads, int headDim, hipStream_t s);
-// Embedding rows of T tokens: kind 0 = Q8 row * scale, 1 = fp16 table, 2 = fp32 table, 3 = Q4_0 split-layout row.
+// Embedding rows of T tokens: kind 0 = Q8 row * scale, 1 = fp16 table, 2 = fp32 table, 3 = Q4_0 split-layout row, 4 = bf16 table.
 hipError_t launch_embed_rows(int kind, const void* table, const float* scales, const int* tokens, float* x, int T, int dim,
                              int vocab, hipStream_t s);
 // One launch: for each of up to three weight matrices, Y[T,N] (+)= (Ahi + Alo)[T,K] . W[N,K]^T * scales[n] (+ bias[n]).

@@ -1,0 +1,96 @@
+// row_ops.h -- row-wise launches of the multi-token path: norms with the depth average, expert routing; and the
+// small side jobs of the decode step that ride along with another launch.
+#pragma once
+#include <hip/hip_runtime.h>
+#include <stddef.h>
+#include "kernels.h"
+
+namespace mg {
+
+// Latent key/value rows of one layer: position p at cache + p * stride, latent (rank values, zero up to rankPad),
+// then the rotated key part (rot values).  bf16 or fp32.
+struct LatentCache {
+    void* rows = nullptr;
+    int f32 = 0;
+    int rank = 0, rankPad = 0, rot = 0, stride = 0;
+    int ropeDims = 0;
+    const float* cosTab = nullptr;   // [pos, ropeDims / 2]
+    const float* sinTab = nullptr;
+};
+
+// Side jobs of a decode launch: workgroup 0 .. wgs() - 1 of them.
+struct SideJobs {
+    const StepState* state = nullptr;
+    // cache row of the current position from z = [latent | rotated part] (raw projection)
+    LatentCache cache;
+    const float* z = nullptr;            // NULL: none
+    const float* gain = nullptr;
+    float eps = 0.f;
+    // part[n] = sum_j coef[j] * X_j[n], j < terms; X_0 = first, X_j = hist + (j - 1) * histStride
+    float* part = nullptr;               // NULL: none
+    const float* coef = nullptr;
+    int terms = 0, n = 0;
+    const float* first = nullptr;
+    const float* hist = nullptr;
+    size_t histStride = 0;
+    __host__ __device__ int wgs() const { return (z ? 1 : 0) + (part ? (n + 255) / 256 : 0); }
+};
+
+// Rows of the multi-token path.  v = norm(yScale * y[t] (+ sum of the row's expert outputs)); normOut = v; then, with terms > 0,
+// v = sum_{j < terms} coef[j] X_j[t] + coef[terms] v; out = v (fp32) and / or outAct (bf16 or fp32).
+struct NormRows {
+    const float* y = nullptr;
+    int T = 0, n = 0, ldy = 0;
+    float yScale = 1.0f;
+    const int* rowIdx = nullptr;         // row t reads y[rowIdx[t]]
+    const float* experts = nullptr;      // [T, top, ldExperts]
+    int top = 0, ldExperts = 0;
+    const float* gain = nullptr;         // NULL: no norm
+    float eps = 0.f;
+    float* normOut = nullptr;
+    int ldNorm = 0;
+    const float* coef = nullptr;
+    int terms = 0;
+    const float* hist = nullptr;         // X_j at hist + j * histStride
+    size_t histStride = 0;
+    int ldHist = 0;
+    float* out = nullptr;
+    int ldOut = 0;
+    void* outAct = nullptr;
+    int actF32 = 0, ldAct = 0;
+};
+hipError_t launch_norm_rows(const NormRows& p, hipStream_t s);
+
+// q latent rows normed into activations, latent and rotated rows into the cache, from the raw projection z.
+struct LatentRows {
+    const float* z = nullptr;
+    int ldz = 0, T = 0, pos0 = 0;
+    int qRank = 0;
+    const float* qGain = nullptr;
+    void* qAct = nullptr;
+    int actF32 = 0, ldq = 0;
+    const float* kvGain = nullptr;       // NULL: the layer has no key/value projection
+    LatentCache cache;                   // rows follow the q latent in z
+    float eps = 0.f;
+};
+hipError_t launch_latent_rows(const LatentRows& p, hipStream_t s);
+
+// Routing of T tokens: z [T, ldz] router logits.  ids / weights [T, top]; then the (token, choice) entries sorted by
+// expert: perm [T * top] entry t * top + choice, and the row tiles of the experts' products (linear.h).
+struct MoeRoute {
+    const float* z = nullptr;
+    int ldz = 0, T = 0, experts = 0, top = 0;
+    int* ids = nullptr;
+    float* weights = nullptr;
+    int* work = nullptr;                 // 2 * experts ints
+    int* perm = nullptr;
+    int4* tiles = nullptr;
+    int* nTiles = nullptr;
+};
+inline int moe_max_tiles(int T, int top, int experts, int tileRows) {
+    const long e = (long)T * top;
+    return (int)(e / tileRows + (e < experts ? e : experts) + 1);
+}
+hipError_t launch_moe_route(const MoeRoute& p, hipStream_t s);
+
+}  // namespace mg

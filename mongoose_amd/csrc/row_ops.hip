@@ -1,0 +1,111 @@
+// row_ops.hip -- row-wise launches of the multi-token path (row_ops.h).
+#include "row_ops.h"
+#include "bf16_util.h"
+#include "device_util.h"
+#include "linear.h"
+#include "side_jobs.h"
+#include "vec_input.h"
+
+namespace mg {
+
+// One workgroup a row; the row stays in LDS between the passes.
+template <typename AT>
+__global__ __launch_bounds__(WG) void norm_rows_kernel(NormRows p) {
+    extern __shared__ float row[];
+    __shared__ float red[4];
+    const int t = blockIdx.x;
+    const float* y = p.y + (size_t)(p.rowIdx ? p.rowIdx[t] : t) * p.ldy;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < p.n; i += WG) {
+        float v = p.yScale * y[i];
+        for (int s = 0; s < p.top; s++) v += p.experts[((size_t)t * p.top + s) * p.ldExperts + i];
+        row[i] = v;
+        ss = fmaf(v, v, ss);
+    }
+    const float rs = p.gain ? 1.0f / sqrtf(block_sum(ss, red) / (float)p.n + p.eps) : 1.0f;
+    for (int i = threadIdx.x; i < p.n; i += WG) {
+        float v = row[i];
+        if (p.gain) v *= rs * p.gain[i];
+        if (p.normOut) p.normOut[(size_t)t * p.ldNorm + i] = v;
+        if (p.terms) {
+            float a = 0.f;
+            for (int j = 0; j < p.terms; j++) a = fmaf(p.coef[j], p.hist[j * p.histStride + (size_t)t * p.ldHist + i], a);
+            v = fmaf(p.coef[p.terms], v, a);
+        }
+        if (p.out) p.out[(size_t)t * p.ldOut + i] = v;
+        if (p.outAct) store_act(static_cast<AT*>(p.outAct) + (size_t)t * p.ldAct + i, v);
+    }
+}
+hipError_t launch_norm_rows(const NormRows& p, hipStream_t s) {
+    if (p.T <= 0) return hipSuccess;
+    if ((size_t)p.n * 4 > (60u << 10)) return hipErrorInvalidValue;
+    if (p.actF32) hipLaunchKernelGGL(norm_rows_kernel<float>, dim3(p.T), dim3(WG), (size_t)p.n * 4, s, p);
+    else hipLaunchKernelGGL(norm_rows_kernel<bf16_t>, dim3(p.T), dim3(WG), (size_t)p.n * 4, s, p);
+    return hipGetLastError();
+}
+
+template <typename AT>
+__global__ __launch_bounds__(WG) void latent_rows_kernel(LatentRows p) {
+    __shared__ float red[4];
+    const int t = blockIdx.x;
+    const float* z = p.z + (size_t)t * p.ldz;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < p.qRank; i += WG) ss = fmaf(z[i], z[i], ss);
+    const float rs = 1.0f / sqrtf(block_sum(ss, red) / (float)p.qRank + p.eps);
+    AT* q = static_cast<AT*>(p.qAct) + (size_t)t * p.ldq;
+    for (int i = threadIdx.x; i < p.qRank; i += WG) store_act(q + i, z[i] * rs * p.qGain[i]);
+    if (p.kvGain) write_latent_row<AT>(p.cache, z + p.qRank, p.kvGain, p.eps, p.pos0 + t, red);
+}
+hipError_t launch_latent_rows(const LatentRows& p, hipStream_t s) {
+    if (p.T <= 0) return hipSuccess;
+    if (p.kvGain && p.cache.f32 != p.actF32) return hipErrorInvalidValue;
+    if (p.actF32) hipLaunchKernelGGL(latent_rows_kernel<float>, dim3(p.T), dim3(WG), 0, s, p);
+    else hipLaunchKernelGGL(latent_rows_kernel<bf16_t>, dim3(p.T), dim3(WG), 0, s, p);
+    return hipGetLastError();
+}
+
+// work: [0, E) entries an expert, [E, 2E) its next free place.
+__global__ __launch_bounds__(WG) void route_choose_kernel(MoeRoute p) {
+    const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t >= p.T) return;
+    choose_experts(p.z + (size_t)t * p.ldz, p.experts, p.top, p.ids + (size_t)t * p.top, p.weights + (size_t)t * p.top);
+}
+__global__ __launch_bounds__(WG) void route_clear_kernel(MoeRoute p) {
+    for (int i = threadIdx.x; i < 2 * p.experts; i += WG) p.work[i] = 0;
+}
+__global__ __launch_bounds__(WG) void route_count_kernel(MoeRoute p) {
+    const int i = blockIdx.x * WG + threadIdx.x;
+    if (i < p.T * p.top) atomicAdd(p.work + p.ids[i], 1);
+}
+// Starts of the experts' ranges and their row tiles, a thread an expert.
+__global__ void route_tiles_kernel(MoeRoute p) {
+    __shared__ int cnt[MAX_EXPERTS];
+    for (int e = threadIdx.x; e < p.experts; e += blockDim.x) cnt[e] = p.work[e];
+    __syncthreads();
+    // thread e: start = entries of the experts before it, first tile = their tiles
+    for (int e = threadIdx.x; e < p.experts; e += blockDim.x) {
+        int start = 0, tile = 0;
+        for (int k = 0; k < e; k++) { start += cnt[k]; tile += (cnt[k] + MOE_TILE_ROWS - 1) / MOE_TILE_ROWS; }
+        p.work[p.experts + e] = start;
+        for (int r = 0; r < cnt[e]; r += MOE_TILE_ROWS) p.tiles[tile++] = make_int4(e, start + r, min(MOE_TILE_ROWS, cnt[e] - r), 0);
+        if (e == p.experts - 1) *p.nTiles = tile;
+    }
+}
+// The order of an expert's entries is whichever workgroup comes first; no result depends on it.
+__global__ __launch_bounds__(WG) void route_place_kernel(MoeRoute p) {
+    const int i = blockIdx.x * WG + threadIdx.x;
+    if (i < p.T * p.top) p.perm[atomicAdd(p.work + p.experts + p.ids[i], 1)] = i;
+}
+hipError_t launch_moe_route(const MoeRoute& p, hipStream_t s) {
+    if (p.T <= 0) return hipSuccess;
+    if (p.experts > MAX_EXPERTS || p.top < 1 || p.top > MAX_TOP || p.top > p.experts) return hipErrorInvalidValue;
+    const unsigned g = (unsigned)((p.T * p.top + WG - 1) / WG);
+    hipLaunchKernelGGL(route_clear_kernel, dim3(1), dim3(WG), 0, s, p);
+    hipLaunchKernelGGL(route_choose_kernel, dim3((p.T + 3) / 4), dim3(WG), 0, s, p);
+    hipLaunchKernelGGL(route_count_kernel, dim3(g), dim3(WG), 0, s, p);
+    hipLaunchKernelGGL(route_tiles_kernel, dim3(1), dim3(512), 0, s, p);
+    hipLaunchKernelGGL(route_place_kernel, dim3(g), dim3(WG), 0, s, p);
+    return hipGetLastError();
+}
+
+}  // namespace mg

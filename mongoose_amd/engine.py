@@ -7,8 +7,10 @@ in for, so that tests read like the reference's:
                                (engine.go:7-29, tensor.go:29-49, cuda.go:198-223)
     Tensor                     tensor.go:15-89
     K* functions               kernels.go:600-1136 wrappers over the per-op launches
+    DecodeModel                what every model class has: decode, generate, prefill, graphs, timing
     HIPFusedInference          CUDAFusedInference (cuda_fused_infer.go,
                                cuda_fused_infer_q4.go, cuda_fused_infer_stub.go:7-49)
+    HIPLayeredInference        models described by a list of layers (no counterpart)
     HIPStreamInfer             CUDAStreamInfer (cuda_fused_stream.go)
 
 Everything here is a thin ctypes call into libmongoose_hip.so; there is no
@@ -18,7 +20,7 @@ import ctypes
 
 import numpy as np
 
-from .lib import lib, last_error
+from .lib import LayerDesc, ModelDesc, lib, last_error
 
 _f = ctypes.POINTER(ctypes.c_float)
 _i = ctypes.POINTER(ctypes.c_int)
@@ -393,13 +395,11 @@ def HasGraphKernel():
     return lib.mg_has_graph_kernel() != 0
 
 
-class HIPFusedInference:
-    """Method set of CUDAFusedInference (cuda_fused_infer_stub.go:11-49)."""
+class DecodeModel:
+    """A model behind an mg_ctx handle: the token loops, graphs and timing every model class has."""
 
-    def __init__(self, handle, shape):
-        self._h = handle
-        (self.dim, self.kvDim, self.headDim, self.nHeads, self.nKVHeads, self.ffnDim, self.vocabSize,
-         self.nLayers, self.maxSeq) = shape
+    def __init__(self, handle, vocabSize, nLayers, maxSeq, dim):
+        self._h, self.vocabSize, self.nLayers, self.maxSeq, self.dim = handle, vocabSize, nLayers, maxSeq, dim
 
     def Close(self):
         if self._h:
@@ -411,6 +411,89 @@ class HIPFusedInference:
             self.Close()
         except Exception:
             pass
+
+    def ResetKV(self):
+        return lib.mg_reset_kv(self._h)
+
+    def ExportHidden(self):
+        out = np.empty(self.dim, dtype=np.float32)
+        rc = lib.mg_export_hidden(self._h, _fp(out))
+        return out if rc == 0 else None
+
+    def DecodeToken(self, token, pos, logitsOut=None):
+        nxt = ctypes.c_int(-1)
+        rc = lib.mg_decode_token(self._h, token, pos, ctypes.byref(nxt), _fp(logitsOut))
+        return rc, nxt.value
+
+    def Generate(self, prompt, nDecode, useGraph=True):
+        p = np.ascontiguousarray(prompt, dtype=np.int32)
+        out = np.empty(max(nDecode, 1), dtype=np.int32)
+        rc = lib.mg_generate(self._h, _ip(p), p.size, nDecode, _ip(out), 1 if useGraph else 0)
+        return rc, out[:nDecode]
+
+    def CaptureTokenGraph(self):
+        """mg_graph_capture: the whole-token graphs (embedding gather .. argmax) that Generate / GraphLaunch replay."""
+        return lib.mg_graph_capture(self._h)
+
+    def GraphLaunch(self, token, pos):
+        nxt = ctypes.c_int(-1)
+        rc = lib.mg_graph_launch(self._h, token, pos, ctypes.byref(nxt))
+        return rc, nxt.value
+
+    def ValidateGraph(self, token, pos):
+        md = ctypes.c_float(0)
+        rc = lib.mg_graph_validate(self._h, token, pos, ctypes.byref(md))
+        return rc, md.value
+
+    def TimedDecode(self, token, pos, steps, useGraph=True):
+        ms = ctypes.c_float(0)
+        rc = lib.mg_timed_decode(self._h, token, pos, steps, 1 if useGraph else 0, ctypes.byref(ms))
+        return rc, ms.value
+
+    def ProfileDecode(self, token, pos, steps, classMask=0):
+        ms = np.zeros(8, dtype=np.float32)
+        n = np.zeros(8, dtype=np.int32)
+        rc = lib.mg_profile_decode(self._h, token, pos, steps, classMask, _fp(ms), _ip(n))
+        return rc, ms, n
+
+    def Prefill(self, tokens, pos0=0, wantLogits=False):
+        """Batched prefill of `tokens` at positions pos0.. ; returns (rc, nextToken, logits or None, device ms)."""
+        toks = np.ascontiguousarray(tokens, dtype=np.int32)
+        nxt = ctypes.c_int(-1)
+        ms = ctypes.c_float(0.0)
+        logits = np.zeros(self.vocabSize, dtype=np.float32) if wantLogits else None
+        rc = lib.mg_prefill(self._h, _ip(toks), len(toks), pos0, ctypes.byref(nxt),
+                            _fp(logits) if wantLogits else None, ctypes.byref(ms))
+        return rc, nxt.value, logits, ms.value
+
+    def GeneratePrefill(self, prompt, nDecode):
+        p = np.ascontiguousarray(prompt, dtype=np.int32)
+        out = np.zeros(max(nDecode, 1), dtype=np.int32)
+        rc = lib.mg_generate_prefill(self._h, _ip(p), len(p), nDecode, _ip(out))
+        return rc, out[:nDecode]
+
+    def WeightBytesPerToken(self):
+        return lib.mg_weight_bytes_per_token(self._h)
+
+    def KVBytesAt(self, pos):
+        return lib.mg_kv_bytes_at(self._h, pos)
+
+    def PrefillLogits(self, tokens, pos0, want):
+        """The tokens at positions pos0 .. in one pass; returns (rc, logits [len(want), vocab]) of the rows `want`
+        (indices into tokens)."""
+        toks = np.ascontiguousarray(tokens, dtype=np.int32)
+        w = np.ascontiguousarray(want, dtype=np.int32)
+        out = np.empty((len(w), self.vocabSize), dtype=np.float32)
+        rc = lib.mg_prefill_logits(self._h, _ip(toks), len(toks), pos0, _ip(w), len(w), _fp(out))
+        return rc, out
+
+
+class HIPFusedInference(DecodeModel):
+    """Method set of CUDAFusedInference (cuda_fused_infer_stub.go:11-49)."""
+
+    def __init__(self, handle, shape):
+        (dim, self.kvDim, self.headDim, self.nHeads, self.nKVHeads, self.ffnDim, vocabSize, nLayers, maxSeq) = shape
+        super().__init__(handle, vocabSize, nLayers, maxSeq, dim)
 
     def NumWeights(self):
         return lib.mg_num_weights(self._h)
@@ -445,9 +528,6 @@ class HIPFusedInference:
     def SetKVFormat(self, fmt):
         """0 = fp32 KV rows, 1 = fp16; before SetLayerRange."""
         return lib.mg_set_kv_format(self._h, fmt)
-
-    def ResetKV(self):
-        return lib.mg_reset_kv(self._h)
 
     def SetExecMode(self, mode):
         """0 = one launch per reference op, 1 = fused launches, 2 = fused without the L2 prefetch helpers,
@@ -501,36 +581,6 @@ class HIPFusedInference:
         h = _as_f32(hiddenIn) if hiddenIn is not None else None
         return lib.mg_step_layer_resident(self._h, layer, pos, _fp(h), _fp(preOut), _fp(postOut), _fp(logitsOut))
 
-    def ExportHidden(self):
-        out = np.empty(self.dim, dtype=np.float32)
-        rc = lib.mg_export_hidden(self._h, _fp(out))
-        return out if rc == 0 else None
-
-    def DecodeToken(self, token, pos, logitsOut=None):
-        nxt = ctypes.c_int(-1)
-        rc = lib.mg_decode_token(self._h, token, pos, ctypes.byref(nxt), _fp(logitsOut))
-        return rc, nxt.value
-
-    def Generate(self, prompt, nDecode, useGraph=True):
-        p = np.ascontiguousarray(prompt, dtype=np.int32)
-        out = np.empty(max(nDecode, 1), dtype=np.int32)
-        rc = lib.mg_generate(self._h, _ip(p), p.size, nDecode, _ip(out), 1 if useGraph else 0)
-        return rc, out[:nDecode]
-
-    def CaptureTokenGraph(self):
-        """mg_graph_capture: the whole-token graphs (embedding gather .. argmax) that Generate / GraphLaunch replay."""
-        return lib.mg_graph_capture(self._h)
-
-    def GraphLaunch(self, token, pos):
-        nxt = ctypes.c_int(-1)
-        rc = lib.mg_graph_launch(self._h, token, pos, ctypes.byref(nxt))
-        return rc, nxt.value
-
-    def ValidateGraph(self, token, pos):
-        md = ctypes.c_float(0)
-        rc = lib.mg_graph_validate(self._h, token, pos, ctypes.byref(md))
-        return rc, md.value
-
     # ---- CUDAGraph mirror, cuda_graph.go:286-739 ----
     def CaptureGraph(self, cfg, pos):
         """(*CUDAFusedInference).CaptureGraph(cfg, pos), cuda_graph.go:315: a HIPGraph over cfg.LayerStart ..
@@ -575,33 +625,6 @@ class HIPFusedInference:
             return False
         g.Destroy()
         return True
-
-    def TimedDecode(self, token, pos, steps, useGraph=True):
-        ms = ctypes.c_float(0)
-        rc = lib.mg_timed_decode(self._h, token, pos, steps, 1 if useGraph else 0, ctypes.byref(ms))
-        return rc, ms.value
-
-    def ProfileDecode(self, token, pos, steps, classMask=0):
-        ms = np.zeros(8, dtype=np.float32)
-        n = np.zeros(8, dtype=np.int32)
-        rc = lib.mg_profile_decode(self._h, token, pos, steps, classMask, _fp(ms), _ip(n))
-        return rc, ms, n
-
-    def Prefill(self, tokens, pos0=0, wantLogits=False):
-        """Batched prefill of `tokens` at positions pos0.. ; returns (rc, nextToken, logits or None, device ms)."""
-        toks = np.ascontiguousarray(tokens, dtype=np.int32)
-        nxt = ctypes.c_int(-1)
-        ms = ctypes.c_float(0.0)
-        logits = np.zeros(self.vocabSize, dtype=np.float32) if wantLogits else None
-        rc = lib.mg_prefill(self._h, _ip(toks), len(toks), pos0, ctypes.byref(nxt),
-                            _fp(logits) if wantLogits else None, ctypes.byref(ms))
-        return rc, nxt.value, logits, ms.value
-
-    def GeneratePrefill(self, prompt, nDecode):
-        p = np.ascontiguousarray(prompt, dtype=np.int32)
-        out = np.zeros(max(nDecode, 1), dtype=np.int32)
-        rc = lib.mg_generate_prefill(self._h, _ip(p), len(p), nDecode, _ip(out))
-        return rc, out[:nDecode]
 
     def FlowExchange(self, layer):
         """The persistent layer launch's exchange block of `layer` after the last step, as a dict of named
@@ -671,12 +694,6 @@ class HIPFusedInference:
         """Per-wait time limit of the persistent layer launch in 10 ns ticks (negative: give up at once)."""
         return lib.mg_flow_set_wait_limit(self._h, int(ticks))
 
-    def WeightBytesPerToken(self):
-        return lib.mg_weight_bytes_per_token(self._h)
-
-    def KVBytesAt(self, pos):
-        return lib.mg_kv_bytes_at(self._h, pos)
-
     def StreamBuild(self):
         h = lib.mg_stream_build(self._h)
         return HIPStreamInfer(h, self) if h else None
@@ -692,6 +709,49 @@ def NewHIPFusedInference(eng, dim, kvDim, headDim, nHeads, nKVHeads, ffnDim, voc
     if not h:
         return None
     return HIPFusedInference(h, (dim, kvDim, headDim, nHeads, nKVHeads, ffnDim, vocabSize, nLayers, maxSeq))
+
+
+class HIPLayeredInference(DecodeModel):
+    """A model described by a list of layers (configs.LayeredModel): tensors by name, bf16 weights."""
+
+    def __init__(self, handle, spec, maxSeq, dtype):
+        super().__init__(handle, spec.vocab, len(spec.layers), maxSeq, spec.width)
+        self.spec, self.dtype = spec, dtype
+
+    def TensorNames(self):
+        return [lib.mg_tensor_name(self._h, i).decode() for i in range(lib.mg_num_tensors(self._h))]
+
+    def TensorShape(self, name):
+        """None for a name the model does not have."""
+        shape = (ctypes.c_int64 * 2)()
+        n = lib.mg_tensor_shape(self._h, name.encode(), shape)
+        return tuple(shape[:n]) if n > 0 else None
+
+    def SetTensor(self, name, bits):
+        """bits: the bf16 values as uint16, in the tensor's shape."""
+        a = np.ascontiguousarray(bits)
+        assert a.dtype == np.uint16
+        return lib.mg_set_tensor_bf16(self._h, name.encode(), a.ctypes.data_as(ctypes.POINTER(ctypes.c_uint16)), a.size)
+
+    def PrefillHidden(self, tokens, pos0, layerEnd):
+        """x of every token after layers 0 .. layerEnd - 1 (the sequence has to be started over afterwards)."""
+        toks = np.ascontiguousarray(tokens, dtype=np.int32)
+        out = np.empty((len(toks), self.dim), dtype=np.float32)
+        rc = lib.mg_prefill_hidden(self._h, _ip(toks), len(toks), pos0, layerEnd, _fp(out))
+        return rc, out
+
+
+def NewHIPLayeredInference(eng, spec, maxSeq, dtype="bfloat16"):
+    """A context for configs.LayeredModel `spec`; None on failure (text in last_error())."""
+    if eng is None:
+        return None
+    if dtype not in ("bfloat16", "float32"):
+        raise ValueError("dtype must be bfloat16 or float32")
+    descs = (LayerDesc * len(spec.layers))(*[LayerDesc(**layer) for layer in spec.layers])
+    model = ModelDesc(width=spec.width, vocab=spec.vocab, n_layers=len(spec.layers), eps=spec.eps, alpha=spec.alpha,
+                      f32=1 if dtype == "float32" else 0)
+    h = lib.mg_create_layered(ctypes.byref(model), descs, maxSeq)
+    return HIPLayeredInference(h, spec, maxSeq, dtype) if h else None
 
 
 class HIPStreamInfer:

@@ -10,19 +10,25 @@ from ctypes import (POINTER, c_char_p, c_double, c_float, c_int, c_int8, c_int32
 
 HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(HERE, "libmongoose_hip.so")
+# Only the model class of layer lists (build.build_layered): used where the full library has not been built.
+LAYERED_LIB_PATH = os.path.join(HERE, "libmongoose_layered.so")
 
-if not os.path.exists(LIB_PATH):
+LOADED_PATH = next((p for p in (LIB_PATH, LAYERED_LIB_PATH) if os.path.exists(p)), None)
+if LOADED_PATH is None:
     raise ImportError(
         f"{LIB_PATH} is missing: the HIP library has not been built "
         "(run `python -m mongoose_amd.build`); there is no CPU fallback")
 
-lib = ctypes.CDLL(LIB_PATH, mode=ctypes.RTLD_GLOBAL)
+lib = ctypes.CDLL(LOADED_PATH, mode=ctypes.RTLD_GLOBAL)
 
 _f = POINTER(c_float)
 _i = POINTER(c_int)
 
 
 def _sig(name, restype, *argtypes):
+    fn = getattr(lib, name, None)
+    if fn is None and LOADED_PATH != LIB_PATH:
+        return                                   # not part of the smaller library: using it raises AttributeError
     fn = getattr(lib, name)
     fn.restype = restype
     fn.argtypes = list(argtypes)
@@ -117,6 +123,7 @@ _sig("mg_has_graph_kernel", c_int)
 _sig("mg_timed_decode", c_int, c_void_p, c_int, c_int, c_int, c_int, _f)
 _sig("mg_profile_decode", c_int, c_void_p, c_int, c_int, c_int, ctypes.c_uint, _f, _i)
 _sig("mg_prefill", c_int, c_void_p, _i, c_int, c_int, _i, _f, _f)
+_sig("mg_prefill_logits", c_int, c_void_p, _i, c_int, c_int, _i, c_int, _f)
 _sig("mg_generate_prefill", c_int, c_void_p, _i, c_int, c_int, _i)
 _sig("mg_bench_matvec", c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, _f)
 _sig("mg_flow_exchange", c_int, c_void_p, c_int, _f, c_size_t, _i)
@@ -134,6 +141,27 @@ _sig("mg_kv_bytes_at", c_uint64, c_void_p, c_int)
 _sig("mg_stream_build", c_void_p, c_void_p)
 _sig("mg_stream_destroy", None, c_void_p)
 _sig("mg_stream_forward_token", c_int, c_void_p, c_int, _f, c_int, POINTER(c_void_p), POINTER(c_int32), _f)
+
+# 4. models described by a list of layers
+class LayerDesc(ctypes.Structure):
+    """mg_layer_desc."""
+    _fields_ = [("mixer", c_int), ("heads", c_int), ("dim", c_int), ("rot_dim", c_int), ("vdim", c_int), ("kv_rank", c_int),
+                ("q_rank", c_int), ("window", c_int), ("kv_from", c_int), ("rope_dims", c_int), ("rope_base", c_double),
+                ("scale", c_float), ("decay_rank", c_int), ("mlp", c_int), ("ff", c_int), ("experts", c_int), ("top", c_int),
+                ("ff_shared", c_int)]
+
+
+class ModelDesc(ctypes.Structure):
+    """mg_model_desc."""
+    _fields_ = [("width", c_int), ("vocab", c_int), ("n_layers", c_int), ("eps", c_float), ("alpha", c_float), ("f32", c_int)]
+
+
+_sig("mg_create_layered", c_void_p, POINTER(ModelDesc), POINTER(LayerDesc), c_int)
+_sig("mg_num_tensors", c_int, c_void_p)
+_sig("mg_tensor_name", c_char_p, c_void_p, c_int)
+_sig("mg_tensor_shape", c_int, c_void_p, c_char_p, POINTER(ctypes.c_int64))
+_sig("mg_set_tensor_bf16", c_int, c_void_p, c_char_p, POINTER(c_uint16), c_size_t)
+_sig("mg_prefill_hidden", c_int, c_void_p, _i, c_int, c_int, c_int, _f)
 
 # host helpers
 _sig("mg_quantize_q8", None, _f, c_int, c_int, c_int, POINTER(c_int8), _f)

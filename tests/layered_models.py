@@ -1,0 +1,199 @@
+"""Small random models of layer lists for the tests: one description and one set of bf16 weights, loaded into the
+oracle (oracle/layered.py) and into the HIP context, and written as a model folder."""
+import json
+import os
+
+import numpy as np
+
+from mongoose_amd import configs as C
+from mongoose_amd import engine as E
+from oracle import layered as O
+
+
+def bf16_bits(a):
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32).astype(np.uint64)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def bf16_values(bits):
+    return (bits.astype(np.uint32) << 16).view(np.float32)
+
+
+def latent(heads=3, dim=40, rot_dim=24, vdim=56, kv_rank=48, q_rank=72, scale=0.3, rope_base=10000.0, window=0, kv_from=None, **kw):
+    return C.latent_attention(heads, dim, rot_dim, vdim, kv_rank, q_rank, scale, rope_base, window=window, kv_from=kv_from, **kw)
+
+
+def delta(heads=3, dim=24, decay_rank=9):
+    return C.general_delta(heads, dim, decay_rank)
+
+
+def model(layers, width=104, vocab=90, eps=1e-5, alpha=1.7):
+    return C.LayeredModel("test", width, vocab, eps, alpha, tuple(layers))
+
+
+def tensor_shapes(s):
+    """Names and sizes, written out here once more (the HIP context has its own list)."""
+    W, out = s.width, {"embed": (s.vocab, s.width), "head": (s.vocab, s.width), "final.norm": (s.width,)}
+    for i, L in enumerate(s.layers):
+        p, m, f = f"l{i}.", f"l{i}.mix.", f"l{i}.mlp."
+        out[p + "norm1"], out[p + "dwa"] = (W,), (i + 2,)
+        H, D = L["heads"], L["dim"]
+        if L["mixer"] == C.MIX_LATENT_ATTENTION:
+            out[m + "dq"], out[m + "dq.norm"] = (L["q_rank"], W), (L["q_rank"],)
+            out[m + "uq"] = (H * (D + L["rot_dim"]), L["q_rank"])
+            if L["kv_from"] < 0:
+                out[m + "dkv"], out[m + "dkv.norm"] = (L["kv_rank"] + L["rot_dim"], W), (L["kv_rank"],)
+            out[m + "uk"], out[m + "uv"] = (H * D, L["kv_rank"]), (H * L["vdim"], L["kv_rank"])
+            out[m + "o"] = (W, H * L["vdim"])
+        else:
+            for n in "rkvga":
+                out[m + n] = (H * D, W)
+            out[m + "w1"], out[m + "w2"] = (L["decay_rank"], W), (H * D, L["decay_rank"])
+            for n in ("a.b", "w0", "norm"):
+                out[m + n] = (H * D,)
+            out[m + "o"] = (W, H * D)
+        kind = L.get("mlp", C.MLP_NONE)
+        if kind == C.MLP_NONE:
+            continue
+        out[p + "norm2"] = (W,)
+        if kind == C.MLP_DENSE:
+            out[f + "up"], out[f + "down"], out[f + "act"] = (L["ff"], W), (W, L["ff"]), (2,)
+        else:
+            out[f + "router"] = (L["experts"], W)
+            for e in range(L["experts"]):
+                out[f"{f}e{e}.up"], out[f"{f}e{e}.down"] = (L["ff"], W), (W, L["ff"])
+            if L["ff_shared"]:
+                out[f + "shared.up"], out[f + "shared.down"] = (L["ff_shared"], W), (W, L["ff_shared"])
+    return out
+
+
+def random_bits(s, seed):
+    rng = np.random.default_rng(seed)
+    out = {}
+    for name, shape in sorted(tensor_shapes(s).items()):
+        if name.endswith("norm") or name.endswith("norm1") or name.endswith("norm2"):
+            a = 1 + 0.2 * rng.standard_normal(shape)
+        elif name.endswith("dwa"):
+            a = 0.4 * rng.standard_normal(shape)
+            a[-1] += 1
+        elif len(shape) == 1:
+            a = 0.7 * rng.standard_normal(shape)
+        elif name == "embed":
+            a = rng.standard_normal(shape)
+        else:
+            a = rng.standard_normal(shape) * (1.6 if name.endswith(("router", "uq", ".w1")) else 1.0) / np.sqrt(shape[1])
+        out[name] = bf16_bits(a)
+    return out
+
+
+def oracle_model(s):
+    layers = []
+    for L in s.layers:
+        if L["mixer"] == C.MIX_LATENT_ATTENTION:
+            mixer = {k: L[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "window", "scale", "rope_base", "rope_dims")}
+            mixer.update(type="latent_attention", kv_from=None if L["kv_from"] < 0 else L["kv_from"],
+                         rot_base=L["rope_base"], rot_dims=L["rope_dims"])
+        else:
+            mixer = dict(type="general_delta", heads=L["heads"], dim=L["dim"])
+        kind = L.get("mlp", C.MLP_NONE)
+        mlp = None if kind == C.MLP_NONE else dict(kind="dense") if kind == C.MLP_DENSE else \
+            dict(kind="moe", experts=L["experts"], top=L["top"], shared=L["ff_shared"] > 0)
+        layers.append(dict(mixer=mixer, mlp=mlp))
+    return dict(width=s.width, vocab=s.vocab, eps=s.eps, alpha=s.alpha, layers=layers)
+
+
+class Pair:
+    """The same model in the oracle and, with an engine, on the GPU."""
+
+    def __init__(self, s, seed=1, eng=None, dtype="float32", maxSeq=256, tweak=None):
+        self.s, self.seed, self.maxSeq = s, seed, maxSeq
+        self.bits = random_bits(s, seed)
+        if tweak:
+            for name, fn in tweak.items():
+                self.bits[name] = bf16_bits(fn(bf16_values(self.bits[name])))
+        self.values = {k: bf16_values(v).astype(np.float64) for k, v in self.bits.items()}
+        self.orc = O.Oracle(oracle_model(s), self.values)
+        self.hip = None
+        if eng is not None:
+            self.hip = self.load(eng, dtype)
+
+    def load(self, eng, dtype):
+        hip = E.NewHIPLayeredInference(eng, self.s, self.maxSeq, dtype)
+        assert hip is not None, E.last_error()
+        for name, b in self.bits.items():
+            assert hip.TensorShape(name) == b.shape, (name, hip.TensorShape(name), b.shape)
+            assert hip.SetTensor(name, b) == 0, E.last_error()
+        return hip
+
+    def tokens(self, n, salt=0):
+        return np.random.default_rng(self.seed * 1000 + salt).integers(0, self.s.vocab, n).astype(np.int32)
+
+    def oracle_logits(self, tokens):
+        self.orc.reset()
+        return self.orc.run(tokens)
+
+    def close(self):
+        if self.hip:
+            self.hip.Close()
+
+
+def run_portions(hip, tokens, sizes):
+    """Logits of every token, the prompt cut into `sizes` (repeated as needed)."""
+    assert hip.ResetKV() == 0
+    rows, at, k = [], 0, 0
+    while at < len(tokens):
+        n = min(sizes[k % len(sizes)], len(tokens) - at)
+        rc, lg = hip.PrefillLogits(tokens[at:at + n], at, list(range(n)))
+        assert rc == 0, E.last_error()
+        rows.append(lg)
+        at += n
+        k += 1
+    return np.concatenate(rows)
+
+
+def errors(got, want):
+    """Per position: RMS difference of the mean-free logits relative to their own RMS over all positions."""
+    d = got.astype(np.float64) - want
+    d -= d.mean(axis=1, keepdims=True)
+    w = want - want.mean(axis=1, keepdims=True)
+    return np.sqrt((d * d).mean(axis=1)) / np.sqrt((w * w).mean())
+
+
+def write_folder(folder, s, bits, config):
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(config, f)
+    header, data, at = {}, [], 0
+    for name, b in bits.items():
+        header[name] = {"dtype": "BF16", "shape": list(b.shape), "data_offsets": [at, at + b.nbytes]}
+        data.append(b.tobytes())
+        at += b.nbytes
+    h = json.dumps(header).encode()
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(len(h).to_bytes(8, "little") + h + b"".join(data))
+
+
+def vadonex_config(s):
+    """config.json of a description (the inverse of configs.read_vadonex)."""
+    layers = []
+    for L in s.layers:
+        if L["mixer"] == C.MIX_LATENT_ATTENTION:
+            m = {k: L[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank", "scale")}
+            m["rot"] = {"base": L["rope_base"], "dims": L["rope_dims"]}
+            m["mask"] = {"size": L["window"]}
+            if L["kv_from"] >= 0:
+                m["kv_from"] = L["kv_from"]
+            e = {"type": "latent_attention", "mixer": m}
+        else:
+            e = {"type": "general_delta", "mixer": {"heads": L["heads"], "dim": L["dim"]}}
+        kind = L.get("mlp", C.MLP_NONE)
+        e["mlp"] = None
+        if kind == C.MLP_DENSE:
+            e["mlp"] = {"kind": "dense", "ff": L["ff"]}
+        elif kind == C.MLP_MOE:
+            e["mlp"] = {"kind": "moe", "router": {"experts": L["experts"], "top": L["top"]}, "expert": {"ff": L["ff"]}}
+            if L["ff_shared"]:
+                e["mlp"]["shared"] = {"ff": L["ff_shared"]}
+        layers.append(e)
+    return {"architecture": "Vadonex", "vocab": s.vocab, "width": s.width, "norm": {"eps": s.eps}, "postln_alpha": s.alpha,
+            "layers": layers}
