@@ -520,6 +520,129 @@ def stream_leg(E, np, configs, f, s, seed, n):
                     "buffers into two device sets (copy of layer l+1 overlaps compute of layer l); logits read back each token"}
 
 
+# Layered (Vadonex) models of realistic layer sizes, and the closest existing model of the same width and layer count.
+LAYERED_SIZES = {
+    "w2048": dict(width=2048, heads=16, dim=128, rot=64, vdim=128, kv_rank=512, q_rank=1536, window=1024, d_heads=32, d_dim=64,
+                  d_rank=96, ff=5632, experts=64, top=6, eff=1024, shared=2048, like="tinyllama-1.1b"),
+    "w4096": dict(width=4096, heads=32, dim=128, rot=64, vdim=128, kv_rank=512, q_rank=1536, window=4096, d_heads=64, d_dim=64,
+                  d_rank=128, ff=14336, experts=32, top=4, eff=2048, shared=4096, like="llama-3-8b"),
+}
+
+
+def layered_spec(configs, z, vocab, eps=1e-5):
+    """Eight layers: latent attention with a cache of its own twice, reading another layer's twice, the delta rule four times."""
+    def lat(kv_from=None):
+        return configs.latent_attention(z["heads"], z["dim"], z["rot"], z["vdim"], z["kv_rank"], z["q_rank"],
+                                        (z["dim"] + z["rot"]) ** -0.5, 1e4, window=z["window"], kv_from=kv_from)
+    dl = configs.general_delta(z["d_heads"], z["d_dim"], z["d_rank"])
+    dense, moe = configs.dense_ff(z["ff"]), configs.moe_ff(z["eff"], z["experts"], z["top"], z["shared"])
+    layers = [{**lat(), **dense}, {**dl, **moe}, {**lat(), **moe}, {**dl, **moe}, {**lat(2), **moe}, {**dl, **moe},
+              {**dl, **dense}, {**lat(2), **dense}]
+    return configs.LayeredModel("vadonex", z["width"], vocab, eps, 2.0, tuple(layers))
+
+
+def layered_model(E, np, eng, spec, maxSeq, seed):
+    f = E.NewHIPLayeredInference(eng, spec, maxSeq)
+    if f is None:
+        raise RuntimeError(E.last_error())
+    rng = np.random.default_rng(seed)
+    pool = (rng.standard_normal(1 << 22).astype(np.float32).view(np.uint32) >> 16).astype(np.uint16)    # N(0, 1), truncated to bf16
+    for k, name in enumerate(f.TensorNames()):
+        shape = f.TensorShape(name)
+        n = int(np.prod(shape))
+        bits = np.resize(np.roll(pool, 7919 * k), n) if n < pool.size else np.resize(pool, n)
+        v = (bits.astype(np.uint32) << 16).view(np.float32)
+        if len(shape) == 2:
+            v = v * np.float32(1.0 if name == "embed" else shape[1] ** -0.5)
+        else:
+            v = 1 + 0.1 * v if "norm" in name else 0.3 * v
+            if name.endswith("dwa"):
+                v[-1] += 1
+        if f.SetTensor(name, (v.astype(np.float32).view(np.uint32) >> 16).astype(np.uint16).reshape(shape)) != 0:
+            raise RuntimeError(f"{name}: " + E.last_error())
+    return f
+
+
+def layered_class_bytes(configs, spec, pos):
+    """Bytes a token's launches of each timing class read (sum over the layers), by the weights' and caches' stored sizes."""
+    pad = lambda n: (n + 63) // 64 * 64                                                    # noqa: E731
+    W, b = pad(spec.width), {c: 0 for c in range(8)}
+    for L in spec.layers:
+        if L["mixer"] == configs.MIX_LATENT_ATTENTION:
+            H = L["heads"]
+            own = L["kv_rank"] + L["rot_dim"] if L["kv_from"] < 0 else 0
+            b[1] += 2 * ((L["q_rank"] + own) * W + H * (L["dim"] + L["rot_dim"]) * pad(L["q_rank"]) + H * L["kv_rank"] * pad(L["dim"]))
+            keys = min(pos + 1, L["window"] or pos + 1)
+            b[2] += 2 * keys * (L["kv_rank"] + L["rot_dim"])
+            b[3] += 2 * (H * L["vdim"] * pad(L["kv_rank"]) + spec.width * pad(H * L["vdim"]))
+        else:
+            HD = L["heads"] * L["dim"]
+            b[1] += 2 * (5 * HD + L["decay_rank"]) * W
+            b[2] += 8 * HD * L["dim"] + 2 * HD * pad(L["decay_rank"])
+            b[3] += 2 * spec.width * pad(HD)
+        if L["mlp"] == configs.MLP_DENSE:
+            b[4] += 2 * L["ff"] * W
+            b[5] += 2 * spec.width * pad(L["ff"])
+        else:
+            b[4] += 2 * (L["experts"] + L["ff_shared"] + L["top"] * L["ff"]) * W
+            b[5] += 2 * spec.width * (L["top"] * pad(L["ff"]) + pad(L["ff_shared"]))
+    b[6] = 2 * spec.vocab * W
+    return b
+
+
+def measure_layered(E, np, configs, eng, name, seed, K, W, prefill, lean=False):
+    """One size: decode at two positions, per-class launch times, prefill; the same of the closest existing model (Q8)."""
+    z = LAYERED_SIZES[name]
+    like = configs.BY_NAME[z["like"]]
+    like = like._replace(nLayers=8, vocab=32000, name=like.name + "-L8")
+    spec = layered_spec(configs, z, like.vocab)
+    ctx = [W, 3000]
+    maxSeq = max(ctx[-1] + K + 40, max(prefill) + 8)
+    out = {"size": name, "layers": "LA dense, GD moe, LA moe, GD moe, LA(2) moe, GD moe, GD dense, LA(2) dense", **{k: v for k, v in z.items() if k != "like"}}
+    for key in ("vadonex", "closest"):
+        f = layered_model(E, np, eng, spec, maxSeq, seed) if key == "vadonex" else load_model(E, np, like, seed, maxSeq, eng)
+        r = {"model": "vadonex" if key == "vadonex" else like.name, "weight_bytes_per_token": int(f.WeightBytesPerToken()), "decode": [], "prefill": []}
+        modes = [None] if key == "vadonex" else [3, 1]
+        for pos in ctx:
+            for mode in modes:
+                if mode is not None:
+                    assert f.SetExecMode(mode) == 0
+                rc, _ = f.TimedDecode(1, pos, 4)
+                rc2, ms = f.TimedDecode(1, pos, K)
+                assert rc == 0 and rc2 == 0, E.last_error()
+                nbytes = f.WeightBytesPerToken() + f.KVBytesAt(pos + K // 2)
+                e = {"position": pos, "ms_per_token": round(ms / K, 5), "tok_s": round(K / ms * 1e3, 1),
+                     "GBps": round(nbytes / (ms / K) / 1e6, 1), "frac_of_peak": round(nbytes / (ms / K) / 1e6 / HBM_PEAK_GBS, 4)}
+                if mode is not None:
+                    e["launches"] = "one persistent launch" if mode == 3 and f.FlowInUse() else "fused launches"
+                if not lean and mode in (None, 1):
+                    if key == "vadonex":
+                        rc, ms8, n8 = f.ProfileDecode(1, pos, 16)
+                        assert rc == 0, E.last_error()
+                        cb = layered_class_bytes(configs, spec, pos + 8)
+                        e["classes"] = [{"cls": LAYERED_NAMES[c], "intervals": int(n8[c]), "us_per_token": round(float(ms8[c] * n8[c]) * 1e3, 2),
+                                         "bytes": int(cb[c]), "frac_of_peak": round(cb[c] / (float(ms8[c] * n8[c]) * 1e-3) / 1e9 / HBM_PEAK_GBS, 4)}
+                                        for c in range(8) if n8[c]]
+                    else:
+                        e["classes"] = launch_table(f, configs, like, 1, pos, 16, ms / K, False)
+                r["decode"].append(e)
+        for T in prefill:
+            toks = E.synth_tokens(seed, 20_000_003, like.vocab, T)
+            best = None
+            for _ in range(4):
+                rc, _, _, ms = f.Prefill(toks, 0)
+                assert rc == 0, E.last_error()
+                best = ms if best is None else min(best, ms)
+            r["prefill"].append({"tokens": T, "ms": round(best, 3), "tok_s": round(T / best * 1e3, 1)})
+        out[key] = r
+        f.Close()
+    return out
+
+
+LAYERED_NAMES = {0: "embed_gather", 1: "input projections (latent: + q up, absorb)", 2: "attention / delta step", 3: "(value up +) output projection",
+                 4: "norm + up (moe: router, shared up, experts up)", 5: "down", 6: "norms + lm_head + argmax partials", 7: "argmax_finish"}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -561,11 +684,36 @@ def main():
                          "from profiles/ are reported instead)")
     ap.add_argument("--no-configs", action="store_true",
                     help="only the configuration named by --config (no 'configs' object with the other benchmark configurations)")
+    ap.add_argument("--layered", default="", metavar="SIZE",
+                    help="instead of the workload above: a Vadonex model of this size (" + ", ".join(LAYERED_SIZES) + ", or all) beside "
+                         "the closest existing model of the same width and layer count; prefill of --prefill tokens (default 512 and 2048)")
     args = ap.parse_args()
     if args.gpus != 1:
         print(f"bench.py: this build measures one GPU only (got --gpus {args.gpus}); "
               "the decode path is batch-1 on a single device", file=sys.stderr)
         sys.exit(2)
+
+    if args.layered:
+        import numpy as np
+        from mongoose_amd import configs
+        from mongoose_amd import engine as E
+        eng = E.NewHIP(0)
+        if eng is None:
+            print("bench.py: no HIP device", file=sys.stderr)
+            sys.exit(1)
+        sizes = list(LAYERED_SIZES) if args.layered == "all" else args.layered.split(",")
+        res = []
+        for name in sizes:
+            print(f"bench.py: layered {name}", file=sys.stderr, flush=True)
+            res.append(measure_layered(E, np, configs, eng, name, args.seed, args.steps, max(args.warmup, 1),
+                                       [args.prefill] if args.prefill else [512, 2048], lean=args.lean))
+        d = res[0]["vadonex"]["decode"][0]
+        print(json.dumps({"metric": f"decode tok/s (bs=1, Vadonex layers {sizes[0]})", "value": d["tok_s"], "unit": "tok/s", "n_gpus": 1,
+                          "steps": args.steps, "warmup": args.warmup, "ms_per_step": d["ms_per_token"], "higher_is_better": True,
+                          "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+                          "config": {"workload": "random-init Vadonex layers, greedy decode, batch 1; the closest existing model beside it"},
+                          "sizes": res, "device": eng.Name()}))
+        return
 
     # HBM traffic of the run's own launches, from counters: before anything here touches the GPU (the profiler runs
     # children of this process).  Only for the default path, whose dispatches the passes can pick out.

@@ -12,8 +12,16 @@ struct ActParam { int kind; float ap, an; };
 
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float gelu_erf_f(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
+// exp(z) - 1 - z for z <= 0: near zero its Taylor series (the difference would cancel), 2^-24 of the result
+__device__ __forceinline__ float exp_m1_mz(float z) {
+    float p = 2.48015873e-5f;                                 // 1/8!
+    p = fmaf(p, z, 1.98412698e-4f); p = fmaf(p, z, 1.38888889e-3f); p = fmaf(p, z, 8.33333333e-3f);
+    p = fmaf(p, z, 4.16666667e-2f); p = fmaf(p, z, 1.66666667e-1f); p = fmaf(p, z, 0.5f);
+    return z > -0.5f ? p * z * z : __expf(z) - 1.0f - z;
+}
 __device__ __forceinline__ float xielu_f(float z, float ap, float an) {
-    return z > 0.f ? ap * z * z + 0.5f * z : an * (expm1f(z) - z) + 0.5f * z;
+    const float q = exp_m1_mz(fminf(z, 0.f));
+    return fmaf(0.5f, z, z > 0.f ? ap * z * z : an * q);
 }
 __device__ __forceinline__ float apply_act(float z, ActParam a) {
     if (a.kind == ACT_GELU) return gelu_erf_f(z);

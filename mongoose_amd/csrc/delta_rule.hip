@@ -11,93 +11,124 @@ constexpr float LOG_DECAY = -0.60653065971263342f;      // -exp(-1/2)
 constexpr float UNIT_EPS = 1e-6f;
 
 // ---------------------------------------------------------------------------
-// decode: one workgroup a head; thread = (value column, group of key channels)
+// decode: one workgroup a head; thread = (value column, group of key channels), its part of the state in registers from
+// the start of the launch
 // ---------------------------------------------------------------------------
-__global__ __launch_bounds__(WG) void delta_step_kernel(DeltaStep p) {
-    extern __shared__ float sh[];
-    __shared__ float red[4];
+template <int NT>
+__device__ __forceinline__ float block_sum_of(float v, float* red) {
+    v = wave_sum(v);
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float t = 0.f;
+#pragma unroll
+    for (int w = 0; w < NT / 64; w++) t += red[w];
+    __syncthreads();
+    return t;
+}
+
+template <int NT, int PER>      // threads; most key channels of a thread
+__global__ __launch_bounds__(NT) void delta_step_kernel(DeltaStep p) {
+    extern __shared__ __attribute__((aligned(16))) float sh[];
+    __shared__ float red[NT / 64];
     const int H = p.d.heads, D = p.d.dim, h = blockIdx.x;
-    if (h >= H) { run_side_job(p.side, h - H, red); return; }
-    const int HD = H * D;
-    float* th = sh;                       // tanh(W1 h) [rank]
-    float* r = th + pad_to(p.d.rank, 64);
+    if (h >= H) {
+        if (threadIdx.x < WG) run_side_job(p.side, h - H, red);         // (only sums: no barrier inside)
+        return;
+    }
+    const int HD = H * D, ldw = p.d.w2.ld;
+    float* th = sh;                       // tanh(W1 h) [ldw], zero past rank
+    float* r = th + ldw;
     float* k = r + D;
     float* u = k + D;
     float* w = u + D;
     float* au = w + D;
-    float* part = au + D;                 // [groups][D]
+    float* e = au + D;                    // W2 tanh(W1 h)
+    float* part = e + D;                 // [groups][D]
     const float* z = p.z;
-    const bool fresh = p.state->pos == 0;
-    for (int i = threadIdx.x; i < p.d.rank; i += WG) th[i] = tanhf(z[(size_t)5 * HD + i]);
-    float kk = 0.f;
-    for (int i = threadIdx.x; i < D; i += WG) {
-        r[i] = z[h * D + i];
-        const float x = z[HD + h * D + i];
-        k[i] = x;
-        kk = fmaf(x, x, kk);
-    }
-    const float inv = 1.0f / sqrtf(block_sum(kk, red) + UNIT_EPS);       // (its barriers also publish th, r, k)
-    for (int i = threadIdx.x; i < D; i += WG) {
-        const int c = h * D + i;
-        const unsigned short* w2 = p.d.w2.w + (size_t)c * p.d.w2.ld;
-        float e = p.d.w0[c];
-        for (int j = 0; j < p.d.rank; j++) e = fmaf(bf16_to_f32(w2[j]), th[j], e);
-        w[i] = expf(LOG_DECAY * sigmoid_f(e));
-        u[i] = k[i] * inv;
-        au[i] = sigmoid_f(z[(size_t)4 * HD + c] + p.d.aBias[c]) * u[i];
+    const int groups = NT / D, g = threadIdx.x / D, j = threadIdx.x % D;      // threads past groups * D only help with the vectors
+    const int per = (D + groups - 1) / groups, i0 = g * per, n = g < groups ? min(per, D - i0) : 0;
+    float* S = p.S + (size_t)h * D * D + (size_t)i0 * D + j;
+    float s[PER];
+#pragma unroll
+    for (int c = 0; c < PER; c++) s[c] = c < n ? S[(size_t)c * D] : 0.f;
+    const float v = z[2 * HD + h * D + j];
+    // the vectors of this head
+    const int x = min((int)threadIdx.x, D - 1), cx = h * D + x;
+    const float rx = z[cx], kx = z[HD + cx], ax = z[(size_t)4 * HD + cx] + p.d.aBias[cx], w0x = p.d.w0[cx];
+    const float gx = z[3 * HD + cx], nx = p.d.norm[cx];
+    for (int i = threadIdx.x; i < ldw; i += NT) th[i] = i < p.d.rank ? tanhf(z[(size_t)5 * HD + i]) : 0.f;
+    const bool vec = (int)threadIdx.x < D;
+    if (vec) { r[x] = rx; k[x] = kx; }
+    if (p.state->pos == 0)
+#pragma unroll
+        for (int c = 0; c < PER; c++) s[c] = 0.f;
+    const float inv = 1.0f / sqrtf(block_sum_of<NT>(vec ? kx * kx : 0.f, red) + UNIT_EPS);       // (its barriers also publish th, r, k)
+    // four threads a row of W2
+    for (int row = threadIdx.x >> 2; row < D; row += NT / 4) {
+        const unsigned short* w2 = p.d.w2.w + (size_t)(h * D + row) * ldw;
+        float a = 0.f;
+#pragma unroll 4
+        for (int c8 = threadIdx.x & 3; c8 < ldw >> 3; c8 += 4) {
+            const uint4 q = *reinterpret_cast<const uint4*>(w2 + c8 * 8);
+            const float* t = th + c8 * 8;
+            a = fmaf(bf16_lo(q.x), t[0], a); a = fmaf(bf16_hi(q.x), t[1], a);
+            a = fmaf(bf16_lo(q.y), t[2], a); a = fmaf(bf16_hi(q.y), t[3], a);
+            a = fmaf(bf16_lo(q.z), t[4], a); a = fmaf(bf16_hi(q.z), t[5], a);
+            a = fmaf(bf16_lo(q.w), t[6], a); a = fmaf(bf16_hi(q.w), t[7], a);
+        }
+        a += __shfl_xor(a, 1, 64);
+        a += __shfl_xor(a, 2, 64);
+        if ((threadIdx.x & 3) == 0) e[row] = a;
     }
     __syncthreads();
-    const int cols = D < WG ? D : WG, groups = WG / cols;     // threads past groups * cols idle
-    const int g = threadIdx.x / cols, j0 = threadIdx.x % cols;
-    const bool on = g < groups;
-    const int per = (D + groups - 1) / groups, i0 = g * per, i1 = min(i0 + per, D);
-    float* S = p.S + (size_t)h * D * D;
-    float ss = 0.f;
-    for (int jb = 0; jb < D; jb += cols) {                    // (one pass up to 256 columns)
-        const int j = jb + j0;
-        const bool in = on && j < D;
-        float dot = 0.f;
-        if (in && !fresh)
-            for (int i = i0; i < i1; i++) dot = fmaf(u[i], S[(size_t)i * D + j], dot);
-        if (in) part[g * cols + j0] = dot;
-        __syncthreads();
-        float d = 0.f;
-        if (in) for (int q = 0; q < groups; q++) d += part[q * cols + j0];
-        __syncthreads();
-        float o = 0.f;
-        if (in) {
-            const float v = z[2 * HD + h * D + j];
-            for (int i = i0; i < i1; i++) {
-                const float old = fresh ? 0.f : S[(size_t)i * D + j];
-                const float s = fmaf(k[i], v, fmaf(w[i], old, -au[i] * d));
-                S[(size_t)i * D + j] = s;
-                o = fmaf(r[i], s, o);
-            }
-            part[g * cols + j0] = o;
-        }
-        __syncthreads();
-        if (in && g == 0) {
-            o = 0.f;
-            for (int q = 0; q < groups; q++) o += part[q * cols + j0];
-            p.y[h * D + j] = o;
-            ss = fmaf(o, o, ss);
-        }
-        __syncthreads();
+    if (vec) {
+        const float un = kx * inv;
+        u[x] = un;
+        w[x] = expf(LOG_DECAY * sigmoid_f(e[x] + w0x));
+        au[x] = sigmoid_f(ax) * un;
     }
-    const float rs = 1.0f / sqrtf(block_sum(ss, red) / (float)D + p.d.eps);
-    if (g == 0)
-        for (int j = j0; j < D; j += cols) {                  // (each thread rewrites what it wrote)
-            const int c = h * D + j;
-            p.y[c] = p.y[c] * rs * p.d.norm[c] * sigmoid_f(z[3 * HD + c]);
+    __syncthreads();
+    float dot = 0.f;
+#pragma unroll
+    for (int c = 0; c < PER; c++)
+        if (c < n) dot = fmaf(u[i0 + c], s[c], dot);
+    if (g < groups) part[g * D + j] = dot;
+    __syncthreads();
+    float d = 0.f;
+    if (g < groups)
+        for (int q = 0; q < groups; q++) d += part[q * D + j];
+    __syncthreads();
+    float o = 0.f;
+#pragma unroll
+    for (int c = 0; c < PER; c++)
+        if (c < n) {
+            const int i = i0 + c;
+            s[c] = fmaf(k[i], v, fmaf(w[i], s[c], -au[i] * d));
+            S[(size_t)c * D] = s[c];
+            o = fmaf(r[i], s[c], o);
         }
+    if (g < groups) part[g * D + j] = o;
+    __syncthreads();
+    o = 0.f;
+    if (vec) {
+        for (int q = 0; q < groups; q++) o += part[q * D + x];
+    }
+    const float rs = 1.0f / sqrtf(block_sum_of<NT>(o * o, red) / (float)D + p.d.eps);
+    if (vec) p.y[cx] = o * rs * nx * sigmoid_f(gx);
+}
+template <int NT, int PER>
+static hipError_t run_delta_step(const DeltaStep& p, hipStream_t s) {
+    const size_t lds = ((size_t)p.d.w2.ld + 6 * (size_t)p.d.dim + NT) * 4;
+    if (lds > (60u << 10)) return hipErrorInvalidValue;
+    hipLaunchKernelGGL((delta_step_kernel<NT, PER>), dim3(p.d.heads + p.side.wgs()), dim3(NT), lds, s, p);
+    return hipGetLastError();
 }
 hipError_t launch_delta_step(const DeltaStep& p, hipStream_t s) {
     const int D = p.d.dim;
-    if (!delta_supported(D) || p.d.heads < 1 || p.d.rank < 1 || p.d.w2.ld < p.d.rank) return hipErrorInvalidValue;
-    const size_t lds = ((size_t)pad_to(p.d.rank, 64) + 5 * (size_t)D + WG) * 4;
-    if (lds > (60u << 10)) return hipErrorInvalidValue;
-    hipLaunchKernelGGL(delta_step_kernel, dim3(p.d.heads + p.side.wgs()), dim3(WG), lds, s, p);
-    return hipGetLastError();
+    if (!delta_supported(D) || p.d.heads < 1 || p.d.rank < 1 || p.d.w2.ld < p.d.rank || p.d.w2.ld % 64 || p.side.z) return hipErrorInvalidValue;
+    if (D <= 64) return run_delta_step<256, 16>(p, s);        // at least 256 / D groups of at most 16 channels
+    if (D <= 128) return run_delta_step<1024, 16>(p, s);
+    return run_delta_step<1024, 64>(p, s);
 }
 
 // ---------------------------------------------------------------------------

@@ -14,7 +14,7 @@
 namespace mg {
 
 struct LatentDecode {
-    const float* qlat = nullptr;     // [T, heads, rank]: W_uk^T q
+    const float* qlat = nullptr;     // [T, heads, rankPad]: W_uk^T q (past rank any finite value: cache rows are zero there)
     const float* q = nullptr;        // [T, heads, headW]: the rotated part (not turned yet) from column ropeOff of a head
     int headW = 0, ropeOff = 0;
     LatentCache cache;

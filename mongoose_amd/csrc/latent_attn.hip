@@ -71,18 +71,40 @@ __global__ __launch_bounds__(LNW * 64) void latent_decode_kernel(LatentDecode p)
     const LatentCache& c = p.cache;
     const int e0 = lane * V;
     const bool own = e0 < c.rankPad;
+    // queries: every load is requested before the first is used
     float ql[LHG][V], qr[LHG][2];
     {
         const size_t tr = (size_t)pos * (c.ropeDims >> 1);
+        float cs[2], sn[2], qa[LHG][2], qb[LHG][2];
+#pragma unroll
+        for (int i = 0; i < 2; i++) {
+            const int d = min(lane + 64 * i, c.rot - 1), turn = min(d, c.ropeDims - 1) >> 1;
+            const bool any = c.ropeDims > 0;
+            cs[i] = any ? c.cosTab[tr + turn] : 1.f;
+            sn[i] = any ? c.sinTab[tr + turn] : 0.f;
+        }
 #pragma unroll
         for (int h = 0; h < LHG; h++) {
             const size_t hd = (size_t)t * p.heads + h0 + min(h, nh - 1);
+            LatentVec<float, V>::load(p.qlat + hd * c.rankPad + (own ? e0 : 0), ql[h]);
+            const float* qp = p.q + hd * p.headW + p.ropeOff;
 #pragma unroll
-            for (int i = 0; i < V; i++) ql[h][i] = e0 + i < c.rank ? p.qlat[hd * c.rank + e0 + i] : 0.f;
+            for (int i = 0; i < 2; i++) {
+                const int d = max(min(lane + 64 * i, c.rot - 1), 0), e = min(d ^ 1, max(c.rot - 1, 0));
+                qa[h][i] = qp[d];
+                qb[h][i] = qp[e];
+            }
+        }
+#pragma unroll
+        for (int h = 0; h < LHG; h++) {
+            if (!own)
+#pragma unroll
+                for (int i = 0; i < V; i++) ql[h][i] = 0.f;
 #pragma unroll
             for (int i = 0; i < 2; i++) {
                 const int d = lane + 64 * i;
-                qr[h][i] = d < c.rot ? rotated_element(p.q + hd * p.headW + p.ropeOff, d, c.ropeDims, c.cosTab + tr, c.sinTab + tr) : 0.f;
+                const float turned = (d & 1) ? qa[h][i] * cs[i] + qb[h][i] * sn[i] : qa[h][i] * cs[i] - qb[h][i] * sn[i];
+                qr[h][i] = d >= c.rot ? 0.f : d < c.ropeDims ? turned : qa[h][i];
             }
         }
     }
@@ -94,18 +116,30 @@ __global__ __launch_bounds__(LNW * 64) void latent_decode_kernel(LatentDecode p)
         for (int i = 0; i < V; i++) acc[h][i] = 0.f;
     }
     const CT* rows = static_cast<const CT*>(c.rows);
-    for (int kb = k0 + wave * LKB; kb < k1; kb += LNW * LKB) {
-        float kv[LKB][V], kr[LKB][2];
+    // keys a batch ahead of their use (but for the widest rows, whose registers that would spill)
+    constexpr bool AHEAD = V <= 8;
+    float kvN[LKB][V], krN[LKB][2];
+    auto fetch = [&](int kb) __attribute__((always_inline)) {
 #pragma unroll
         for (int k = 0; k < LKB; k++) {
             const CT* row = rows + (size_t)min(kb + k, k1 - 1) * c.stride;
-            if (own) LatentVec<CT, V>::load(row + e0, kv[k]);
-            else
+            LatentVec<CT, V>::load(row + (own ? e0 : 0), kvN[k]);
 #pragma unroll
-                for (int i = 0; i < V; i++) kv[k][i] = 0.f;
-#pragma unroll
-            for (int i = 0; i < 2; i++) kr[k][i] = lane + 64 * i < c.rot ? load_act(row + c.rankPad + lane + 64 * i) : 0.f;
+            for (int i = 0; i < 2; i++) krN[k][i] = load_act(row + c.rankPad + max(min(lane + 64 * i, c.rot - 1), 0));
         }
+    };
+    if (AHEAD) fetch(k0 + wave * LKB);
+    for (int kb = k0 + wave * LKB; kb < k1; kb += LNW * LKB) {
+        if (!AHEAD) fetch(kb);
+        float kv[LKB][V], kr[LKB][2];
+#pragma unroll
+        for (int k = 0; k < LKB; k++) {
+#pragma unroll
+            for (int i = 0; i < V; i++) kv[k][i] = own ? kvN[k][i] : 0.f;
+#pragma unroll
+            for (int i = 0; i < 2; i++) kr[k][i] = krN[k][i];          // (past rot the query's part is zero)
+        }
+        if (AHEAD && kb + LNW * LKB < k1) fetch(kb + LNW * LKB);
         float s[LKB][LHG];
 #pragma unroll
         for (int k = 0; k < LKB; k++)
@@ -179,10 +213,10 @@ static int latent_lane_elems(int rankPad) {
 bool latent_decode_supported(int rank, int rot) { return rank >= 1 && latent_lane_elems(pad_to(rank, 64)) <= 16 && rot >= 0 && rot <= 128; }
 
 void latent_decode_splits(int span, int heads, int T, int* splits, int* splitLen) {
-    // one batch of keys a wave at least; at most 32 partial results for the consumer to merge
+    // one batch of keys a wave at least; at most 16 partial results for the consumer to merge
     const int groups = (heads + LHG - 1) / LHG;
     int n = std::max(1, 512 / std::max(1, groups * T));
-    n = std::min({n, 32, (span + LNW * LKB - 1) / (LNW * LKB)});
+    n = std::min({n, 16, (span + LNW * LKB - 1) / (LNW * LKB)});
     n = std::max(n, 1);
     *splitLen = pad_to((span + n - 1) / n, LNW * LKB);
     *splits = (span + *splitLen - 1) / *splitLen;

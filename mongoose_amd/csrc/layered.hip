@@ -213,7 +213,7 @@ int LayeredInference::build(const mg_layer_desc* descs) {
             L.down = mat(dim, d.ff); wantMat(L.down, d.experts);
             L.upStride = (size_t)L.up.rows * L.up.ld;
             L.downStride = (size_t)L.down.rows * L.down.ld;
-            L.gate = mat(d.experts + d.ff_shared, dim); wantMat(L.gate);
+            L.gate = mat(pad_to(d.experts, 4) + d.ff_shared, dim); wantMat(L.gate);
             if (d.ff_shared) { L.downShared = mat(dim, d.ff_shared); wantMat(L.downShared); }
             L.act.kind = ACT_GELU;
         }
@@ -246,7 +246,7 @@ int LayeredInference::build(const mg_layer_desc* descs) {
             TensorSlot& wo = addMat(mx + "o", L.out, 0, dim, d.heads * d.vdim);
             wo.colMap = {d.vdim, L.vPad, d.vdim, 0};
             qMax = std::max(qMax, (size_t)L.uq.rows);
-            qlatMax = std::max(qlatMax, (size_t)d.heads * d.kv_rank);
+            qlatMax = std::max(qlatMax, (size_t)d.heads * L.cache.rankPad);
             oMax = std::max(oMax, (size_t)d.heads * L.vPad);
             paccMax = std::max(paccMax, (size_t)d.heads * L.splits * L.cache.rankPad);
             pmMax = std::max(pmMax, (size_t)d.heads * L.splits);
@@ -277,11 +277,11 @@ int LayeredInference::build(const mg_layer_desc* descs) {
             }
             addMat(ml + "router", L.gate, 0, d.experts, dim);
             if (d.ff_shared) {
-                addMat(ml + "shared.up", L.gate, d.experts, d.ff_shared, dim);
+                addMat(ml + "shared.up", L.gate, pad_to(d.experts, 4), d.ff_shared, dim);
                 addMat(ml + "shared.down", L.downShared, 0, dim, d.ff_shared);
             }
-            gateMax = std::max(gateMax, (size_t)L.gate.rows);
-            hidMax = std::max(hidMax, (size_t)d.top * d.ff);
+            gateMax = std::max(gateMax, (size_t)pad_to(d.experts, 4) + L.downShared.ld);
+            hidMax = std::max(hidMax, (size_t)d.top * L.down.ld);
         }
     }
     {
@@ -458,7 +458,7 @@ int LayeredInference::enqueueLatent(LayerBlock& L, const VecInput& in, const flo
     // the query moves into the latent's space; the same launch writes this position's cache row
     HeadMv a;
     a.src = q; a.rowStride = L.uq.rows; a.headStride = L.headW; a.K = d.dim;
-    a.w = L.ukT; a.heads = d.heads; a.rows = d.kv_rank; a.ld = L.ldUkT; a.out = qlat;
+    a.w = L.ukT; a.heads = d.heads; a.rows = d.kv_rank; a.ld = L.ldUkT; a.out = qlat; a.ldOut = L.cache.rankPad;
     a.side = dwa;
     if (d.kv_from < 0) { a.side.cache = L.cache; a.side.z = z + d.q_rank; a.side.gain = L.kvNorm; a.side.eps = eps; }
     HIPCHK(launch_head_matvec(a, stream));
@@ -471,7 +471,7 @@ int LayeredInference::enqueueLatent(LayerBlock& L, const VecInput& in, const flo
     if (mark(3)) return MG_E_HIP;
     HeadMv v;
     v.K = d.kv_rank; v.pacc = pacc; v.pm = pm; v.pl = pl; v.splits = L.splits; v.accLd = L.cache.rankPad;
-    v.w = L.uv.w; v.heads = d.heads; v.rows = L.vPad; v.ld = L.uv.ld; v.out = o;
+    v.w = L.uv.w; v.heads = d.heads; v.rows = L.vPad; v.ld = L.uv.ld; v.out = o; v.ldOut = L.vPad;
     HIPCHK(launch_head_matvec(v, stream));
     m = MvBf16();
     m.in.src = o; m.in.n = d.heads * L.vPad;
@@ -514,18 +514,18 @@ int LayeredInference::enqueueMlp(LayerBlock& L) {
         HIPCHK(launch_matvec_bf16(m, nullptr, stream));
         return MG_OK;
     }
-    m.in = in; m.w = L.gate; m.act = L.act; m.actFrom = d.experts; m.out = gateOut;
+    m.in = in; m.w = L.gate; m.act = L.act; m.actFrom = pad_to(d.experts, 4); m.out = gateOut;
     HIPCHK(launch_matvec_bf16(m, nullptr, stream));
     m = MvBf16();
     m.in.src = x1; m.in.n = dim;
     m.w = L.up; m.act = L.act; m.out = hid;
-    m.routerLogits = gateOut; m.experts = d.experts; m.top = d.top; m.expertStride = L.upStride;
+    m.routerLogits = gateOut; m.experts = d.experts; m.top = d.top; m.expertStride = L.upStride; m.ldOut = L.down.ld;
     HIPCHK(launch_matvec_bf16(m, nullptr, stream));
     if (mark(5)) return MG_E_HIP;
     MvMoeDown p;
-    p.routerLogits = gateOut; p.experts = d.experts; p.top = d.top; p.hid = hid; p.ff = d.ff;
+    p.routerLogits = gateOut; p.experts = d.experts; p.top = d.top; p.hid = hid; p.ldHid = L.down.ld;
     p.down = L.down; p.expertStride = L.downStride;
-    p.hidShared = gateOut + d.experts; p.ffShared = d.ff_shared; p.downShared = L.downShared;
+    p.hidShared = gateOut + pad_to(d.experts, 4); p.downShared = L.downShared;
     p.resid = x1; p.alpha = alpha; p.out = y2;
     HIPCHK(launch_moe_down(p, stream));
     return MG_OK;
@@ -601,7 +601,7 @@ int LayeredInference::ensureRows(int rows, int pos0) {
             cq = std::max(cq, (size_t)L.uq.ld);
             qMax = std::max(qMax, (size_t)L.uq.rows);
             const size_t rowsA = L.expanded ? EXPANDED_MIN_ROWS : T, groups = (d.heads + 3) / 4;
-            qlat = std::max(qlat, rowsA * d.heads * d.kv_rank);
+            qlat = std::max(qlat, rowsA * d.heads * L.cache.rankPad);
             const size_t parts = 4 * std::max<size_t>(512, groups * rowsA);
             pacc = std::max(pacc, parts * L.cache.rankPad);
             pms = std::max(pms, parts);
@@ -687,7 +687,7 @@ int LayeredInference::rowsLatent(LayerBlock& L, int T, int pos0) {
         HIPCHK(launch_gemm_bf16w(g, stream));
         HeadMv a;
         a.src = rQf; a.rowStride = L.uq.rows; a.headStride = L.headW; a.K = d.dim;
-        a.w = L.ukT; a.heads = d.heads; a.rows = d.kv_rank; a.ld = L.ldUkT; a.out = rQlat; a.T = T;
+        a.w = L.ukT; a.heads = d.heads; a.rows = d.kv_rank; a.ld = L.ldUkT; a.out = rQlat; a.ldOut = L.cache.rankPad; a.T = T;
         HIPCHK(launch_head_matvec(a, stream));
         LatentDecode p;
         p.qlat = rQlat; p.q = rQf; p.headW = L.headW; p.ropeOff = L.dimPad; p.cache = L.cache;
@@ -738,7 +738,7 @@ int LayeredInference::rowsMlp(LayerBlock& L, int T, NormRows& after) {
     const int ldg = pad_to(d.experts, 4);
     g.A = aX1; g.f32 = f32; g.lda = widthPad; g.M = T;
     g.W = L.gate.w; g.ldw = L.gate.ld; g.N = L.gate.rows; g.K = L.gate.ld;
-    g.mode = GEMM_SPLIT; g.nSplit = d.experts; g.out = rGate; g.ldc = ldg;
+    g.mode = GEMM_SPLIT; g.nSplit = ldg; g.out = rGate; g.ldc = ldg;
     g.outAct = aShared; g.ldo = L.downShared.ld; g.act = L.act;
     HIPCHK(launch_gemm_bf16w(g, stream));
     MoeRoute r;

@@ -48,10 +48,11 @@ struct MvBf16 {
     float* amaxVal = nullptr;        // MV_ARGMAX: one (max, index) per workgroup
     int* amaxIdx = nullptr;
     // mixture of experts, expert s of the chosen ones in grid row s: w is expert 0, expert e lies expertStride
-    // elements further; out is [top, w.rows]
+    // elements further; out is [top, ldOut]
     const float* routerLogits = nullptr;
     int experts = 0, top = 0;
     size_t expertStride = 0;
+    int ldOut = 0;
 };
 hipError_t launch_matvec_bf16(const MvBf16& p, int* gridOut, hipStream_t s);
 
@@ -59,12 +60,11 @@ hipError_t launch_matvec_bf16(const MvBf16& p, int* gridOut, hipStream_t s);
 struct MvMoeDown {
     const float* routerLogits = nullptr;
     int experts = 0, top = 0;
-    const float* hid = nullptr;      // [top, ff]
-    int ff = 0;
+    const float* hid = nullptr;      // [top, ldHid], ldHid >= down.ld (finite past the expert's size)
+    int ldHid = 0;
     Bf16Mat down;                    // expert 0
     size_t expertStride = 0;
-    const float* hidShared = nullptr;
-    int ffShared = 0;
+    const float* hidShared = nullptr;    // 16-byte aligned, readable up to downShared.ld
     Bf16Mat downShared;              // rows 0: none
     const float* resid = nullptr;
     float alpha = 0.f;
@@ -85,7 +85,8 @@ struct HeadMv {
     int splits = 0, accLd = 0;
     const unsigned short* w = nullptr;   // [heads, rows, ld]
     int heads = 0, rows = 0, ld = 0;
-    float* out = nullptr;            // [T, heads, rows]  (fp32), or
+    float* out = nullptr;            // [T, heads, ldOut] (fp32; ldOut >= rows), or
+    int ldOut = 0;
     void* outAct = nullptr;          // the same as activations (bf16 or fp32) with rows of ldAct
     int actF32 = 0, ldAct = 0;
     int T = 1;

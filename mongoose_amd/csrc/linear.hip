@@ -47,7 +47,7 @@ __global__ __launch_bounds__(WG) void matvec_bf16_kernel(MvBf16 p) {
         if (wave == 0) choose_experts(p.routerLogits, p.experts, p.top, ids, wts);
         __syncthreads();
         W += (size_t)ids[blockIdx.y] * p.expertStride;
-        p.out += (size_t)blockIdx.y * N;
+        p.out += (size_t)blockIdx.y * p.ldOut;
     }
     // load cursor (lg, lc) and use cursor (g, c) over (row group, chunk)
     int g = blockIdx.x * 4 + wave, lg = g, lc = 0;
@@ -69,11 +69,14 @@ __global__ __launch_bounds__(WG) void matvec_bf16_kernel(MvBf16 p) {
     const int last8 = (Kp >> 3) - 1;
     float best = -INFINITY;
     int besti = INT_MAX;
-    float acc[NR];
+    float acc[NR], res[NR];
 #pragma unroll
-    for (int r = 0; r < NR; r++) acc[r] = 0.f;
+    for (int r = 0; r < NR; r++) { acc[r] = 0.f; res[r] = 0.f; }
     int c = 0;
     while (g < groups) {
+        if (c == 0 && p.epi == MV_RESID)
+#pragma unroll
+            for (int r = 0; r < NR; r++) res[r] = p.resid[min(g * NR + r, N - 1)];
 #pragma unroll
         for (int d = 0; d < DEP; d++) {
             if (g >= groups) break;
@@ -90,7 +93,7 @@ __global__ __launch_bounds__(WG) void matvec_bf16_kernel(MvBf16 p) {
                     acc[r] = 0.f;
                     if (row < N) {
                         if (p.act.kind && row >= p.actFrom) v = apply_act(v, p.act);
-                        if (p.epi == MV_RESID) v = fmaf(p.alpha, p.resid[row], v);
+                        if (p.epi == MV_RESID) v = fmaf(p.alpha, res[r], v);
                         if (lane == 0) p.out[row] = v;
                         if (v > best) { best = v; besti = row; }
                     }
@@ -125,53 +128,88 @@ hipError_t launch_matvec_bf16(const MvBf16& p, int* gridOut, hipStream_t s) {
         return hipErrorInvalidValue;
     const size_t lds = (size_t)p.w.ld * 4;
     if (lds > (144u << 10)) return hipErrorInvalidValue;
-    const int rows = p.w.rows * (p.top ? p.top : 1);
-    const int nr = rows >= 16384 ? 4 : rows >= 6144 ? 2 : 1;
+    // Workgroups that are all resident at once (a second round would start cold) and stay for several row groups.
+    const int slices = p.top ? p.top : 1;
+    const int nr = p.w.rows * slices >= 24576 ? 2 : 1;
     const int groups = (p.w.rows + nr - 1) / nr;
-    int grid = (groups + 3) / 4;
-    // workgroups that stay for several row groups share one staging of the vector
-    const int cap = p.top ? std::max(1, 2048 / p.top) : 2048;
-    if (grid > cap) grid = cap;
+    const int perCu = std::max(1, std::min(4, (int)((160u << 10) / (lds + 512))));
+    const int grid = std::min((groups + 3) / 4, std::max(1, 256 * perCu / slices));
     if (gridOut) *gridOut = grid;
-    if (nr == 4) return run_matvec<4, 2>(p, grid, lds, s);
     if (nr == 2) return run_matvec<2, 4>(p, grid, lds, s);
-    return run_matvec<1, 4>(p, grid, lds, s);
+    return run_matvec<1, 8>(p, grid, lds, s);
 }
 
-// One wave a row of the output: the chosen experts' rows one after the other, then the shared expert's.
+// One wave a row of the output: the chosen experts' rows one after the other, then the shared expert's, as one stream
+// of 512-weight chunks with a ring of loads in flight that starts before the hidden vectors are staged.
 __global__ __launch_bounds__(WG) void moe_down_kernel(MvMoeDown p) {
+    constexpr int DEP = 8;
     extern __shared__ __attribute__((aligned(16))) float act[];       // [top][ld], [ldShared]
     __shared__ int ids[MAX_TOP];
     __shared__ float wts[MAX_TOP];
-    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int Kp = p.down.ld, Ks = p.downShared.rows ? p.downShared.ld : 0;
+    const int row = min((int)blockIdx.x * 4 + wave, p.down.rows - 1);
+    const int ncE = (Kp + 511) >> 9, ncS = (Ks + 511) >> 9, total = p.top * ncE + ncS;
+    const float res = p.resid[row];
     if (wave == 0) choose_experts(p.routerLogits, p.experts, p.top, ids, wts);
     __syncthreads();
-    for (int s = 0; s < p.top; s++)
-        for (int i = threadIdx.x; i < Kp; i += WG)
-            act[s * Kp + plane_index(i, Kp >> 3)] = i < p.ff ? wts[s] * p.hid[(size_t)s * p.ff + i] : 0.f;
-    for (int i = threadIdx.x; i < Ks; i += WG)
-        act[p.top * Kp + plane_index(i, Ks >> 3)] = i < p.ffShared ? p.hidShared[i] : 0.f;
+    uint4 ring[DEP];
+    int ls = 0, lc = 0;                                               // load cursor: segment (top = the shared expert), chunk
+    auto issue = [&](uint4& slot) __attribute__((always_inline)) {
+        const bool sh = ls == p.top;
+        const int ld = sh ? Ks : Kp, col = lc * 512 + lane * 8;
+        const unsigned short* w = sh ? p.downShared.w + (size_t)row * Ks
+                                     : p.down.w + (size_t)ids[min(ls, p.top - 1)] * p.expertStride + (size_t)row * Kp;
+        slot = ls <= p.top && col < ld ? *reinterpret_cast<const uint4*>(w + col) : make_uint4(0, 0, 0, 0);
+        if (++lc >= (sh ? ncS : ncE)) { lc = 0; ls++; }
+    };
+#pragma unroll
+    for (int d = 0; d < DEP; d++) issue(ring[d]);
+    // staged four floats at a time, eight of them in flight; past the real lengths the vectors hold finite values and
+    // the weights zeros
+    {
+        const int kq = Kp >> 2, sq = Ks >> 2, quads = p.top * kq + sq;
+        int seg = 0, q = threadIdx.x;
+        for (int i0 = threadIdx.x; i0 < quads; i0 += 8 * WG) {
+            float4 v[8];
+            int at[8];
+#pragma unroll
+            for (int k = 0; k < 8; k++) {
+                while (seg < p.top && q >= kq) { q -= kq; seg++; }
+                const bool on = i0 + k * WG < quads;
+                const float* src = seg < p.top ? p.hid + (size_t)seg * p.ldHid : p.hidShared;
+                v[k] = on ? reinterpret_cast<const float4*>(src)[q] : make_float4(0.f, 0.f, 0.f, 0.f);
+                const float w = seg < p.top ? wts[seg] : 1.0f;
+                v[k].x *= w; v[k].y *= w; v[k].z *= w; v[k].w *= w;
+                at[k] = on ? seg * kq + (q & 1) * ((seg < p.top ? Kp : Ks) >> 3) + (q >> 1) : -1;
+                q += WG;
+            }
+#pragma unroll
+            for (int k = 0; k < 8; k++)
+                if (at[k] >= 0) reinterpret_cast<float4*>(act)[at[k]] = v[k];
+        }
+    }
     __syncthreads();
-    const int row = blockIdx.x * 4 + wave;
-    if (row >= p.down.rows) return;
     float acc = 0.f;
-    for (int s = 0; s <= p.top; s++) {
-        const bool sh = s == p.top;
-        const int ld = sh ? Ks : Kp;
-        if (!ld) break;
-        const unsigned short* w = sh ? p.downShared.w + (size_t)row * ld
-                                     : p.down.w + (size_t)__builtin_amdgcn_readfirstlane(ids[s]) * p.expertStride + (size_t)row * ld;
-        const float4* lo = reinterpret_cast<const float4*>(act + s * Kp);
-        const float4* hi = lo + (ld >> 3);
-#pragma unroll 4
-        for (int c8 = lane; c8 < ld >> 3; c8 += 64) acc = dot8(*reinterpret_cast<const uint4*>(w + c8 * 8), lo, hi, c8, acc);
+    int us = 0, uc = 0, n = 0;
+    while (n < total) {
+#pragma unroll
+        for (int d = 0; d < DEP; d++) {
+            if (n >= total) break;
+            const bool sh = us == p.top;
+            const int nc8 = (sh ? Ks : Kp) >> 3;
+            const float4* lo = reinterpret_cast<const float4*>(act + us * Kp);
+            acc = dot8(ring[d], lo, lo + nc8, min(uc * 64 + lane, nc8 - 1), acc);
+            issue(ring[d]);
+            if (++uc == (sh ? ncS : ncE)) { uc = 0; us++; }
+            n++;
+        }
     }
     acc = wave_sum(acc);
-    if (lane == 0) p.out[row] = fmaf(p.alpha, p.resid[row], acc);
+    if (lane == 0 && (int)blockIdx.x * 4 + wave < p.down.rows) p.out[row] = fmaf(p.alpha, res, acc);
 }
 hipError_t launch_moe_down(const MvMoeDown& p, hipStream_t s) {
-    if (p.top < 1 || p.top > MAX_TOP || p.experts > MAX_EXPERTS || p.down.ld % 64 || p.ff > p.down.ld) return hipErrorInvalidValue;
+    if (p.top < 1 || p.top > MAX_TOP || p.experts > MAX_EXPERTS || p.down.ld % 64 || p.ldHid < p.down.ld) return hipErrorInvalidValue;
     const size_t lds = ((size_t)p.top * p.down.ld + (p.downShared.rows ? p.downShared.ld : 0)) * 4;
     if (lds > (144u << 10)) return hipErrorInvalidValue;
     if (lds > (48u << 10)) {
@@ -194,21 +232,42 @@ __global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG
     }
     const int ld = p.ld, nc8 = ld >> 3;
     if (p.splits) {
-        // out = sum_s e^(m_s - M) acc_s / sum_s e^(m_s - M) l_s; a split that saw no key has m = -inf
+        // out = sum_s e^(m_s - M) acc_s / sum_s e^(m_s - M) l_s; a split that saw no key has m = -inf.  A thread takes
+        // four consecutive elements of every gs-th split.
         const size_t b = ((size_t)t * p.heads + h) * p.splits;
-        float M = -INFINITY;
-        for (int s = 0; s < p.splits; s++) M = fmaxf(M, p.pm[b + s]);
-        float L = 0.f;
-        for (int s = 0; s < p.splits; s++) L += p.pm[b + s] == -INFINITY ? 0.f : expf(p.pm[b + s] - M) * p.pl[b + s];
-        const float inv = 1.0f / L;
-        for (int i = threadIdx.x; i < ld; i += WG) {
-            float v = 0.f;
-            if (i < p.K)
-                for (int s = 0; s < p.splits; s++) {
-                    const float m = p.pm[b + s];
-                    if (m != -INFINITY) v = fmaf(expf(m - M), p.pacc[(b + s) * p.accLd + i], v);
+        float* f = act + ld;                                  // [splits] factors
+        float4* part = reinterpret_cast<float4*>(act + ld + 64);
+        if (threadIdx.x < 64) {
+            const int s = threadIdx.x;
+            const float m = s < p.splits ? p.pm[b + s] : -INFINITY, l = s < p.splits ? p.pl[b + s] : 0.f;
+            const float M = wave_max(m);
+            const float e = m == -INFINITY ? 0.f : expf(m - M);
+            const float L = wave_sum(e * l);
+            f[s] = e / L;
+        }
+        __syncthreads();
+        const int nq = ld >> 2, gs = nq < WG ? WG / nq : 1;
+        for (int q0 = 0; q0 < nq; q0 += WG) {
+            const int q = nq < WG ? (int)threadIdx.x % nq : q0 + (int)threadIdx.x, g = nq < WG ? (int)threadIdx.x / nq : 0;
+            float4 v = make_float4(0.f, 0.f, 0.f, 0.f);
+            const bool on = g < gs && q < nq && 4 * q < p.accLd;
+            if (on)
+#pragma unroll 8
+                for (int s = g; s < p.splits; s += gs) {
+                    const float w = f[s];                     // (0 for a split without keys, whose sums are finite leftovers)
+                    const float4 a = *reinterpret_cast<const float4*>(p.pacc + (b + s) * p.accLd + 4 * q);
+                    v.x = fmaf(w, a.x, v.x); v.y = fmaf(w, a.y, v.y); v.z = fmaf(w, a.z, v.z); v.w = fmaf(w, a.w, v.w);
                 }
-            act[plane_index(i, nc8)] = v * inv;
+            if (gs > 1) {
+                if (g < gs) part[g * nq + q] = v;
+                __syncthreads();
+                if (g == 0)
+                    for (int k = 1; k < gs; k++) {
+                        const float4 a = part[k * nq + q];
+                        v.x += a.x; v.y += a.y; v.z += a.z; v.w += a.w;
+                    }
+            }
+            if (g == 0 && q < nq) reinterpret_cast<float4*>(act)[(q & 1) * nc8 + (q >> 1)] = v;
         }
     } else {
         const float* src = p.src + (size_t)t * p.rowStride + (size_t)h * p.headStride;
@@ -229,7 +288,7 @@ __global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG
         }
         for (int o = lpr >> 1; o > 0; o >>= 1) acc += __shfl_xor(acc, o, 64);
         if (sub == 0 && row < r1) {
-            if (p.out) p.out[((size_t)t * p.heads + h) * p.rows + row] = acc;
+            if (p.out) p.out[((size_t)t * p.heads + h) * p.ldOut + row] = acc;
             if (p.outAct) {
                 const size_t o = (size_t)t * p.ldAct + (size_t)h * p.rows + row;
                 if (p.actF32) static_cast<float*>(p.outAct)[o] = acc;
@@ -240,13 +299,16 @@ __global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG
 }
 hipError_t launch_head_matvec(const HeadMv& p, hipStream_t s) {
     if (p.T < 1) return hipSuccess;
-    if (p.side.wgs() && p.T != 1) return hipErrorInvalidValue;
-    if (p.ld % 64 || p.K > p.ld || p.rows < 1 || (size_t)p.ld * 4 > (48u << 10)) return hipErrorInvalidValue;
+    if ((p.side.wgs() && p.T != 1) || (p.out && p.ldOut < p.rows)) return hipErrorInvalidValue;
+    if (p.ld % 64 || p.K > p.ld || p.rows < 1 || (size_t)p.ld * 4 > (40u << 10)) return hipErrorInvalidValue;
     int lprLog2 = 3;
     while (lprLog2 < 6 && (8 << lprLog2) < p.ld) lprLog2++;
     // enough workgroups for the chip at one row t; a workgroup's staging is worth some rows
     const int slots = WG >> lprLog2;
     int rowsPerWG = pad_to((p.rows * p.heads * p.T + 511) / 512, slots);
+    if (p.splits > 4) rowsPerWG = std::max(rowsPerWG, pad_to(16, slots));          // (merging the splits is the larger part)
+    const size_t lds = ((size_t)p.ld + (p.splits ? 64 + 4 * WG : 0)) * 4;
+    if (p.splits > 64) return hipErrorInvalidValue;
     if (rowsPerWG < slots) rowsPerWG = slots;
     if (rowsPerWG > pad_to(p.rows, slots)) rowsPerWG = pad_to(p.rows, slots);
     for (int t0 = 0; t0 < p.T; t0 += 32768) {
@@ -255,10 +317,10 @@ hipError_t launch_head_matvec(const HeadMv& p, hipStream_t s) {
         if (q.src) q.src += (size_t)t0 * p.rowStride;
         const size_t b = (size_t)t0 * p.heads * p.splits;
         if (q.splits) { q.pacc += b * p.accLd; q.pm += b; q.pl += b; }
-        if (q.out) q.out += (size_t)t0 * p.heads * p.rows;
+        if (q.out) q.out += (size_t)t0 * p.heads * p.ldOut;
         if (q.outAct) q.outAct = static_cast<char*>(p.outAct) + (size_t)t0 * p.ldAct * (p.actF32 ? 4 : 2);
         const int gx = (p.rows + rowsPerWG - 1) / rowsPerWG;
-        hipLaunchKernelGGL(head_matvec_kernel, dim3(gx, p.heads + (p.side.wgs() + gx - 1) / gx, q.T), dim3(WG), (size_t)p.ld * 4, s, q, rowsPerWG, lprLog2);
+        hipLaunchKernelGGL(head_matvec_kernel, dim3(gx, p.heads + (p.side.wgs() + gx - 1) / gx, q.T), dim3(WG), lds, s, q, rowsPerWG, lprLog2);
         hipError_t e = hipGetLastError();
         if (e != hipSuccess) return e;
     }
@@ -358,11 +420,13 @@ __device__ __forceinline__ bool find_tile(const Gemm& g, TileAt& t) {
     return true;
 }
 
-// bf16 activations.  BM rows x BN columns, 4 waves as 2 x 2, K in steps of 64 through two LDS buffers filled by direct
-// global -> LDS loads.  LDS rows are 128 bytes (64 k); the 16-byte piece q of row r lies at q ^ (r & 7).
-template <int BM, int BN>
+// bf16 activations.  BM rows x BN columns, 4 waves (MW along the rows), K in steps of 64 through a ring of ST LDS buffers
+// filled by direct global -> LDS loads, ST - 1 steps ahead.  LDS rows are 128 bytes (64 k); the 16-byte piece q of row r
+// lies at q ^ (r & 7).
+template <int BM, int BN, int MW, int ST>
 __global__ __launch_bounds__(256) void gemm_bf16_kernel(Gemm g) {
-    constexpr int WM = BM / 64, WN = BN / 64;            // 32 x 32 blocks a wave: rows, columns
+    constexpr int NW = 4 / MW;
+    constexpr int WM = BM / (32 * MW), WN = BN / (32 * NW);     // 32 x 32 blocks a wave: rows, columns
     constexpr int ABYTES = BM * 128, BUF = (BM + BN) * 128;
     constexpr int LOADS = (BM + BN) / 32;                // wave-loads (8 rows of 128 bytes) a wave issues a step
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
@@ -400,14 +464,20 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(Gemm g) {
         for (int b = 0; b < WM; b++)
 #pragma unroll
             for (int e = 0; e < 16; e++) acc[a][b][e] = 0.f;
-    const int wm = (wave & 1) * (BM / 2), wn = (wave >> 1) * (BN / 2);
+    const int wm = (wave % MW) * (BM / MW), wn = (wave / MW) * (BN / NW);
     const int fr = lane & 31, fh = lane >> 5;
     const int steps = g.K >> 6;
-    issue(0, 0);
+#pragma unroll
+    for (int i = 0; i < ST - 1; i++)
+        if (i < steps) issue(i, i);
+    int buf = 0;
     for (int st = 0; st < steps; st++) {
-        asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
-        if (st + 1 < steps) issue(st + 1, (st + 1) & 1);
-        const unsigned char* base = lds + (st & 1) * BUF;
+        // this step's buffer has landed (the loads of up to ST - 2 later steps stay in flight); the one before it is free
+        if (ST > 2 && st + ST - 2 < steps) asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)\n\ts_barrier" ::"n"((ST - 2) * LOADS) : "memory");
+        else asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+        if (st + ST - 1 < steps) issue(st + ST - 1, buf == 0 ? ST - 1 : buf - 1);
+        const unsigned char* base = lds + buf * BUF;
+        buf = buf == ST - 1 ? 0 : buf + 1;
 #pragma unroll
         for (int ks = 0; ks < 4; ks++) {
             const int piece = 2 * ks + fh;
@@ -498,10 +568,10 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(Gemm g) {
     }
 }
 
-template <int BM, int BN>
+template <int BM, int BN, int MW, int ST>
 static hipError_t run_gemm_bf16(const Gemm& g, hipStream_t s) {
-    const size_t lds = (size_t)(BM + BN) * 128 * 2;
-    auto k = gemm_bf16_kernel<BM, BN>;
+    const size_t lds = (size_t)(BM + BN) * 128 * ST;
+    auto k = gemm_bf16_kernel<BM, BN, MW, ST>;
     if (lds > (48u << 10)) {
         hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
@@ -522,10 +592,11 @@ hipError_t launch_gemm_bf16w(const Gemm& g, hipStream_t s) {
         return hipGetLastError();
     }
     if (g.wF32) return hipErrorInvalidValue;
-    if (g.tiles) return g.N >= 512 ? run_gemm_bf16<MOE_TILE_ROWS, 128>(g, s) : run_gemm_bf16<MOE_TILE_ROWS, 64>(g, s);
+    if (g.tiles) return g.N >= 512 ? run_gemm_bf16<MOE_TILE_ROWS, 256, 1, 2>(g, s) : run_gemm_bf16<MOE_TILE_ROWS, 64, 2, 3>(g, s);
     const long big = (long)((g.M + 127) / 128) * ((g.N + 127) / 128);
-    if (big >= 192) return run_gemm_bf16<128, 128>(g, s);
-    return run_gemm_bf16<64, 64>(g, s);
+    if (big > 320) return run_gemm_bf16<128, 128, 2, 2>(g, s);       // two workgroups a CU cover each other's waits
+    if (big >= 160) return run_gemm_bf16<128, 128, 2, 4>(g, s);      // about one a CU: loads three steps ahead instead
+    return run_gemm_bf16<64, 64, 2, 4>(g, s);
 }
 
 }  // namespace mg

@@ -73,9 +73,16 @@ __global__ __launch_bounds__(WG) void route_choose_kernel(MoeRoute p) {
 __global__ __launch_bounds__(WG) void route_clear_kernel(MoeRoute p) {
     for (int i = threadIdx.x; i < 2 * p.experts; i += WG) p.work[i] = 0;
 }
+constexpr int ROUTE_ENTRIES = 1024;      // entries a workgroup counts or places
 __global__ __launch_bounds__(WG) void route_count_kernel(MoeRoute p) {
-    const int i = blockIdx.x * WG + threadIdx.x;
-    if (i < p.T * p.top) atomicAdd(p.work + p.ids[i], 1);
+    __shared__ int cnt[MAX_EXPERTS];
+    for (int e = threadIdx.x; e < p.experts; e += WG) cnt[e] = 0;
+    __syncthreads();
+    const int i0 = blockIdx.x * ROUTE_ENTRIES, i1 = min(i0 + ROUTE_ENTRIES, p.T * p.top);
+    for (int i = i0 + threadIdx.x; i < i1; i += WG) atomicAdd(cnt + p.ids[i], 1);
+    __syncthreads();
+    for (int e = threadIdx.x; e < p.experts; e += WG)
+        if (cnt[e]) atomicAdd(p.work + e, cnt[e]);
 }
 // Starts of the experts' ranges and their row tiles, a thread an expert.
 __global__ void route_tiles_kernel(MoeRoute p) {
@@ -93,13 +100,21 @@ __global__ void route_tiles_kernel(MoeRoute p) {
 }
 // The order of an expert's entries is whichever workgroup comes first; no result depends on it.
 __global__ __launch_bounds__(WG) void route_place_kernel(MoeRoute p) {
-    const int i = blockIdx.x * WG + threadIdx.x;
-    if (i < p.T * p.top) p.perm[atomicAdd(p.work + p.experts + p.ids[i], 1)] = i;
+    __shared__ int cnt[MAX_EXPERTS], at[MAX_EXPERTS];
+    for (int e = threadIdx.x; e < p.experts; e += WG) cnt[e] = 0;
+    __syncthreads();
+    const int i0 = blockIdx.x * ROUTE_ENTRIES, i1 = min(i0 + ROUTE_ENTRIES, p.T * p.top);
+    for (int i = i0 + threadIdx.x; i < i1; i += WG) atomicAdd(cnt + p.ids[i], 1);
+    __syncthreads();
+    for (int e = threadIdx.x; e < p.experts; e += WG)
+        if (cnt[e]) at[e] = atomicAdd(p.work + p.experts + e, cnt[e]);
+    __syncthreads();
+    for (int i = i0 + threadIdx.x; i < i1; i += WG) p.perm[atomicAdd(at + p.ids[i], 1)] = i;
 }
 hipError_t launch_moe_route(const MoeRoute& p, hipStream_t s) {
     if (p.T <= 0) return hipSuccess;
     if (p.experts > MAX_EXPERTS || p.top < 1 || p.top > MAX_TOP || p.top > p.experts) return hipErrorInvalidValue;
-    const unsigned g = (unsigned)((p.T * p.top + WG - 1) / WG);
+    const unsigned g = (unsigned)((p.T * p.top + ROUTE_ENTRIES - 1) / ROUTE_ENTRIES);
     hipLaunchKernelGGL(route_clear_kernel, dim3(1), dim3(WG), 0, s, p);
     hipLaunchKernelGGL(route_choose_kernel, dim3((p.T + 3) / 4), dim3(WG), 0, s, p);
     hipLaunchKernelGGL(route_count_kernel, dim3(g), dim3(WG), 0, s, p);

@@ -10,11 +10,85 @@ namespace mg {
 // neighbouring chunks) read 16 bytes apart.
 __device__ __forceinline__ int plane_index(int i, int nc8) { return ((((i >> 2) & 1) * nc8 + (i >> 3)) << 2) + (i & 3); }
 
+__device__ __forceinline__ bool quad_aligned(const void* p) { return ((uintptr_t)p & 15) == 0; }
+
 // Stages in.src (transformed as VecInput says) as Kp floats, zero past in.n; ends with a barrier.  store: this
-// workgroup writes normOut / out.
+// workgroup writes normOut / out.  Everything a thread needs is requested before the first wait: up to 4096 elements
+// in registers, four consecutive ones at a time.
+template <int Q>
+__device__ __forceinline__ void stage_quads(const VecInput& in, float* act, int Kp, bool store, float* red) {
+    const int nq = in.n >> 2, kq = Kp >> 2, nc8 = Kp >> 3;
+    float4* planes = reinterpret_cast<float4*>(act);
+    float4 v[Q], g[Q], pt[Q];
+    const float4 zero = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+    for (int k = 0; k < Q; k++) {
+        const int q = min((int)threadIdx.x + k * WG, nq - 1);
+        v[k] = reinterpret_cast<const float4*>(in.src)[q];
+        g[k] = in.gain ? reinterpret_cast<const float4*>(in.gain)[q] : zero;
+        pt[k] = in.part ? reinterpret_cast<const float4*>(in.part)[q] : zero;
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < Q; k++) {
+        if ((int)threadIdx.x + k * WG >= nq) v[k] = zero;
+        ss = fmaf(v[k].x, v[k].x, fmaf(v[k].y, v[k].y, fmaf(v[k].z, v[k].z, fmaf(v[k].w, v[k].w, ss))));
+    }
+    if (in.gain) {
+        const float rs = 1.0f / sqrtf(block_sum(ss, red) / (float)in.n + in.eps);
+        float s2 = 0.f;
+#pragma unroll
+        for (int k = 0; k < Q; k++) {
+            const int q = threadIdx.x + k * WG;
+            if (q >= nq) continue;
+            float4 x = make_float4(v[k].x * rs * g[k].x, v[k].y * rs * g[k].y, v[k].z * rs * g[k].z, v[k].w * rs * g[k].w);
+            if (store && in.normOut) reinterpret_cast<float4*>(in.normOut)[q] = x;
+            if (in.part) {
+                x.x = fmaf(in.coef, x.x, pt[k].x); x.y = fmaf(in.coef, x.y, pt[k].y);
+                x.z = fmaf(in.coef, x.z, pt[k].z); x.w = fmaf(in.coef, x.w, pt[k].w);
+            }
+            if (store && in.out) reinterpret_cast<float4*>(in.out)[q] = x;
+            v[k] = x;
+            s2 = fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, fmaf(x.w, x.w, s2))));
+        }
+        if (in.gain2) {
+            const float r2 = 1.0f / sqrtf(block_sum(s2, red) / (float)in.n + in.eps);
+#pragma unroll
+            for (int k = 0; k < Q; k++) {
+                const int q = threadIdx.x + k * WG;
+                if (q >= nq) continue;
+                const float4 h = reinterpret_cast<const float4*>(in.gain2)[q];
+                v[k] = make_float4(v[k].x * r2 * h.x, v[k].y * r2 * h.y, v[k].z * r2 * h.z, v[k].w * r2 * h.w);
+            }
+        }
+    }
+#pragma unroll
+    for (int k = 0; k < Q; k++) {
+        const int q = threadIdx.x + k * WG;
+        if (q < kq) planes[(q & 1) * nc8 + (q >> 1)] = v[k];
+    }
+    __syncthreads();
+}
 __device__ __forceinline__ void stage_vector(const VecInput& in, float* act, int Kp, bool store, float* red) {
     const int nc8 = Kp >> 3;
     const int n = in.n;
+    if ((n & 3) == 0 && quad_aligned(in.src) && quad_aligned(in.gain) && quad_aligned(in.part) && quad_aligned(in.normOut) &&
+        quad_aligned(in.out) && quad_aligned(in.gain2)) {
+        if (Kp <= 1024) { stage_quads<1>(in, act, Kp, store, red); return; }
+        if (Kp <= 2048) { stage_quads<2>(in, act, Kp, store, red); return; }
+        if (Kp <= 4096) { stage_quads<4>(in, act, Kp, store, red); return; }
+        if (!in.gain) {
+            float4* planes = reinterpret_cast<float4*>(act);
+#pragma unroll 8
+            for (int q = threadIdx.x; q < Kp >> 2; q += WG) {
+                float4 v = reinterpret_cast<const float4*>(in.src)[min(q, (n >> 2) - 1)];
+                if (q >= n >> 2) v = make_float4(0.f, 0.f, 0.f, 0.f);
+                planes[(q & 1) * nc8 + (q >> 1)] = v;
+            }
+            __syncthreads();
+            return;
+        }
+    }
     float ss = 0.f;
     for (int i = threadIdx.x; i < Kp; i += WG) {
         const float v = i < n ? in.src[i] : 0.f;
@@ -45,34 +119,41 @@ constexpr int MAX_TOP = 32;
 
 // The `top` largest of E logits (the lower index on ties) and their softmax over all E, by one full wave.
 // ids / w: LDS or global, written by lane 0.
-__device__ __forceinline__ void choose_experts(const float* z, int E, int top, int* ids, float* w) {
+template <int EPL>      // logits a lane holds
+__device__ __forceinline__ void choose_experts_of(const float* z, int E, int top, int* ids, float* w) {
     const int lane = threadIdx.x & 63;
-    float v[MAX_EXPERTS / 64];
+    float v[EPL];
     float m = -INFINITY;
 #pragma unroll
-    for (int k = 0; k < MAX_EXPERTS / 64; k++) {
+    for (int k = 0; k < EPL; k++) {
         const int e = k * 64 + lane;
-        v[k] = e < E ? z[e] : -INFINITY;
+        v[k] = z[min(e, E - 1)];
+        if (e >= E) v[k] = -INFINITY;
         m = fmaxf(m, v[k]);
     }
     m = wave_max(m);
     float sum = 0.f;
 #pragma unroll
-    for (int k = 0; k < MAX_EXPERTS / 64; k++) sum += expf(v[k] - m);
+    for (int k = 0; k < EPL; k++) sum += expf(v[k] - m);
     sum = wave_sum(sum);
     for (int s = 0; s < top; s++) {
         float bv = -INFINITY;
         int bi = INT_MAX;
 #pragma unroll
-        for (int k = 0; k < MAX_EXPERTS / 64; k++)
+        for (int k = 0; k < EPL; k++)
             if (v[k] > bv) { bv = v[k]; bi = k * 64 + lane; }
         wave_argmax(bv, bi);
         if (bi >= E) bi = 0;                      // (only with non-finite logits)
 #pragma unroll
-        for (int k = 0; k < MAX_EXPERTS / 64; k++)
+        for (int k = 0; k < EPL; k++)
             if (bi == k * 64 + lane) v[k] = -INFINITY;
         if (lane == 0) { ids[s] = bi; w[s] = expf(bv - m) / sum; }
     }
+}
+__device__ __forceinline__ void choose_experts(const float* z, int E, int top, int* ids, float* w) {
+    if (E <= 64) choose_experts_of<1>(z, E, top, ids, w);
+    else if (E <= 128) choose_experts_of<2>(z, E, top, ids, w);
+    else choose_experts_of<MAX_EXPERTS / 64>(z, E, top, ids, w);
 }
 
 }  // namespace mg
