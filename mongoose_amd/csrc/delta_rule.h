@@ -41,9 +41,13 @@ struct DeltaRows {
     float* au = nullptr;             // work: a u
     float* u = nullptr;              // work
     float* o = nullptr;              // work: [T, heads * dim]
+    float* chunks = nullptr;         // work: delta_chunk_floats() floats, or NULL: always token by token
     void* yAct = nullptr;            // [T, ldAct]
     int actF32 = 0, ldAct = 0;
 };
+constexpr int DELTA_CHUNK_MIN_ROWS = 64;     // fewer rows go token by token
+// Workspace of the chunked form for T rows; 0 where it is not used.
+size_t delta_chunk_floats(int heads, int dim, int T);
 bool delta_supported(int dim);
 hipError_t launch_delta_rows(const DeltaRows& p, hipStream_t s);
 

@@ -157,7 +157,7 @@ __global__ __launch_bounds__(64) void delta_gates_kernel(DeltaRows p) {
     }
 }
 
-// The recurrence itself.  The value columns of a state do not touch each other: 16 lanes (one DPP row) own a column,
+// The recurrence token by token, for few rows and for heads wider than the chunked form has variants for.  The value columns of a state do not touch each other: 16 lanes (one DPP row) own a column,
 // CPL key channels each; a workgroup 16 columns of one head.  Tokens go through LDS in chunks of TC.
 template <int CPL>
 __global__ __launch_bounds__(WG) void delta_scan_kernel(DeltaRows p) {
@@ -223,6 +223,253 @@ __global__ __launch_bounds__(WG) void delta_scan_kernel(DeltaRows p) {
         }
 }
 
+// ---------------------------------------------------------------------------
+// The recurrence in chunks of 32 tokens, for many rows.  With W_t the product of the decays up to and including token t
+// of a chunk (per key channel) and S_t = diag(W_t) Z_t,
+//   Z_t = Z_(t-1) - b_t d_t + k_t v_t^T,  d_t = u_t^T Z_(t-1),   u_t := W_(t-1) u_t,  b_t := (a u)_t / W_t,
+//   o_t = r_t^T Z_t,                                             k_t := k_t / W_t,    r_t := W_t r_t,
+// so that, over a chunk (rows are tokens; low / low0: lower triangle with / without the diagonal),
+//   D = P Z_0 + Q,   (I + low0(U B^T)) [P | Q] = [U | low0(U K^T) V],
+//   S_end = M S_0 + N,   M = diag(W_end)(I - B^T P),   N = diag(W_end)(K^T V - B^T Q),
+//   O     = G S_0 + Ol,  G = R - low(R B^T) P,         Ol = low(R K^T) V - low(R B^T) Q.
+// delta_chunk_kernel makes M, N, G, Ol of all chunks at once; delta_chain_kernel goes through the chunks, which is
+// one small matrix product a chunk.  Decays are at least exp(-exp(-1/2)) a token, so W_t stays above 3e-9.
+// Everything in fp32, on v_mfma_f32_16x16x4_f32.
+// ---------------------------------------------------------------------------
+constexpr int CH = 32;                   // tokens of a chunk
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+// acc += A[row][k] B[k][col] over K; element strides (ar, ak), (bk, bc); this lane's row / column is lane % 16, its k
+// lane / 16 of every four.
+__device__ __forceinline__ f32x4 mfma_tile(f32x4 acc, const float* A, int ar, int ak, const float* B, int bk, int bc, int K) {
+    const int lane = threadIdx.x & 63;
+    const float* a = A + (lane & 15) * ar + (lane >> 4) * ak;
+    const float* b = B + (lane & 15) * bc + (lane >> 4) * bk;
+    for (int k = 0; k < K; k += 8) {
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[k * ak], b[k * bk], acc, 0, 0, 0);
+        acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[(k + 4) * ak], b[(k + 4) * bk], acc, 0, 0, 0);
+    }
+    return acc;
+}
+// floats of one (chunk, head): M and N [DP, DP], G and Ol [CH, DP]
+__host__ __device__ inline size_t chunk_floats(int DP) { return (size_t)2 * DP * DP + (size_t)2 * CH * DP; }
+
+// grid (heads, chunks)
+template <int DP>
+__global__ __launch_bounds__(256) void delta_chunk_kernel(DeltaRows p) {
+    constexpr int LD = DP + 4, LA = CH + 4, NT = DP / 16;
+    extern __shared__ __attribute__((aligned(16))) float sm[];
+    float* U = sm;                        // [CH][LD] each
+    float* B = U + CH * LD;
+    float* K = B + CH * LD;
+    float* R = K + CH * LD;
+    float* V = R + CH * LD;
+    float* P = V + CH * LD;
+    float* Q = P + CH * LD;
+    float* Aub = Q + CH * LD;             // [CH][LA] each
+    float* Auk = Aub + CH * LA;
+    float* Arb = Auk + CH * LA;
+    float* Ark = Arb + CH * LA;
+    float* wc = Ark + CH * LA;            // [DP]
+    const int h = blockIdx.x, c = blockIdx.y, D = p.d.dim, HD = p.d.heads * D, t0 = c * CH;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    // cumulative decays; channels past dim and tokens past T change nothing
+    if ((int)threadIdx.x < DP) {
+        const int i = threadIdx.x;
+        const bool ok = i < D;
+        const int ci = h * D + (ok ? i : 0);
+        float W = 1.f;
+#pragma unroll 8
+        for (int t = 0; t < CH; t++) {
+            const int tt = min(t0 + t, p.T - 1);
+            const bool on = ok && t0 + t < p.T;
+            const size_t o = (size_t)tt * HD + ci;
+            const float* z = p.z + (size_t)tt * p.ldz + ci;
+            const float dec = p.dec[o], au = p.au[o], u = p.u[o], r = z[0], k = z[HD], v = z[2 * HD];
+            U[t * LD + i] = on ? W * u : 0.f;
+            if (on) W *= dec;
+            const float inv = 1.0f / W;
+            B[t * LD + i] = on ? au * inv : 0.f;
+            K[t * LD + i] = on ? k * inv : 0.f;
+            R[t * LD + i] = on ? W * r : 0.f;
+            V[t * LD + i] = on ? v : 0.f;
+        }
+        wc[i] = W;
+    }
+    __syncthreads();
+    {   // wave: one of the four C x C products, its three tiles that are not above the diagonal
+        const float* X = wave < 2 ? U : R;
+        const float* Y = wave & 1 ? K : B;
+        float* O = Aub + wave * CH * LA;                        // Aub, Auk, Arb, Ark
+        const int strict = wave < 2 ? 1 : 0;
+#pragma unroll
+        for (int q = 0; q < 3; q++) {
+            const int tr = q == 0 ? 0 : 16, tc = q == 2 ? 16 : 0;
+            f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+            acc = mfma_tile(acc, X + tr * LD, LD, 1, Y + tc * LD, 1, LD, DP);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int t = tr + 4 * (lane >> 4) + e, s = tc + (lane & 15);
+                O[t * LA + s] = s + strict <= t ? acc[e] : 0.f;
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; e++) O[(4 * (lane >> 4) + e) * LA + 16 + (lane & 15)] = 0.f;
+    }
+    __syncthreads();
+    for (int q = wave; q < 2 * NT; q += 4) {                    // Q <- low0(U K^T) V
+        const int tr = (q & 1) * 16, tc = (q >> 1) * 16;
+        f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+        acc = mfma_tile(acc, Auk + tr * LA, LA, 1, V + tc, LD, 1, CH);
+#pragma unroll
+        for (int e = 0; e < 4; e++) Q[(tr + 4 * (lane >> 4) + e) * LD + tc + (lane & 15)] = acc[e];
+    }
+    __syncthreads();
+    if ((int)threadIdx.x < 2 * DP) {                            // forward substitution, a column a thread
+        const bool isQ = (int)threadIdx.x >= DP;
+        const int i = isQ ? threadIdx.x - DP : threadIdx.x;
+        const float* in = (isQ ? Q : U) + i;
+        float* out = (isQ ? Q : P) + i;
+        float x[CH];
+#pragma unroll
+        for (int t = 0; t < CH; t++) {
+            float v = in[t * LD];
+#pragma unroll
+            for (int s4 = 0; s4 < t; s4 += 4) {
+                const float4 a = *reinterpret_cast<const float4*>(Aub + t * LA + s4);
+                v = fmaf(-a.x, x[s4], v);
+                if (s4 + 1 < t) v = fmaf(-a.y, x[s4 + 1], v);
+                if (s4 + 2 < t) v = fmaf(-a.z, x[s4 + 2], v);
+                if (s4 + 3 < t) v = fmaf(-a.w, x[s4 + 3], v);
+            }
+            x[t] = v;
+        }
+#pragma unroll
+        for (int t = 0; t < CH; t++) out[t * LD] = x[t];
+    }
+    __syncthreads();
+    // results in the order the chain reads them: M and G as first operands (lane: row lane % 16, four steps of k), N and Ol
+    // as accumulators (column tile by column tile)
+    float* M = p.chunks + ((size_t)c * p.d.heads + h) * chunk_floats(DP);
+    float* N = M + DP * DP;
+    float* G = N + DP * DP;
+    float* Ol = G + CH * DP;
+    for (int q = wave; q < NT * NT; q += 4) {
+        const int rt = q / NT, ct = q % NT;
+        f32x4 bp = {0.f, 0.f, 0.f, 0.f}, bq = bp, kv = bp;
+        bp = mfma_tile(bp, B + rt * 16, 1, LD, P + ct * 16, LD, 1, CH);
+        bq = mfma_tile(bq, B + rt * 16, 1, LD, Q + ct * 16, LD, 1, CH);
+        kv = mfma_tile(kv, K + rt * 16, 1, LD, V + ct * 16, LD, 1, CH);
+        float4 n;
+        float* np = &n.x;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int r = 4 * (lane >> 4) + e, col = lane & 15;
+            const float w = wc[rt * 16 + r];
+            M[((size_t)(rt * NT + ct) * 64 + r + 16 * (col & 3)) * 4 + (col >> 2)] = w * ((rt == ct && r == col ? 1.f : 0.f) - bp[e]);
+            np[e] = w * (kv[e] - bq[e]);
+        }
+        reinterpret_cast<float4*>(N)[(size_t)(ct * NT + rt) * 64 + lane] = n;
+    }
+    for (int q = wave; q < 2 * NT; q += 4) {
+        const int tt = q & 1, ct = q >> 1;
+        f32x4 gp = {0.f, 0.f, 0.f, 0.f}, oq = gp, ov = gp;
+        gp = mfma_tile(gp, Arb + tt * 16 * LA, LA, 1, P + ct * 16, LD, 1, CH);
+        oq = mfma_tile(oq, Arb + tt * 16 * LA, LA, 1, Q + ct * 16, LD, 1, CH);
+        ov = mfma_tile(ov, Ark + tt * 16 * LA, LA, 1, V + ct * 16, LD, 1, CH);
+        float4 n;
+        float* np = &n.x;
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const int r = 4 * (lane >> 4) + e, col = lane & 15;
+            G[((size_t)(tt * NT + ct) * 64 + r + 16 * (col & 3)) * 4 + (col >> 2)] = R[(tt * 16 + r) * LD + ct * 16 + col] - gp[e];
+            np[e] = ov[e] - oq[e];
+        }
+        reinterpret_cast<float4*>(Ol)[(size_t)(ct * 2 + tt) * 64 + lane] = n;
+    }
+}
+
+// grid (heads, DP / 16): 16 value columns of a head's state through all chunks.  Waves 0 .. NT - 1: a row tile of the
+// state each; the last two: the chunk's 32 output rows.
+template <int DP>
+__global__ __launch_bounds__(64 * (DP / 16 + 2)) void delta_chain_kernel(DeltaRows p) {
+    constexpr int NT = DP / 16;
+    __shared__ float S[2][DP * 16];
+    const int h = blockIdx.x, ct = blockIdx.y, D = p.d.dim, HD = p.d.heads * D;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const bool state = wave < NT;
+    float* Sg = p.S + (size_t)h * D * D;
+    for (int x = threadIdx.x; x < DP * 16; x += blockDim.x) {
+        const int i = x >> 4, j = ct * 16 + (x & 15);
+        S[0][x] = i < D && j < D && p.pos0 > 0 ? Sg[(size_t)i * D + j] : 0.f;
+    }
+    const int chunks = (p.T + CH - 1) / CH;
+    const size_t step = chunk_floats(DP) * p.d.heads;
+    const float* base = p.chunks + h * chunk_floats(DP);
+    const float4* a = reinterpret_cast<const float4*>(state ? base + (size_t)wave * 16 * DP : base + 2 * DP * DP + (size_t)(wave - NT) * 16 * DP) + lane;
+    const float4* n = reinterpret_cast<const float4*>(state ? base + DP * DP + (size_t)(ct * NT + wave) * 256
+                                                            : base + 2 * DP * DP + CH * DP + (size_t)(ct * 2 + wave - NT) * 256) + lane;
+    float4 fa[NT], fn;
+    auto fetch = [&](int c) __attribute__((always_inline)) {
+        const float4* ac = a + (size_t)c * (step / 4);
+#pragma unroll
+        for (int k = 0; k < NT; k++) fa[k] = ac[k * 64];
+        fn = n[(size_t)c * (step / 4)];
+    };
+    fetch(0);
+    __syncthreads();
+    for (int c = 0; c < chunks; c++) {
+        const float* s = S[c & 1];
+        float4 ca[NT];
+#pragma unroll
+        for (int k = 0; k < NT; k++) ca[k] = fa[k];
+        f32x4 acc = {fn.x, fn.y, fn.z, fn.w};
+        if (c + 1 < chunks) fetch(c + 1);
+#pragma unroll
+        for (int k = 0; k < NT; k++) {                          // k tile: S rows 16 k + 4 e + lane / 16
+            const float* sk = s + 16 * k * 16 + (lane >> 4) * 16 + (lane & 15);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ca[k].x, sk[0], acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ca[k].y, sk[64], acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ca[k].z, sk[128], acc, 0, 0, 0);
+            acc = __builtin_amdgcn_mfma_f32_16x16x4f32(ca[k].w, sk[192], acc, 0, 0, 0);
+        }
+        if (state) {
+#pragma unroll
+            for (int e = 0; e < 4; e++) S[(c + 1) & 1][(wave * 16 + 4 * (lane >> 4) + e) * 16 + (lane & 15)] = acc[e];
+        } else {
+            const int j = ct * 16 + (lane & 15);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const int t = c * CH + (wave - NT) * 16 + 4 * (lane >> 4) + e;
+                if (t < p.T && j < D) p.o[(size_t)t * HD + h * D + j] = acc[e];
+            }
+        }
+        __syncthreads();
+    }
+    for (int x = threadIdx.x; x < DP * 16; x += blockDim.x) {
+        const int i = x >> 4, j = ct * 16 + (x & 15);
+        if (i < D && j < D) Sg[(size_t)i * D + j] = S[chunks & 1][x];
+    }
+}
+
+template <int DP>
+static hipError_t run_delta_chunks(const DeltaRows& p, hipStream_t s) {
+    const size_t lds = ((size_t)7 * CH * (DP + 4) + 4 * CH * (CH + 4) + DP) * 4;
+    auto k = delta_chunk_kernel<DP>;
+    if (lds > (48u << 10)) {
+        hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(k, dim3(p.d.heads, (p.T + CH - 1) / CH), dim3(256), lds, s, p);
+    hipLaunchKernelGGL(delta_chain_kernel<DP>, dim3(p.d.heads, DP / 16), dim3(64 * (DP / 16 + 2)), 0, s, p);
+    return hipGetLastError();
+}
+static int chunk_dim(int dim) { return dim <= 16 ? 16 : dim <= 32 ? 32 : dim <= 64 ? 64 : dim <= 128 ? 128 : 0; }
+size_t delta_chunk_floats(int heads, int dim, int T) {
+    const int DP = chunk_dim(dim);
+    return DP && T >= DELTA_CHUNK_MIN_ROWS ? chunk_floats(DP) * heads * ((T + CH - 1) / CH) : 0;
+}
+
 template <typename AT>
 __global__ __launch_bounds__(64) void delta_output_kernel(DeltaRows p) {
     const int h = blockIdx.x, t = blockIdx.y, D = p.d.dim, HD = p.d.heads * D;
@@ -250,13 +497,23 @@ hipError_t launch_delta_rows(const DeltaRows& p, hipStream_t s) {
     hipError_t e = launch_gemm_bf16w(g, s);
     if (e != hipSuccess) return e;
     hipLaunchKernelGGL(delta_gates_kernel, dim3(H, p.T), dim3(64), 0, s, p);
-    const dim3 grid(H, (D + 15) / 16);
-    const int cpl = (D + 15) / 16;
-    if (cpl <= 1) hipLaunchKernelGGL(delta_scan_kernel<1>, grid, dim3(WG), 0, s, p);
-    else if (cpl <= 2) hipLaunchKernelGGL(delta_scan_kernel<2>, grid, dim3(WG), 0, s, p);
-    else if (cpl <= 4) hipLaunchKernelGGL(delta_scan_kernel<4>, grid, dim3(WG), 0, s, p);
-    else if (cpl <= 8) hipLaunchKernelGGL(delta_scan_kernel<8>, grid, dim3(WG), 0, s, p);
-    else hipLaunchKernelGGL(delta_scan_kernel<16>, grid, dim3(WG), 0, s, p);
+    if (p.chunks && delta_chunk_floats(H, D, p.T)) {
+        switch (chunk_dim(D)) {
+        case 16: e = run_delta_chunks<16>(p, s); break;
+        case 32: e = run_delta_chunks<32>(p, s); break;
+        case 64: e = run_delta_chunks<64>(p, s); break;
+        default: e = run_delta_chunks<128>(p, s); break;
+        }
+        if (e != hipSuccess) return e;
+    } else {
+        const dim3 grid(H, (D + 15) / 16);
+        const int cpl = (D + 15) / 16;
+        if (cpl <= 1) hipLaunchKernelGGL(delta_scan_kernel<1>, grid, dim3(WG), 0, s, p);
+        else if (cpl <= 2) hipLaunchKernelGGL(delta_scan_kernel<2>, grid, dim3(WG), 0, s, p);
+        else if (cpl <= 4) hipLaunchKernelGGL(delta_scan_kernel<4>, grid, dim3(WG), 0, s, p);
+        else if (cpl <= 8) hipLaunchKernelGGL(delta_scan_kernel<8>, grid, dim3(WG), 0, s, p);
+        else hipLaunchKernelGGL(delta_scan_kernel<16>, grid, dim3(WG), 0, s, p);
+    }
     if (p.actF32) hipLaunchKernelGGL(delta_output_kernel<float>, dim3(H, p.T), dim3(64), 0, s, p);
     else hipLaunchKernelGGL(delta_output_kernel<bf16_t>, dim3(H, p.T), dim3(64), 0, s, p);
     return hipGetLastError();

@@ -51,6 +51,39 @@ template <int V> struct LatentVec<float, V> {
     }
 };
 
+// Sums of 16 values over the wave, each exchange halving the number of registers instead of summing every value by
+// itself: after it, value (k, h) is in the four lanes from fold16_lane(k, h).
+__device__ __forceinline__ float fold16(float (&s)[LKB][LHG]) {
+    static_assert(LKB == 4 && LHG == 4, "");
+    const int lane = threadIdx.x & 63;
+    float a[8], b[4], c[2];
+#pragma unroll
+    for (int k = 0; k < 4; k++)                      // lanes 0..31: h = 0, 1; 32..63: h = 2, 3
+#pragma unroll
+        for (int h = 0; h < 2; h++) {
+            float x = s[k][h], y = s[k][h + 2];
+            row_swap32(x, y);
+            a[2 * k + h] = x + y;
+        }
+#pragma unroll
+    for (int k = 0; k < 4; k++) {                    // odd rows of 16 lanes: the odd h
+        float x = a[2 * k], y = a[2 * k + 1];
+        row_swap16(x, y);
+        b[k] = x + y;
+    }
+#pragma unroll
+    for (int k = 0; k < 2; k++) {                    // upper half of a row: k + 2
+        const bool up = lane & 8;
+        c[k] = (up ? b[k + 2] : b[k]) + dpp_f<0x128>(up ? b[k] : b[k + 2]);
+    }
+    const bool up = lane & 4;                        // upper quad of a half: the odd k; partner lane ^ 7
+    float t = (up ? c[1] : c[0]) + dpp_f<0x141>(up ? c[0] : c[1]);
+    t += dpp_f<0xB1>(t);
+    t += dpp_f<0x4E>(t);
+    return t;
+}
+__device__ __forceinline__ constexpr int fold16_lane(int k, int h) { return (h >> 1) * 32 + (h & 1) * 16 + (k >> 1) * 8 + (k & 1) * 4; }
+
 // A lane owns V consecutive latent elements: one load of a key serves its score and the weighted sum.  grid (splits,
 // ceil(heads / LHG), T).
 template <typename CT, int V>
@@ -151,14 +184,13 @@ __global__ __launch_bounds__(LNW * 64) void latent_decode_kernel(LatentDecode p)
                 for (int i = 0; i < V; i++) a = fmaf(ql[h][i], kv[k][i], a);
                 s[k][h] = a;
             }
+        float tot = fold16(s);
 #pragma unroll
         for (int k = 0; k < LKB; k++)
 #pragma unroll
-            for (int h = 0; h < LHG; h += 2) {
-                const float r = wave_sum2(s[k][h], s[k][h + 1]);
-                s[k][h] = lane_value(r, 0) * p.scale;
-                s[k][h + 1] = lane_value(r, 32) * p.scale;
-                if (kb + k >= k1) { s[k][h] = -INFINITY; s[k][h + 1] = -INFINITY; }
+            for (int h = 0; h < LHG; h++) {
+                s[k][h] = lane_value(tot, fold16_lane(k, h)) * p.scale;
+                if (kb + k >= k1) s[k][h] = -INFINITY;
             }
 #pragma unroll
         for (int h = 0; h < LHG; h++) {
@@ -213,10 +245,10 @@ static int latent_lane_elems(int rankPad) {
 bool latent_decode_supported(int rank, int rot) { return rank >= 1 && latent_lane_elems(pad_to(rank, 64)) <= 16 && rot >= 0 && rot <= 128; }
 
 void latent_decode_splits(int span, int heads, int T, int* splits, int* splitLen) {
-    // one batch of keys a wave at least; at most 16 partial results for the consumer to merge
+    // one batch of keys a wave at least; at most 32 partial results for the consumer to merge
     const int groups = (heads + LHG - 1) / LHG;
-    int n = std::max(1, 512 / std::max(1, groups * T));
-    n = std::min({n, 16, (span + LNW * LKB - 1) / (LNW * LKB)});
+    int n = std::max(1, 256 / std::max(1, groups * T));
+    n = std::min({n, 32, (span + LNW * LKB - 1) / (LNW * LKB)});
     n = std::max(n, 1);
     *splitLen = pad_to((span + n - 1) / n, LNW * LKB);
     *splits = (span + *splitLen - 1) / *splitLen;

@@ -132,7 +132,7 @@ private:
     int* rTokens = nullptr;
     int* rWant = nullptr;
     float *rX = nullptr, *rXs = nullptr, *rY = nullptr, *rX1 = nullptr, *rZ = nullptr, *rQf = nullptr, *rQlat = nullptr;
-    float *rGate = nullptr, *rExp = nullptr, *rDec = nullptr, *rAu = nullptr, *rU = nullptr, *rO = nullptr, *rW1 = nullptr;
+    float *rGate = nullptr, *rExp = nullptr, *rDec = nullptr, *rAu = nullptr, *rU = nullptr, *rO = nullptr, *rW1 = nullptr, *rChunks = nullptr;
     float *rPacc = nullptr, *rPm = nullptr, *rPl = nullptr, *rLogits = nullptr, *rWeights = nullptr;
     void *aX = nullptr, *aX1 = nullptr, *aCq = nullptr, *aQ = nullptr, *aO = nullptr, *aHid = nullptr, *aShared = nullptr, *aWant = nullptr;
     unsigned short *rK = nullptr, *rVt = nullptr;

@@ -592,7 +592,7 @@ int LayeredInference::ensureRows(int rows, int pos0) {
     rowCap = keyCap = 0;
     const size_t ae = f32 ? 4 : 2;
     size_t zMax = 1, cq = 64, qMax = 64, qlat = 1, oMax = 64, gate = 1, hidA = 64, sh = 64, expOut = 1, HD = 1, w1 = 64, kMax = 1, vMax = 1, tiles = 1, work = 1;
-    size_t top = 1, pacc = 1, pms = 1;
+    size_t top = 1, pacc = 1, pms = 1, chunks = 1;
     for (const LayerBlock& L : layers) {
         const mg_layer_desc& d = L.d;
         zMax = std::max(zMax, (size_t)pad_to(L.proj.rows, 4));
@@ -609,6 +609,7 @@ int LayeredInference::ensureRows(int rows, int pos0) {
         } else {
             HD = std::max(HD, (size_t)d.heads * d.dim);
             w1 = std::max(w1, (size_t)L.w2.ld);
+            chunks = std::max(chunks, delta_chunk_floats(d.heads, d.dim, T));
         }
         if (d.mlp == MG_MLP_DENSE) hidA = std::max(hidA, (size_t)T * L.down.ld);
         if (d.mlp == MG_MLP_MOE) {
@@ -628,7 +629,7 @@ int LayeredInference::ensureRows(int rows, int pos0) {
     p.want(rX, (size_t)(nLayers + 1) * Ts * dim); p.want(rXs, Ts * dim); p.want(rY, Ts * dim); p.want(rX1, Ts * dim);
     p.want(rZ, Ts * zMax); p.want(rQf, (size_t)qMax * Ts); p.want(rQlat, qlat);
     p.want(rGate, Ts * gate); p.want(rExp, Ts * expOut);
-    p.want(rDec, Ts * HD); p.want(rAu, Ts * HD); p.want(rU, Ts * HD); p.want(rO, Ts * HD); p.want(rW1, Ts * w1);
+    p.want(rDec, Ts * HD); p.want(rAu, Ts * HD); p.want(rU, Ts * HD); p.want(rO, Ts * HD); p.want(rW1, Ts * w1); p.want(rChunks, chunks);
     p.want(rPacc, pacc); p.want(rPm, pms); p.want(rPl, pms);
     p.want(rLogits, (size_t)256 * vocabSize); p.want(rWeights, Ts * top);
     p.want(aX, Ts * widthPad, ae); p.want(aX1, Ts * widthPad, ae); p.want(aCq, Ts * cq, ae); p.want(aQ, Ts * qMax, ae);
@@ -713,7 +714,7 @@ int LayeredInference::rowsDelta(LayerBlock& L, int T, int pos0) {
     HIPCHK(launch_gemm_bf16w(g, stream));
     DeltaRows p;
     p.d = L.delta; p.z = rZ; p.ldz = ldz; p.T = T; p.pos0 = pos0; p.S = L.S;
-    p.w1 = rW1; p.dec = rDec; p.au = rAu; p.u = rU; p.o = rO;
+    p.w1 = rW1; p.dec = rDec; p.au = rAu; p.u = rU; p.o = rO; p.chunks = rChunks;
     p.yAct = aO; p.actF32 = f32; p.ldAct = L.out.ld;
     HIPCHK(launch_delta_rows(p, stream));
     return MG_OK;

@@ -56,6 +56,7 @@ MECHANISMS = {
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("name", sorted(MECHANISMS))
 def test_each_mechanism_alone(hip, name, dtype):
+    """70 tokens: one pass (matrix forms of attention and recurrence), token by token, and small portions."""
     p = M.Pair(M.model(MECHANISMS[name]), seed=3, eng=hip, dtype=dtype, maxSeq=128)
     toks = p.tokens(70)
     want = p.oracle_logits(toks)
@@ -69,6 +70,20 @@ def all_experts(layers):
     """The same layers with every expert chosen: in bf16 two router scores closer than rounding pick another expert,
     which is no fault but would need tolerances that hide faults (the choice itself is tested alone)."""
     return [{**L, "experts": L["top"]} if L.get("mlp") == C.MLP_MOE else L for L in layers]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("w0, ab", [(9.0, 9.0), (-9.0, 9.0), (9.0, -9.0), (-9.0, -9.0)])
+def test_delta_rule_at_the_ends_of_its_gates(hip, dtype, w0, ab):
+    """Fastest and slowest decay, full and no removal, over several chunks of the many-row form and a ragged end."""
+    p = M.Pair(M.model([M.delta(heads=2, dim=64, decay_rank=8)]), seed=6, eng=hip, dtype=dtype, maxSeq=256,
+               tweak={"l0.mix.w0": lambda a: 0.1 * a + w0, "l0.mix.a.b": lambda a: 0.1 * a + ab})
+    toks = p.tokens(215)
+    want = p.oracle_logits(toks)
+    for sizes in ([215], [64], [100, 3], [1]):
+        e = M.errors(M.run_portions(p.hip, toks, sizes), want)
+        assert e.max() < TOL[dtype], (sizes, int(e.argmax()), float(e.max()))
+    p.close()
 
 
 @pytest.fixture(scope="module", params=["float32", "bfloat16"])
