@@ -6,7 +6,7 @@
 namespace mg {
 
 // What is applied to a finished row of a product.
-enum ActKind { ACT_NONE = 0, ACT_GELU = 1, ACT_XIELU = 2, ACT_TANH = 3 };
+enum ActKind { ACT_NONE = 0, ACT_GELU = 1, ACT_XIELU = 2 };
 // xIELU: z > 0: ap z^2 + z/2;  z <= 0: an (exp(z) - 1 - z) + z/2 with ap = softplus(p), an = 1/2 + softplus(q).
 struct ActParam { int kind; float ap, an; };
 
@@ -26,7 +26,6 @@ __device__ __forceinline__ float xielu_f(float z, float ap, float an) {
 __device__ __forceinline__ float apply_act(float z, ActParam a) {
     if (a.kind == ACT_GELU) return gelu_erf_f(z);
     if (a.kind == ACT_XIELU) return xielu_f(z, a.ap, a.an);
-    if (a.kind == ACT_TANH) return tanhf(z);
     return z;
 }
 

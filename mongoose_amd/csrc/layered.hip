@@ -618,7 +618,7 @@ int LayeredInference::ensureRows(int rows, int pos0) {
             if (d.ff_shared) sh = std::max(sh, (size_t)L.downShared.ld);
             expOut = std::max(expOut, (size_t)d.top * dim);
             top = std::max(top, (size_t)d.top);
-            tiles = std::max(tiles, (size_t)moe_max_tiles(T, d.top, d.experts, MOE_TILE_ROWS));
+            tiles = std::max(tiles, (size_t)moe_max_tiles(T, d.top, d.experts, 64));
             work = std::max(work, (size_t)2 * d.experts);
         }
     }
@@ -742,13 +742,17 @@ int LayeredInference::rowsMlp(LayerBlock& L, int T, NormRows& after) {
     g.mode = GEMM_SPLIT; g.nSplit = ldg; g.out = rGate; g.ldc = ldg;
     g.outAct = aShared; g.ldo = L.downShared.ld; g.act = L.act;
     HIPCHK(launch_gemm_bf16w(g, stream));
+    // wide row tiles where the experts have the rows to fill them
+    const int tileRows = !f32 && (long)T * d.top >= 96L * d.experts ? 128 : 64;
     MoeRoute r;
+    r.tileRows = tileRows;
     r.z = rGate; r.ldz = ldg; r.T = T; r.experts = d.experts; r.top = d.top;
     r.ids = rIds; r.weights = rWeights; r.work = rWork; r.perm = rPerm; r.tiles = rTiles; r.nTiles = rNTiles;
     HIPCHK(launch_moe_route(r, stream));
     Gemm e;
     e.f32 = f32; e.M = T * d.top; e.tiles = rTiles; e.nTiles = rNTiles; e.perm = rPerm;
-    e.maxTiles = moe_max_tiles(T, d.top, d.experts, MOE_TILE_ROWS);
+    e.tileRows = tileRows;
+    e.maxTiles = moe_max_tiles(T, d.top, d.experts, tileRows);
     g = e;
     g.A = aX1; g.lda = widthPad; g.permDiv = d.top;
     g.W = L.up.w; g.ldw = L.up.ld; g.N = d.ff; g.K = L.up.ld; g.expertStride = L.upStride;

@@ -130,8 +130,8 @@ struct Gemm {
     int permDiv = 0;                 // > 0: A row = perm[r] / permDiv; 0: A row = r
     const float* rowScale = nullptr;
     size_t expertStride = 0;
+    int tileRows = 64;               // most rows of a tile: 64, or (bf16) 128
 };
-constexpr int MOE_TILE_ROWS = 64;    // rows of a tile of the experts' products
 hipError_t launch_gemm_bf16w(const Gemm& g, hipStream_t s);
 
 }  // namespace mg

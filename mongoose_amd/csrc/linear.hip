@@ -333,21 +333,22 @@ hipError_t launch_head_matvec(const HeadMv& p, hipStream_t s) {
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 
-// Four consecutive columns n .. n+3 of row m (sorted row r of an expert tile; m is where it goes).
-template <typename AT>
+// Four consecutive columns n .. n+3 of row m (of an expert tile: m is where the row goes).
+template <typename AT, int MODE, int ACT>
 __device__ __forceinline__ void gemm_store4(const Gemm& g, int m, int n, float4 v) {
     const int left = g.N - n;
     float e[4] = {v.x, v.y, v.z, v.w};
-    if (g.mode == GEMM_SPLIT) {
+    const ActParam act{ACT, g.act.ap, g.act.an};
+    if (MODE == GEMM_SPLIT) {
 #pragma unroll
         for (int i = 0; i < 4; i++) {
             if (i >= left) break;
             if (n + i < g.nSplit) g.out[(size_t)m * g.ldc + n + i] = e[i];
-            else store_act(static_cast<AT*>(g.outAct) + (size_t)m * g.ldo + (n + i - g.nSplit), apply_act(e[i], g.act));
+            else store_act(static_cast<AT*>(g.outAct) + (size_t)m * g.ldo + (n + i - g.nSplit), apply_act(e[i], act));
         }
         return;
     }
-    if (g.mode == GEMM_ROPE) {
+    if (MODE == GEMM_ROPE) {
         const int hc = n % g.headW - g.ropeOff;               // headW and ropeOff are multiples of 32
         if (hc >= 0 && hc < g.ropeDims) {
             const size_t row = (size_t)(g.pos0 + m) * (g.ropeDims >> 1);
@@ -361,10 +362,10 @@ __device__ __forceinline__ void gemm_store4(const Gemm& g, int m, int n, float4 
             }
         }
     }
-    if (g.mode == GEMM_ACT || g.mode == GEMM_ROPE) {
-        if (g.mode == GEMM_ACT && g.act.kind)
+    if (MODE == GEMM_ACT || MODE == GEMM_ROPE) {
+        if (MODE == GEMM_ACT)
 #pragma unroll
-            for (int i = 0; i < 4; i++) e[i] = apply_act(e[i], g.act);
+            for (int i = 0; i < 4; i++) e[i] = apply_act(e[i], act);
         AT* o = static_cast<AT*>(g.outAct) + (size_t)m * g.ldo + n;
         if (left >= 4) {
             if (sizeof(AT) == 2) *reinterpret_cast<uint2*>(o) = make_uint2(bf16_pack(e[0], e[1]), bf16_pack(e[2], e[3]));
@@ -377,10 +378,10 @@ __device__ __forceinline__ void gemm_store4(const Gemm& g, int m, int n, float4 
         return;
     }
     float* o = g.out + (size_t)m * g.ldc + n;
-    const float* r = g.mode == GEMM_RESID ? g.res + (size_t)m * g.ldres + n : nullptr;
-    const float sc = g.mode == GEMM_SCATTER ? g.rowScale[m] : 1.0f;
-    if (left >= 4 && ((g.ldc | g.ldres) & 3) == 0) {
-        if (r) {
+    const float* r = MODE == GEMM_RESID ? g.res + (size_t)m * g.ldres + n : nullptr;
+    const float sc = MODE == GEMM_SCATTER ? g.rowScale[m] : 1.0f;
+    if (left >= 4 && ((g.ldc | (MODE == GEMM_RESID ? g.ldres : 0)) & 3) == 0) {
+        if (MODE == GEMM_RESID) {
             const float4 x = *reinterpret_cast<const float4*>(r);
             e[0] = fmaf(g.alpha, x.x, e[0]); e[1] = fmaf(g.alpha, x.y, e[1]);
             e[2] = fmaf(g.alpha, x.z, e[2]); e[3] = fmaf(g.alpha, x.w, e[3]);
@@ -389,7 +390,42 @@ __device__ __forceinline__ void gemm_store4(const Gemm& g, int m, int n, float4 
     } else {
 #pragma unroll
         for (int i = 0; i < 4; i++)
-            if (i < left) o[i] = (r ? fmaf(g.alpha, r[i], e[i]) : e[i]) * sc;
+            if (i < left) o[i] = (MODE == GEMM_RESID ? fmaf(g.alpha, r[i], e[i]) : e[i]) * sc;
+    }
+}
+// A wave's blocks: acc[a][b] is columns n0 + 32 a .., rows r0 + 32 b ..; lane: row r0 + 32 b + lane % 32, columns
+// 8 q + 4 (lane / 32) + 0..3 of a 32-column block.
+template <typename AT, int MODE, int ACT, int WN, int WM, typename ACC>
+__device__ __forceinline__ void gemm_store(const Gemm& g, int row0, int rows, int r0, int n0, const ACC (&acc)[WN][WM]) {
+    const int fr = threadIdx.x & 31, fh = (threadIdx.x >> 5) & 1;
+#pragma unroll
+    for (int b = 0; b < WM; b++) {
+        const int r = r0 + 32 * b + fr;
+        if (r >= rows) continue;
+        const int m = MODE == GEMM_SCATTER ? g.perm[row0 + r] : row0 + r;
+#pragma unroll
+        for (int a = 0; a < WN; a++)
+#pragma unroll
+            for (int q = 0; q < 4; q++) {
+                const int n = n0 + 32 * a + 8 * q + 4 * fh;
+                if (n < g.N)
+                    gemm_store4<AT, MODE, ACT>(g, m, n, make_float4(acc[a][b][4 * q], acc[a][b][4 * q + 1], acc[a][b][4 * q + 2], acc[a][b][4 * q + 3]));
+            }
+    }
+}
+// One choice a workgroup, not one a value.
+template <typename AT, int WN, int WM, typename ACC>
+__device__ __forceinline__ void gemm_epilogue(const Gemm& g, int row0, int rows, int r0, int n0, const ACC (&acc)[WN][WM]) {
+    switch (g.mode) {
+    case GEMM_F32: gemm_store<AT, GEMM_F32, ACT_NONE>(g, row0, rows, r0, n0, acc); break;
+    case GEMM_RESID: gemm_store<AT, GEMM_RESID, ACT_NONE>(g, row0, rows, r0, n0, acc); break;
+    case GEMM_SPLIT: gemm_store<AT, GEMM_SPLIT, ACT_GELU>(g, row0, rows, r0, n0, acc); break;
+    case GEMM_ROPE: gemm_store<AT, GEMM_ROPE, ACT_NONE>(g, row0, rows, r0, n0, acc); break;
+    case GEMM_SCATTER: gemm_store<AT, GEMM_SCATTER, ACT_NONE>(g, row0, rows, r0, n0, acc); break;
+    default:
+        if (g.act.kind == ACT_GELU) gemm_store<AT, GEMM_ACT, ACT_GELU>(g, row0, rows, r0, n0, acc);
+        else if (g.act.kind == ACT_XIELU) gemm_store<AT, GEMM_ACT, ACT_XIELU>(g, row0, rows, r0, n0, acc);
+        else gemm_store<AT, GEMM_ACT, ACT_NONE>(g, row0, rows, r0, n0, acc);
     }
 }
 
@@ -420,15 +456,15 @@ __device__ __forceinline__ bool find_tile(const Gemm& g, TileAt& t) {
     return true;
 }
 
-// bf16 activations.  BM rows x BN columns, 4 waves (MW along the rows), K in steps of 64 through a ring of ST LDS buffers
+// bf16 activations.  BM rows x BN columns, NWV waves (MW along the rows), K in steps of 64 through a ring of ST LDS buffers
 // filled by direct global -> LDS loads, ST - 1 steps ahead.  LDS rows are 128 bytes (64 k); the 16-byte piece q of row r
 // lies at q ^ (r & 7).
-template <int BM, int BN, int MW, int ST>
-__global__ __launch_bounds__(256) void gemm_bf16_kernel(Gemm g) {
-    constexpr int NW = 4 / MW;
+template <int BM, int BN, int NWV, int MW, int ST>
+__global__ __launch_bounds__(64 * NWV) void gemm_bf16_kernel(Gemm g) {
+    constexpr int NW = NWV / MW;
     constexpr int WM = BM / (32 * MW), WN = BN / (32 * NW);     // 32 x 32 blocks a wave: rows, columns
     constexpr int ABYTES = BM * 128, BUF = (BM + BN) * 128;
-    constexpr int LOADS = (BM + BN) / 32;                // wave-loads (8 rows of 128 bytes) a wave issues a step
+    constexpr int LOADS = (BM + BN) / (8 * NWV);         // wave-loads (8 rows of 128 bytes) a wave issues a step
     extern __shared__ __attribute__((aligned(16))) unsigned char lds[];
     TileAt tl;
     if (!find_tile<BM, BN>(g, tl)) return;
@@ -478,41 +514,31 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(Gemm g) {
         if (st + ST - 1 < steps) issue(st + ST - 1, buf == 0 ? ST - 1 : buf - 1);
         const unsigned char* base = lds + buf * BUF;
         buf = buf == ST - 1 ? 0 : buf + 1;
+        // all fragments of the step are requested before the first product, which then waits for its own only
+        bf16x8 fa[4][WM], fw[4][WN];
 #pragma unroll
         for (int ks = 0; ks < 4; ks++) {
             const int piece = 2 * ks + fh;
-            bf16x8 fa[WM], fw[WN];
 #pragma unroll
             for (int b = 0; b < WM; b++) {
                 const int r = wm + 32 * b + fr;
-                fa[b] = *reinterpret_cast<const bf16x8*>(base + r * 128 + ((piece ^ (r & 7)) << 4));
+                fa[ks][b] = *reinterpret_cast<const bf16x8*>(base + r * 128 + ((piece ^ (r & 7)) << 4));
             }
 #pragma unroll
             for (int a = 0; a < WN; a++) {
                 const int r = wn + 32 * a + fr;
-                fw[a] = *reinterpret_cast<const bf16x8*>(base + ABYTES + r * 128 + ((piece ^ (r & 7)) << 4));
+                fw[ks][a] = *reinterpret_cast<const bf16x8*>(base + ABYTES + r * 128 + ((piece ^ (r & 7)) << 4));
             }
+        }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int ks = 0; ks < 4; ks++)
 #pragma unroll
             for (int a = 0; a < WN; a++)
 #pragma unroll
-                for (int b = 0; b < WM; b++) acc[a][b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fw[a], fa[b], acc[a][b], 0, 0, 0);
-        }
+                for (int b = 0; b < WM; b++) acc[a][b] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(fw[ks][a], fa[ks][b], acc[a][b], 0, 0, 0);
     }
-    // lane: row m = wm + 32 b + lane % 32; columns n = 8 q + 4 (lane / 32) + 0..3 of the 32-column block
-#pragma unroll
-    for (int b = 0; b < WM; b++) {
-        const int r = wm + 32 * b + fr;
-        if (r >= tl.rows) continue;
-        const int sr = tl.row0 + r;
-        const int m = g.mode == GEMM_SCATTER ? g.perm[sr] : sr;
-#pragma unroll
-        for (int a = 0; a < WN; a++)
-#pragma unroll
-            for (int q = 0; q < 4; q++) {
-                const int n = tl.n0 + wn + 32 * a + 8 * q + 4 * fh;
-                if (n < g.N) gemm_store4<bf16_t>(g, m, n, make_float4(acc[a][b][4 * q], acc[a][b][4 * q + 1], acc[a][b][4 * q + 2], acc[a][b][4 * q + 3]));
-            }
-    }
+    gemm_epilogue<bf16_t, WN, WM>(g, tl.row0, tl.rows, wm, tl.n0 + wn, acc);
 }
 
 // fp32 activations: 64 x 64, 4 waves as 2 x 2 of one 32 x 32 block, K in steps of 32.
@@ -531,9 +557,9 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(Gemm g) {
     const int sr = tl.row0 + min(lr, tl.rows - 1);
     const float* ap = A + (size_t)(g.permDiv ? g.perm[sr] / g.permDiv : sr) * g.lda + lk;
     const WT* wp = W + (size_t)min(tl.n0 + lr, g.N - 1) * g.ldw + lk;
-    f32x16 acc;
+    f32x16 acc[1][1];
 #pragma unroll
-    for (int e = 0; e < 16; e++) acc[e] = 0.f;
+    for (int e = 0; e < 16; e++) acc[0][0][e] = 0.f;
     const int wm = (wave & 1) * 32, wn = (wave >> 1) * 32, fr = lane & 31, fh = lane >> 5;
     for (int k0 = 0; k0 < g.K; k0 += 32) {
         const float4 a0 = *reinterpret_cast<const float4*>(ap + k0), a1 = *reinterpret_cast<const float4*>(ap + k0 + 4);
@@ -555,48 +581,57 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(Gemm g) {
         __syncthreads();
 #pragma unroll
         for (int k = 0; k < 32; k += 2)
-            acc = __builtin_amdgcn_mfma_f32_32x32x2f32(Ws[(wn + fr) * LDT + k + fh], As[(wm + fr) * LDT + k + fh], acc, 0, 0, 0);
+            acc[0][0] = __builtin_amdgcn_mfma_f32_32x32x2f32(Ws[(wn + fr) * LDT + k + fh], As[(wm + fr) * LDT + k + fh], acc[0][0], 0, 0, 0);
     }
-    const int r = wm + fr;
-    if (r >= tl.rows) return;
-    const int s2 = tl.row0 + r;
-    const int m = g.mode == GEMM_SCATTER ? g.perm[s2] : s2;
-#pragma unroll
-    for (int q = 0; q < 4; q++) {
-        const int n = tl.n0 + wn + 8 * q + 4 * fh;
-        if (n < g.N) gemm_store4<float>(g, m, n, make_float4(acc[4 * q], acc[4 * q + 1], acc[4 * q + 2], acc[4 * q + 3]));
-    }
+    gemm_epilogue<float, 1, 1>(g, tl.row0, tl.rows, wm, tl.n0 + wn, acc);
 }
 
-template <int BM, int BN, int MW, int ST>
+template <int BM, int BN, int NWV, int MW, int ST>
 static hipError_t run_gemm_bf16(const Gemm& g, hipStream_t s) {
     const size_t lds = (size_t)(BM + BN) * 128 * ST;
-    auto k = gemm_bf16_kernel<BM, BN, MW, ST>;
+    auto k = gemm_bf16_kernel<BM, BN, NWV, MW, ST>;
     if (lds > (48u << 10)) {
         hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
     const int tilesN = (g.N + BN - 1) / BN;
     const int tilesM = g.tiles ? g.maxTiles : (g.M + BM - 1) / BM;
-    hipLaunchKernelGGL(k, dim3((unsigned)(tilesN * tilesM)), dim3(256), lds, s, g);
+    hipLaunchKernelGGL(k, dim3((unsigned)(tilesN * tilesM)), dim3(64 * NWV), lds, s, g);
     return hipGetLastError();
 }
 
 hipError_t launch_gemm_bf16w(const Gemm& g, hipStream_t s) {
     if (g.M <= 0 || g.N <= 0) return hipSuccess;
     if (g.K <= 0 || g.K % 64 || g.lda < g.K || g.ldw < g.K || g.lda % 8 || g.ldw % 8) return hipErrorInvalidValue;
+    if (g.mode == GEMM_SPLIT && g.nSplit < g.N && g.act.kind != ACT_GELU) return hipErrorInvalidValue;
     if (g.f32) {
         const unsigned grid = (unsigned)((g.N + 63) / 64) * (unsigned)(g.tiles ? g.maxTiles : (g.M + 63) / 64);
+        if (g.tiles && g.tileRows != 64) return hipErrorInvalidValue;
         if (g.wF32) hipLaunchKernelGGL(gemm_f32_kernel<float>, dim3(grid), dim3(256), 0, s, g);
         else hipLaunchKernelGGL(gemm_f32_kernel<bf16_t>, dim3(grid), dim3(256), 0, s, g);
         return hipGetLastError();
     }
     if (g.wF32) return hipErrorInvalidValue;
-    if (g.tiles) return g.N >= 512 ? run_gemm_bf16<MOE_TILE_ROWS, 256, 1, 2>(g, s) : run_gemm_bf16<MOE_TILE_ROWS, 64, 2, 3>(g, s);
-    const long big = (long)((g.M + 127) / 128) * ((g.N + 127) / 128);
-    if (big > 320) return run_gemm_bf16<128, 128, 2, 2>(g, s);       // two workgroups a CU cover each other's waits
-    if (big >= 160) return run_gemm_bf16<128, 128, 2, 4>(g, s);      // about one a CU: loads three steps ahead instead
-    return run_gemm_bf16<64, 64, 2, 4>(g, s);
+    if (g.tiles) {
+        if (g.tileRows == 128) return g.N > 128 ? run_gemm_bf16<128, 256, 8, 2, 3>(g, s) : run_gemm_bf16<128, 128, 4, 2, 2>(g, s);
+        if (g.tileRows != 64) return hipErrorInvalidValue;
+        return g.N > 128 ? run_gemm_bf16<64, 256, 4, 1, 3>(g, s) : run_gemm_bf16<64, 64, 4, 2, 4>(g, s);
+    }
+    // The tile whose rounds over the 256 CUs take least: microseconds a step of 64 k and around the loop, as measured.
+    const double steps = g.K / 64.0;
+    auto cost = [&](int bm, int bn, int atOnce, double step, double rest) {
+        const long tiles = (long)((g.M + bm - 1) / bm) * ((g.N + bn - 1) / bn);
+        return (double)((tiles + atOnce - 1) / atOnce) * (steps * step + rest);
+    };
+    const double c[5] = {cost(256, 256, 256, 1.53, 18), cost(128, 256, 256, 0.88, 10), cost(128, 128, 256, 0.625, 7.5),
+                         cost(128, 128, 512, 0.85, 6.8), cost(64, 64, 512, 0.37, 2.5)};
+    switch ((int)(std::min_element(c, c + 5) - c)) {
+    case 0: return run_gemm_bf16<256, 256, 8, 2, 2>(g, s);
+    case 1: return run_gemm_bf16<128, 256, 8, 2, 3>(g, s);
+    case 2: return run_gemm_bf16<128, 128, 4, 2, 4>(g, s);
+    case 3: return run_gemm_bf16<128, 128, 4, 2, 2>(g, s);
+    default: return run_gemm_bf16<64, 64, 4, 2, 4>(g, s);
+    }
 }
 
 }  // namespace mg

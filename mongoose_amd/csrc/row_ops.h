@@ -86,6 +86,7 @@ struct MoeRoute {
     int* perm = nullptr;
     int4* tiles = nullptr;
     int* nTiles = nullptr;
+    int tileRows = 64;
 };
 inline int moe_max_tiles(int T, int top, int experts, int tileRows) {
     const long e = (long)T * top;

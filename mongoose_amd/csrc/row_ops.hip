@@ -92,9 +92,9 @@ __global__ void route_tiles_kernel(MoeRoute p) {
     // thread e: start = entries of the experts before it, first tile = their tiles
     for (int e = threadIdx.x; e < p.experts; e += blockDim.x) {
         int start = 0, tile = 0;
-        for (int k = 0; k < e; k++) { start += cnt[k]; tile += (cnt[k] + MOE_TILE_ROWS - 1) / MOE_TILE_ROWS; }
+        for (int k = 0; k < e; k++) { start += cnt[k]; tile += (cnt[k] + p.tileRows - 1) / p.tileRows; }
         p.work[p.experts + e] = start;
-        for (int r = 0; r < cnt[e]; r += MOE_TILE_ROWS) p.tiles[tile++] = make_int4(e, start + r, min(MOE_TILE_ROWS, cnt[e] - r), 0);
+        for (int r = 0; r < cnt[e]; r += p.tileRows) p.tiles[tile++] = make_int4(e, start + r, min(p.tileRows, cnt[e] - r), 0);
         if (e == p.experts - 1) *p.nTiles = tile;
     }
 }
