@@ -148,20 +148,24 @@ __global__ __launch_bounds__(WG) void moe_down_kernel(MvMoeDown p) {
     __shared__ float wts[MAX_TOP];
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int Kp = p.down.ld, Ks = p.downShared.rows ? p.downShared.ld : 0;
-    const int row = min((int)blockIdx.x * 4 + wave, p.down.rows - 1);
+    int row = blockIdx.x * 4 + wave;                                  // then every gridDim.x * 4th
+    const int stride = gridDim.x * 4, last = p.down.rows - 1;
     const int ncE = (Kp + 511) >> 9, ncS = (Ks + 511) >> 9, total = p.top * ncE + ncS;
-    const float res = p.resid[row];
+    float res = p.resid[min(row, last)];
     if (wave == 0) choose_experts(p.routerLogits, p.experts, p.top, ids, wts);
     __syncthreads();
     uint4 ring[DEP];
-    int ls = 0, lc = 0;                                               // load cursor: segment (top = the shared expert), chunk
+    int lr = row, ls = 0, lc = 0;                                     // load cursor: row, segment (top = the shared expert), chunk
+    const int segs = p.top + (Ks ? 1 : 0);
     auto issue = [&](uint4& slot) __attribute__((always_inline)) {
         const bool sh = ls == p.top;
         const int ld = sh ? Ks : Kp, col = lc * 512 + lane * 8;
-        const unsigned short* w = sh ? p.downShared.w + (size_t)row * Ks
-                                     : p.down.w + (size_t)ids[min(ls, p.top - 1)] * p.expertStride + (size_t)row * Kp;
-        slot = ls <= p.top && col < ld ? *reinterpret_cast<const uint4*>(w + col) : make_uint4(0, 0, 0, 0);
-        if (++lc >= (sh ? ncS : ncE)) { lc = 0; ls++; }
+        const unsigned short* w = sh ? p.downShared.w : p.down.w + (size_t)ids[min(ls, p.top - 1)] * p.expertStride;
+        slot = lr <= last && col < ld ? *reinterpret_cast<const uint4*>(w + (size_t)lr * ld + col) : make_uint4(0, 0, 0, 0);
+        if (++lc >= (sh ? ncS : ncE)) {
+            lc = 0;
+            if (++ls == segs) { ls = 0; lr += stride; }
+        }
     };
 #pragma unroll
     for (int d = 0; d < DEP; d++) issue(ring[d]);
@@ -192,21 +196,26 @@ __global__ __launch_bounds__(WG) void moe_down_kernel(MvMoeDown p) {
     __syncthreads();
     float acc = 0.f;
     int us = 0, uc = 0, n = 0;
-    while (n < total) {
+    while (row <= last) {
 #pragma unroll
         for (int d = 0; d < DEP; d++) {
-            if (n >= total) break;
+            if (row > last) break;
             const bool sh = us == p.top;
             const int nc8 = (sh ? Ks : Kp) >> 3;
             const float4* lo = reinterpret_cast<const float4*>(act + us * Kp);
             acc = dot8(ring[d], lo, lo + nc8, min(uc * 64 + lane, nc8 - 1), acc);
             issue(ring[d]);
             if (++uc == (sh ? ncS : ncE)) { uc = 0; us++; }
-            n++;
+            if (++n == total) {
+                acc = wave_sum(acc);
+                if (lane == 0) p.out[row] = fmaf(p.alpha, res, acc);
+                acc = 0.f;
+                us = uc = n = 0;
+                row += stride;
+                res = p.resid[min(row, last)];
+            }
         }
     }
-    acc = wave_sum(acc);
-    if (lane == 0 && (int)blockIdx.x * 4 + wave < p.down.rows) p.out[row] = fmaf(p.alpha, res, acc);
 }
 hipError_t launch_moe_down(const MvMoeDown& p, hipStream_t s) {
     if (p.top < 1 || p.top > MAX_TOP || p.experts > MAX_EXPERTS || p.down.ld % 64 || p.ldHid < p.down.ld) return hipErrorInvalidValue;
@@ -216,7 +225,10 @@ hipError_t launch_moe_down(const MvMoeDown& p, hipStream_t s) {
         hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(moe_down_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL(moe_down_kernel, dim3((p.down.rows + 3) / 4), dim3(WG), lds, s, p);
+    // all workgroups resident at once, with equal numbers of rows a wave
+    const int most = 256 * std::max(1, std::min(4, (int)((160u << 10) / (lds + 512))));
+    const int rounds = (p.down.rows + 4 * most - 1) / (4 * most);
+    hipLaunchKernelGGL(moe_down_kernel, dim3((p.down.rows + 4 * rounds - 1) / (4 * rounds)), dim3(WG), lds, s, p);
     return hipGetLastError();
 }
 
@@ -231,6 +243,14 @@ __global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG
         return;
     }
     const int ld = p.ld, nc8 = ld >> 3;
+    const int lpr = 1 << lprLog2, sub = threadIdx.x & (lpr - 1), slot = threadIdx.x >> lprLog2, slots = WG >> lprLog2;
+    const int r0 = blockIdx.x * rowsPerWG, r1 = min(r0 + rowsPerWG, p.rows);
+    // the first chunk of this thread's first rows, requested before the input is there
+    constexpr int AHEAD = 4;
+    uint4 pre[AHEAD];
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++)
+        pre[i] = *reinterpret_cast<const uint4*>(p.w + ((size_t)h * p.rows + min(r0 + i * slots + slot, p.rows - 1)) * ld + min(sub, nc8 - 1) * 8);
     if (p.splits) {
         // out = sum_s e^(m_s - M) acc_s / sum_s e^(m_s - M) l_s; a split that saw no key has m = -inf.  A thread takes
         // four consecutive elements of every gs-th split.
@@ -276,16 +296,7 @@ __global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG
     __syncthreads();
     const float4* lo = reinterpret_cast<const float4*>(act);
     const float4* hi = lo + nc8;
-    const int lpr = 1 << lprLog2, sub = threadIdx.x & (lpr - 1), slot = threadIdx.x >> lprLog2, slots = WG >> lprLog2;
-    const int r0 = blockIdx.x * rowsPerWG, r1 = min(r0 + rowsPerWG, p.rows);
-    for (int rb = r0; rb < r1; rb += slots) {
-        const int row = rb + slot;
-        float acc = 0.f;
-        if (row < r1) {
-            const unsigned short* w = p.w + ((size_t)h * p.rows + row) * ld;
-#pragma unroll 2
-            for (int c8 = sub; c8 < nc8; c8 += lpr) acc = dot8(*reinterpret_cast<const uint4*>(w + c8 * 8), lo, hi, c8, acc);
-        }
+    auto finish = [&](int row, float acc) __attribute__((always_inline)) {
         for (int o = lpr >> 1; o > 0; o >>= 1) acc += __shfl_xor(acc, o, 64);
         if (sub == 0 && row < r1) {
             if (p.out) p.out[((size_t)t * p.heads + h) * p.ldOut + row] = acc;
@@ -295,6 +306,24 @@ __global__ __launch_bounds__(WG) void head_matvec_kernel(HeadMv p, int rowsPerWG
                 else store_act(static_cast<bf16_t*>(p.outAct) + o, acc);
             }
         }
+    };
+    auto rest = [&](int row, int c0, float acc) __attribute__((always_inline)) {
+        const unsigned short* w = p.w + ((size_t)h * p.rows + row) * ld;
+#pragma unroll 2
+        for (int c8 = c0; c8 < nc8; c8 += lpr) acc = dot8(*reinterpret_cast<const uint4*>(w + c8 * 8), lo, hi, c8, acc);
+        return acc;
+    };
+#pragma unroll
+    for (int i = 0; i < AHEAD; i++) {
+        if (r0 + i * slots >= r1) break;
+        const int row = r0 + i * slots + slot;
+        float acc = sub < nc8 ? dot8(pre[i], lo, hi, sub, 0.f) : 0.f;
+        if (row < r1) acc = rest(row, sub + lpr, acc);
+        finish(row, acc);
+    }
+    for (int rb = r0 + AHEAD * slots; rb < r1; rb += slots) {
+        const int row = rb + slot;
+        finish(row, row < r1 ? rest(row, sub, 0.f) : 0.f);
     }
 }
 hipError_t launch_head_matvec(const HeadMv& p, hipStream_t s) {
