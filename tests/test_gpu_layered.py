@@ -73,6 +73,25 @@ def all_experts(layers):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("width, vocab", [(70, 37), (65, 1), (130, 131), (320, 257), (1100, 70)])
+def test_other_widths(hip, dtype, width, vocab):
+    """Widths and vocabularies that are no multiple of anything the kernels work in."""
+    layers = [with_ff(M.latent(window=11, heads=2), C.dense_ff(width // 2 + 1)), with_ff(M.delta(), C.moe_ff(9, 3, 3, 5)),
+              M.latent(kv_from=0, window=23, heads=3, vdim=20, q_rank=31)]
+    p = M.Pair(M.model(layers, width=width, vocab=vocab, alpha=3.1, eps=1e-3), seed=8, eng=hip, dtype=dtype, maxSeq=128)
+    toks = p.tokens(90)
+    want = p.oracle_logits(toks)
+    for sizes in ([90], [1], [50, 2]):
+        got = M.run_portions(p.hip, toks, sizes)
+        if vocab == 1:
+            assert np.abs(got - want).max() < TOL[dtype] * np.abs(want).max()
+            continue
+        e = M.errors(got, want)
+        assert e.max() < TOL[dtype], (sizes, int(e.argmax()), float(e.max()))
+    p.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("w0, ab", [(9.0, 9.0), (-9.0, 9.0), (9.0, -9.0), (-9.0, -9.0)])
 def test_delta_rule_at_the_ends_of_its_gates(hip, dtype, w0, ab):
     """Fastest and slowest decay, full and no removal, over several chunks of the many-row form and a ragged end."""
@@ -242,6 +261,26 @@ def test_needle_far_away_without_a_window(hip, dtype):
     for sizes in ([1200], [700, 2], [1100] + [1] * 100):
         e = M.errors(M.run_portions(p.hip, toks, sizes), want)
         assert e.max() < TOL[dtype], (sizes, int(e.argmax()), float(e.max()))
+    p.close()
+
+
+def test_large_tiles_agree_with_small_ones(hip):
+    """Sizes at which a long prompt takes the large tiles of the matrix products and of the experts: one pass against
+    portions of 64 tokens, whose products take the small tiles, and the first tokens against the oracle."""
+    layers = [with_ff(M.latent(heads=8, dim=128, rot_dim=64, vdim=128, kv_rank=256, q_rank=512, scale=0.07, window=700), C.dense_ff(5632)),
+              with_ff(M.delta(heads=32, dim=64, decay_rank=64), C.moe_ff(512, 3, 3, 256)),
+              with_ff(M.latent(heads=4, dim=128, rot_dim=64, vdim=128, kv_rank=256, q_rank=512, scale=0.07, window=0, kv_from=0), C.dense_ff(4096))]
+    p = M.Pair(M.model(layers, width=2048, vocab=300, alpha=2.2), seed=17, eng=hip, dtype="bfloat16", maxSeq=2100)
+    toks = p.tokens(2050)
+    assert p.hip.ResetKV() == 0
+    rows = list(range(0, 2050, 7)) + list(range(1980, 2050))
+    rc, one = p.hip.PrefillLogits(toks, 0, rows)
+    assert rc == 0, E.last_error()
+    small = M.run_portions(p.hip, toks, [64])
+    e = M.errors(one, small[rows].astype(np.float64))
+    assert e.max() < 0.02, (rows[int(e.argmax())], float(e.max()))
+    e = M.errors(small[:12], p.oracle_logits(toks[:12]))
+    assert e.max() < TOL["bfloat16"], float(e.max())
     p.close()
 
 

@@ -219,3 +219,22 @@ def test_prefill_q4_0_short_prompt_and_k_tail(hip):
     s = configs.TOY._replace(fmt="q4_0", name="toy-q4")
     m, _, _ = _prefill_case(hip, s, seed=6, nPrompt=40, nDecode=6, maxSeq=64)
     m.close()
+
+
+def test_prefill_logits_of_chosen_rows(hip):
+    """mg_prefill_logits on the quantized model class: rows in any order, against the decode step at those positions."""
+    s = H.with_layers(configs.TOY, 2)
+    m = H.Model(s, seed=31, maxSeq=64, eng=hip, oracle=False)
+    toks = m.prompt(40)
+    want = np.empty((40, s.vocab), np.float32)
+    for pos in range(40):
+        rc, _ = m.hip.DecodeToken(int(toks[pos]), pos, want[pos])
+        assert rc == 0, E.last_error()
+    assert m.hip.ResetKV() == 0
+    rc, got = m.hip.PrefillLogits(toks[:30], 0, [29, 0, 7])
+    assert rc == 0, E.last_error()
+    assert H.rel_err(got, want[[29, 0, 7]]) < 1e-3
+    rc, got = m.hip.PrefillLogits(toks[30:], 30, [0, 9])
+    assert rc == 0 and H.rel_err(got, want[[30, 39]]) < 1e-3
+    assert m.hip.PrefillLogits(toks[:3], 0, [3])[0] == -2
+    m.close()

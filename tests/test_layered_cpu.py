@@ -1,0 +1,156 @@
+"""The oracle of layer-list models against closed forms, and the readers of model folders (no GPU needed)."""
+import json
+import math
+
+import numpy as np
+import pytest
+
+from mongoose_amd import configs as C
+from mongoose_amd import loader
+from oracle import layered as O
+from tests import layered_models as M
+
+rng = np.random.default_rng(4)
+
+
+def test_norm_and_activations():
+    x = rng.standard_normal(7)
+    y = O.rms_norm(x, 0.0)
+    assert abs(np.mean(y * y) - 1) < 1e-12
+    assert np.allclose(O.rms_norm(x, 1e30) * 1e15, x)             # eps sits inside the root
+    assert abs(O.gelu_erf(np.array([1.0]))[0] - 0.841344746068543) < 1e-12
+    # xIELU: continuous with slope 1/2 at zero, the two parameters act on their own sides
+    for p, q in ((0.3, -0.8), (-2.0, 4.0)):
+        e = 1e-6
+        lo, hi = O.xielu(np.array([-e]), p, q)[0], O.xielu(np.array([e]), p, q)[0]
+        assert abs(lo + e / 2) < 1e-10 and abs(hi - e / 2) < 1e-10
+        assert abs(O.xielu(np.array([2.0]), p, q)[0] - (math.log1p(math.exp(p)) * 4 + 1)) < 1e-12
+        assert abs(O.xielu(np.array([-1.0]), p, q)[0] - ((0.5 + math.log1p(math.exp(q))) * math.exp(-1) - 0.5)) < 1e-12
+
+
+def test_rotation_is_interleaved_and_relative():
+    v = np.zeros(6)
+    v[2] = 1.0
+    r = O.rotate(v, 3, 100.0, 4)                                   # pair 1 of 2: frequency 100^(-1/2)
+    assert np.allclose(r, [0, 0, math.cos(0.3), math.sin(0.3), 0, 0])
+    assert np.allclose(O.rotate(np.arange(6.0), 9, 100.0, 4)[4:], [4, 5])
+    q, k = rng.standard_normal(8), rng.standard_normal(8)
+    dots = [O.rotate(q, p + 5, 50.0, 8) @ O.rotate(k, p, 50.0, 8) for p in (0, 3, 77)]
+    assert np.ptp(dots) < 1e-12
+
+
+def test_routing_scores_and_ties():
+    ids, w = O.route(np.array([1.0, 3.0, 3.0, 0.0]), 2)
+    assert ids == [1, 2] and abs(w[0] - w[1]) < 1e-15
+    s = np.exp([1, 3, 3, 0])
+    assert np.allclose(w, s[1] / s.sum())                          # softmax over all, not renormalised
+
+
+def test_delta_update_closed_forms():
+    D = 5
+    S = rng.standard_normal((D, D))
+    k, v = rng.standard_normal(D), rng.standard_normal(D)
+    u = k / np.linalg.norm(k)
+    one, zero = np.ones(D), np.zeros(D)
+    assert np.allclose(O.delta_update(S, one, zero, u, k, v), S + np.outer(k, v))      # no decay, no removal
+    T = O.delta_update(S, one, one, u, k, v)
+    assert np.allclose(T.T @ u, np.linalg.norm(k) * v)             # full removal: the key's slot now holds its value only
+    w = rng.uniform(0.5, 1, D)
+    assert np.allclose(O.delta_update(S, w, zero, u, zero, v), w[:, None] * S)
+
+
+def test_attention_sees_exactly_its_window():
+    s = M.model([M.latent(window=6)])
+    p = M.Pair(s, seed=2)
+    toks = p.tokens(20)
+    base = p.oracle_logits(toks)
+    for j in (0, 4, 9):
+        t2 = toks.copy()
+        t2[j] = (t2[j] + 1) % s.vocab
+        changed = np.abs(p.oracle_logits(t2) - base).max(axis=1) > 1e-9
+        assert np.array_equal(np.flatnonzero(changed), np.arange(j, min(j + 6, 20)))
+
+
+def test_a_shared_cache_is_the_other_layers():
+    s = M.model([M.latent(), M.latent(window=3, kv_from=0)])
+    names = M.tensor_shapes(s)
+    assert "l0.mix.dkv" in names and "l1.mix.dkv" not in names
+    p = M.Pair(s, seed=2)
+    p.oracle_logits(p.tokens(5))
+    assert len(p.orc.C[0]) == 5 and len(p.orc.C[1]) == 0
+
+
+def test_depth_average_of_the_last_output_only_is_a_plain_stack():
+    s = M.model([M.delta(), M.delta()])
+    p = M.Pair(s, tweak={f"l{i}.dwa": lambda a: np.eye(1, len(a), len(a) - 1)[0] for i in range(2)})
+    p.orc.reset()
+    x = p.values["embed"][3]
+    p.orc.step(3)
+    for i in range(2):
+        S = np.zeros((3, 24, 24))
+        y = O.general_delta(p.orc.m["layers"][i]["mixer"], p.values, f"l{i}.mix.", x, s.eps, S)
+        x = O.rms_norm(s.alpha * x + y, s.eps, p.values[f"l{i}.norm1"])
+        assert np.allclose(p.orc.trail[i], x)
+
+
+LAYERS = [{**M.latent(window=7), **C.dense_ff(20)}, {**M.delta(), **C.moe_ff(16, 5, 2, 12)},
+          {**M.latent(kv_from=0, window=9, heads=2), **C.moe_ff(16, 3, 1)}, M.delta(decay_rank=4)]
+
+
+def test_config_reader_round_trip():
+    s = M.model(LAYERS)
+    shapes = M.tensor_shapes(s)
+    got = C.ARCHITECTURES["Vadonex"](json.loads(json.dumps(M.vadonex_config(s))), shapes.__getitem__)
+    assert got._replace(name=s.name) == s
+    bad = M.vadonex_config(s)
+    bad["layers"][1]["type"] = "something"
+    with pytest.raises(ValueError, match="layer 1"):
+        C.read_vadonex(bad, shapes.__getitem__)
+
+
+def test_model_folder(tmp_path):
+    s = M.model(LAYERS)
+    bits = M.random_bits(s, 3)
+    M.write_folder(str(tmp_path / "m"), s, bits, M.vadonex_config(s))
+    spec, weights = loader.read_model(str(tmp_path / "m"))
+    assert spec._replace(name=s.name) == s and set(weights.names()) == set(bits)
+    for name, b in bits.items():
+        assert weights.shape(name) == b.shape and np.array_equal(weights.array(name), b)
+    M.write_folder(str(tmp_path / "n"), s, bits, {**M.vadonex_config(s), "architecture": "Other"})
+    with pytest.raises(ValueError, match="Other"):
+        loader.read_model(str(tmp_path / "n"))
+    # a header whose offsets do not fit the shape is an error, not a read past the end
+    f = tmp_path / "bad.safetensors"
+    h = json.dumps({"t": {"dtype": "BF16", "shape": [4], "data_offsets": [0, 8]}}).encode()
+    f.write_bytes(len(h).to_bytes(8, "little") + h + b"\0" * 6)
+    with pytest.raises(ValueError):
+        loader.SafeTensors(str(f)).array("t")
+
+
+class FakeModel:
+    def __init__(self, shapes):
+        self.shapes, self.got = shapes, {}
+
+    def TensorNames(self):
+        return list(self.shapes)
+
+    def TensorShape(self, name):
+        return self.shapes.get(name)
+
+    def SetTensor(self, name, bits):
+        self.got[name] = bits
+        return 0
+
+
+def test_set_weights_checks_names_and_shapes(tmp_path):
+    s = M.model(LAYERS)
+    bits = M.random_bits(s, 3)
+    M.write_folder(str(tmp_path), s, bits, M.vadonex_config(s))
+    _, w = loader.read_model(str(tmp_path))
+    m = FakeModel(M.tensor_shapes(s))
+    loader.set_weights(m, w)
+    assert set(m.got) == set(bits)
+    with pytest.raises(ValueError, match="missing"):
+        loader.set_weights(FakeModel({**M.tensor_shapes(s), "more": (2,)}), w)
+    with pytest.raises(ValueError, match="head"):
+        loader.set_weights(FakeModel({**M.tensor_shapes(s), "head": (2, 2)}), w)
