@@ -15,7 +15,9 @@
  *   3. mg_*            fused-inference context: what CUDAFusedInference,
  *                      CUDAStreamInfer and CUDAGraph do behind their Go methods
  *                      (cuda_fused_infer.go, cuda_fused_infer_q4.go,
- *                       cuda_q4_0.go, cuda_fused_stream.go, cuda_graph.go)
+ *                       cuda_q4_0.go, cuda_fused_stream.go, cuda_graph.go),
+ *                      and, behind the same handle, models described by a list
+ *                      of layers (no counterpart in the reference)
  *
  * Error convention.  The reference's kernels return void and report nothing;
  * its Go methods return -1 when the object is not built.  Here mongoose_*
